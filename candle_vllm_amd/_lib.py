@@ -348,7 +348,8 @@ class HybridLayer(ctypes.Structure):
                 ("moe_experts", c_i32), ("moe_top", c_i32), ("moe_shared_ff", c_i32), ("moe_scale", c_f32),
                 ("moe_sigmoid", c_i32), ("moe_groups", c_i32), ("moe_keep_groups", c_i32), ("moe_normalise", c_i32),
                 ("d_norm_groups", c_i32), ("a_dist_bias", c_i32), ("a_q_rank", c_i32), ("a_out_gate", c_i32), ("kv_from", c_i32),
-                ("side_dim", c_i32), ("side_col", c_i32), ("depth_terms", c_i32)]
+                ("side_dim", c_i32), ("side_col", c_i32), ("depth_terms", c_i32),
+                ("a_mask_kind", c_i32), ("a_v_is_k", c_i32), ("moe_relu2", c_i32), ("moe_bias", c_i32), ("moe_shared_plain", c_i32)]
 
 
 class HybridConfig(ctypes.Structure):
@@ -356,7 +357,8 @@ class HybridConfig(ctypes.Structure):
     _fields_ = [("width", c_i32), ("vocab", c_i32), ("n_layers", c_i32), ("dtype", c_i32), ("block_size", c_i32),
                 ("state_slots", c_i32), ("norm_eps", c_f32), ("unit_eps", c_f32),
                 ("residual_form", c_i32), ("resid_alpha", c_f32), ("norm_groups", c_i32), ("logit_scale", c_f32),
-                ("norm_kind", c_i32), ("embed_scale", c_f32), ("logit_softcap", c_f32), ("tie_head", c_i32), ("side_cols", c_i32)]
+                ("norm_kind", c_i32), ("embed_scale", c_f32), ("logit_softcap", c_f32), ("tie_head", c_i32), ("side_cols", c_i32),
+                ("streams", c_i32), ("bigram_buckets", c_i32), ("bigram_mul_prev", c_i64), ("bigram_mul_cur", c_i64)]
 
 
 _sig("mi355_be_state_init", c_i32, [c_vp, c_i32])
@@ -368,6 +370,7 @@ _sig("mi355_hybrid_create", c_vp, [ctypes.POINTER(HybridConfig), ctypes.POINTER(
 _sig("mi355_hybrid_destroy", None, [c_vp])
 _sig("mi355_hybrid_in_proj_rows", c_i32, [ctypes.POINTER(HybridLayer), c_vp])
 _sig("mi355_hybrid_set_weight", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i64])
+_sig("mi355_hybrid_set_weight_f32", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i64])
 _sig("mi355_hybrid_set_weight_dev", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i64, c_i64])
 _sig("mi355_hybrid_set_rope_tables", ctypes.c_int, [c_vp, c_i32, c_vp, c_vp, c_i32])
 _sig("mi355_hybrid_alloc_cache", ctypes.c_int, [c_vp, c_i32])
@@ -440,6 +443,17 @@ _sig("mi355_hyb_biased_attention", ctypes.c_int, [c_vp, c_i32, c_i32, c_i32] + [
 _sig("mi355_hyb_latent_prepare_ex", ctypes.c_int, [c_vp, c_vp, c_vp, c_i32, c_i32, c_vp, c_i32, c_i32] + [c_vp] * 6 + [c_i32] * 7 + [c_f32, c_i32, c_i64])
 _sig("mi355_hyb_moe_route_ex", ctypes.c_int, [c_vp, c_vp, c_vp, c_vp, c_i32, c_vp, c_vp, c_vp, c_vp, c_vp, c_i32, c_i32, c_i32, c_i32, c_f32, c_f32,
                                                 c_i32, c_i32, c_i32, c_i32, c_i32, c_i64])
+_sig("mi355_hyb_linear_act", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i32, c_i32, c_vp, c_vp] + [c_i32] * 6 + [c_i64])
+_sig("mi355_hyb_linear_grouped_act", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i32, c_i32, c_vp, c_vp, c_i64, c_vp] + [c_i32] * 6 + [c_i64])
+_sig("mi355_hyb_attention", ctypes.c_int, [c_vp, c_i32, c_i32, c_i32] + [c_vp] * 9 + [c_i32] * 11 + [c_f32, c_f32, c_i32, c_i32, c_f32, c_i32, c_i32,
+                                                                                                       c_i64])
+_sig("mi355_hyb_moe_route_biased", ctypes.c_int, [c_vp, c_vp, c_vp, c_vp, c_i32] + [c_vp] * 6 + [c_i32] * 4 + [c_f32, c_f32] + [c_i32] * 5 + [c_i64])
+_sig("mi355_hyb_bigram_rows", ctypes.c_int, [c_vp, c_vp, c_i64, c_vp, c_vp, c_vp, c_vp, c_i32, c_i32, c_i32, c_i64, c_i64, c_i64])
+_sig("mi355_hyb_embed_streams", ctypes.c_int, [c_vp] * 5 + [c_i32] * 4 + [c_f32, c_i32, c_i64])
+_sig("mi355_hyb_stream_step", ctypes.c_int, [c_vp] * 5 + [c_i32] + [c_vp] * 6 + [c_i32, c_vp, c_i32, c_i32, c_i32, c_f32, c_i64])
+_sig("mi355_hyb_norm_sigmoid_gate", ctypes.c_int, [c_vp, c_i32, c_vp, c_vp, c_i32, c_vp, c_i32, c_i32, c_i32, c_f32, c_i64])
+_sig("mi355_hyb_decay_attention", ctypes.c_int, [c_vp, c_vp, c_i64, c_vp, c_i32, c_i32, c_i32, c_i32] + [c_vp] * 4 + [c_i32] * 5 + [c_vp, c_i64])
+_sig("mi355_hyb_decay_attention_scratch", c_i64, [c_i32] * 5)
 
 # the hand-written ctypes mirrors must have the layout the library was built with
 for _id, _cls in ((0, QmmDesc), (1, LlamaConfig), (2, DenseConfig), (3, RopeScaling), (4, HybridConfig), (5, HybridLayer)):

@@ -1,7 +1,7 @@
 // More kernels of the layer-list host layer (include/mi355_hybrid.h): the mechanisms of designs whose layers read ONE norm and add
 // mixer and feed-forward side by side -- layer norm, the state-space scan (scalar decay per head) with its gated group norm, the
-// per-layer token input, the weighted average over the depth of the stack, the experts' sum without a norm, and small elementwise
-// glue.  Numerics as in hybrid_kernels.hip: residual stream, norms, recurrent state and everything that enters the recurrence are f32.
+// per-layer token input, the weighted average over the depth of the stack, the experts' sum without a norm, linear attention with a
+// constant decay per head (the same scan, and a form by pieces on the f32 matrix cores), and small elementwise glue.  Numerics as in hybrid_kernels.hip: residual stream, norms, recurrent state and everything that enters the recurrence are f32.
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 #include <math.h>
@@ -11,8 +11,6 @@
 #include "../../include/mi355_hybrid.h"
 
 namespace {
-
-__device__ __forceinline__ float gelu_tanhf_(float z) { return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 
 template <typename TW> __global__ void embed_scaled_kernel(float* x, const TW* table, const uint32_t* ids, int width, int vocab, float scale) {
     const int t = blockIdx.x;
@@ -166,6 +164,8 @@ struct SsdArgs {
     const float* a_log; const float* dt_bias; const float* skip;
     const uint32_t* ctx; const uint32_t* cu_q; const int32_t* slots;
     int H, G, N, vd;
+    int x_off, b_off, c_off;                 // columns of xbc where the heads' x, the groups' B and C start
+    const float* decay;                      // != NULL: the decay of a head is this constant and the step size is 1 (dt_in, a_log, dt_bias unused)
 };
 // A workgroup of 256 threads owns 256 / LPC columns of one (sequence, head)'s state S [N, vd]; LPC neighbouring lanes share a column,
 // each holding DP = ceil(N / LPC) of its rows in registers, and walk the new tokens in order:
@@ -189,9 +189,9 @@ template <int DP, int LPC, int CH> __global__ __launch_bounds__(256) void ssd_sc
     float S[DP];
 #pragma unroll
     for (int r = 0; r < DP; ++r) { const int i = part * DP + r; S[r] = (own && i < N && start_pos > 0) ? stt[(size_t)i * vd + col] : 0.f; }
-    const int x_col = h * vd + col, b_off = p.H * vd + g * N, c_off = p.H * vd + p.G * N + g * N;
-    const float a_rate = expf(p.a_log[h]), dtb = p.dt_bias[h], skip = p.skip ? p.skip[h] : 0.f;
-    float rB[NPT], rC[NPT], rv[CH], rdt = 0.f, rdec = 1.f;
+    const int x_col = p.x_off + h * vd + col, b_off = p.b_off + g * N, c_off = p.c_off + g * N;
+    const float a_rate = p.decay ? 0.f : expf(p.a_log[h]), dtb = p.decay ? 0.f : p.dt_bias[h], skip = p.skip ? p.skip[h] : 0.f;
+    float rB[NPT], rC[NPT], rv[CH], rdt = p.decay ? 1.f : 0.f, rdec = p.decay ? p.decay[h] : 1.f;
     auto fetch = [&](int t0) {
 #pragma unroll
         for (int n = 0; n < NPT; ++n) {
@@ -203,7 +203,7 @@ template <int DP, int LPC, int CH> __global__ __launch_bounds__(256) void ssd_sc
         }
 #pragma unroll
         for (int c = 0; c < CH; ++c) rv[c] = (own && t0 + c < te) ? p.xbc[(size_t)(t0 + c) * p.ldx + x_col] : 0.f;
-        if (tid < CH && t0 + tid < te) {
+        if (!p.decay && tid < CH && t0 + tid < te) {
             rdt = softplusf_(p.dt_in[(size_t)(t0 + tid) * p.ldd + h] + dtb);
             rdec = expf(-a_rate * rdt);
         }
@@ -253,6 +253,176 @@ template <int DP, int LPC, int CH> __global__ __launch_bounds__(256) void ssd_sc
     if (own)
 #pragma unroll
         for (int r = 0; r < DP; ++r) { const int i = part * DP + r; if (i < N) stt[(size_t)i * vd + col] = S[r]; }
+}
+
+// ------------------------------------------------------------------------------------------------------------ constant decay, by pieces
+// Linear attention with a constant decay per head, portions of prompts: the new tokens of a sequence are cut into pieces of LC tokens
+// that are worked on side by side (i, t: places in the piece, n: its tokens, S_in: the state in front of it, a: the decay),
+//   U = sum_t a^(n-1-t) k_t v_t^T                                   piece_state: what the piece adds to the state
+//   S_in of the next piece = a^n S_in + U                           piece_scan: the only sequential part, elementwise over the state
+//   o_i = sum_(t <= i) a^(i-t) (q_i . k_t) v_t + a^(i+1) q_i S_in   piece_output
+// All products run on the f32 matrix cores (16 x 16 tiles, 4 deep; no reduced precision): the result is the recurrence's up to f32 rounding.
+constexpr int LC = 64;
+struct PieceArgs {
+    float* o; float* state; int64_t state_stride;
+    const float* qkv; int ldq, q_off, k_off, v_off;
+    const float* decay; float* U;                // U [pieces, H, d, vd]: first what a piece adds, then the state in front of it
+    const uint32_t* ctx; const uint32_t* cu_q; const int32_t* slots;
+    int n_seqs, H, d, vd;
+};
+__device__ __forceinline__ f32x4_t mfma_f32(float a, float b, const f32x4_t& c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+// piece b of the step -> its first token and its tokens (0: past the last piece)
+__device__ __forceinline__ int piece_of(const PieceArgs& p, int b, int& t0) {
+    for (int s = 0; s < p.n_seqs; ++s) {
+        const int tb = (int)p.cu_q[s], n = (int)p.cu_q[s + 1] - tb, pieces = (n + LC - 1) / LC;
+        if (b < pieces) { t0 = tb + b * LC; return min(LC, n - b * LC); }
+        b -= pieces;
+    }
+    return 0;
+}
+
+// a wave takes 16 columns of U and walks its rows 128 at a time: 8 tiles of K^T against one of V
+__global__ __launch_bounds__(256) void decay_piece_state_kernel(PieceArgs p) {
+    __shared__ float pw[LC + 1];
+    int t0;
+    const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y;
+    if (n == 0) return;
+    for (int i = threadIdx.x; i <= LC; i += blockDim.x) pw[i] = powf(p.decay[h], (float)i);
+    __syncthreads();
+    const int lane = threadIdx.x & 63, m16 = lane & 15, kg = lane >> 4, col = (blockIdx.z * 4 + (threadIdx.x >> 6)) * 16 + m16;
+    if (col - m16 >= p.vd) return;
+    const float* K = p.qkv + (size_t)t0 * p.ldq + p.k_off + h * p.d;
+    const float* V = p.qkv + (size_t)t0 * p.ldq + p.v_off + h * p.vd + col;
+    float* U = p.U + ((size_t)blockIdx.x * p.H + h) * p.d * p.vd;
+    for (int r0 = 0; r0 < p.d; r0 += 128) {
+        f32x4_t acc[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+        for (int t = 0; t < n; t += 4) {
+            const bool on = t + kg < n;
+            const float b = on ? V[(size_t)(t + kg) * p.ldq] * pw[n - 1 - t - kg] : 0.f;
+            float a[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) a[i] = (on && r0 + 16 * i < p.d) ? K[(size_t)(t + kg) * p.ldq + r0 + 16 * i + m16] : 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) acc[i] = mfma_f32(a[i], b, acc[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+            if (r0 + 16 * i < p.d)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) U[(size_t)(r0 + 16 * i + 4 * kg + v) * p.vd + col] = acc[i][v];
+    }
+}
+
+// a thread per element of a (sequence, head)'s state: the states in front of its pieces, then the one behind the last
+__global__ __launch_bounds__(256) void decay_piece_scan_kernel(PieceArgs p) {
+    const int s = blockIdx.x, h = blockIdx.y, e = blockIdx.z * 256 + threadIdx.x, per = p.d * p.vd;
+    const int n = (int)p.cu_q[s + 1] - (int)p.cu_q[s];
+    if (e >= per || n <= 0) return;
+    int first = 0;
+    for (int i = 0; i < s; ++i) first += ((int)p.cu_q[i + 1] - (int)p.cu_q[i] + LC - 1) / LC;
+    const int pieces = (n + LC - 1) / LC;
+    float* stt = p.state + (size_t)p.slots[s] * p.state_stride + (size_t)h * per + e;
+    float S = (int)p.ctx[s] > n ? *stt : 0.f;
+    const float a = p.decay[h], whole = powf(a, (float)LC), rest = powf(a, (float)(n - (pieces - 1) * LC));
+    const size_t step = (size_t)p.H * per;
+    float* u = p.U + (size_t)first * step + (size_t)h * per + e;
+    constexpr int AHEAD = 8;                      // pieces whose contributions are requested together
+    for (int c0 = 0; c0 < pieces; c0 += AHEAD) {
+        float add[AHEAD];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) add[i] = c0 + i < pieces ? u[(size_t)(c0 + i) * step] : 0.f;
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i)
+            if (c0 + i < pieces) {
+                u[(size_t)(c0 + i) * step] = S;
+                S = fmaf(c0 + i + 1 < pieces ? whole : rest, S, add[i]);
+            }
+    }
+    *stt = S;
+}
+
+// a wave takes 16 queries of the piece and 16 VT columns of the output: the scores against the keys up to its own tile, masked and
+// weighted with the powers of the decay, through LDS into the layout of a left operand; then the two products into one accumulator.
+// (The depth of a product is walked in the order 16 j + 4 kg + e, e innermost, on both operands: rows are read 16 bytes at a time.)
+template <int VT> __global__ __launch_bounds__(256) void decay_piece_output_kernel(PieceArgs p) {
+    constexpr int PR = LC + 4;
+    __shared__ float pw[LC + 1];
+    __shared__ __align__(16) float P[4][16 * PR];
+    int t0;
+    const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y;
+    if (n == 0) return;
+    for (int i = threadIdx.x; i <= LC; i += blockDim.x) pw[i] = powf(p.decay[h], (float)i);
+    __syncthreads();
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4, row0 = 16 * wave;
+    if (row0 >= n) return;
+    const int d = p.d, vd = p.vd, col0 = blockIdx.z * 16 * VT;
+    const float* base = p.qkv + (size_t)t0 * p.ldq;
+    const float* Q = base + p.q_off + h * d + (size_t)min(row0 + m16, n - 1) * p.ldq + 4 * kg;
+    const float* K = base + p.k_off + h * d + 4 * kg;
+    const float* V = base + p.v_off + h * vd + col0 + m16;
+    const float* S = p.U + ((size_t)blockIdx.x * p.H + h) * d * vd + col0 + m16;
+    const float qscale = pw[row0 + m16 + 1];
+    f32x4_t sc[4], acc[VT];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) sc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int c = 0; c < VT; ++c) acc[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const float* Kr[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) Kr[i] = K + (size_t)min(16 * i + m16, n - 1) * p.ldq;
+    for (int j = 0; j < d; j += 16) {
+        const float4 q = *reinterpret_cast<const float4*>(Q + j);
+        const float qa[4] = {q.x, q.y, q.z, q.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            if (i > wave) break;
+            const float4 k = *reinterpret_cast<const float4*>(Kr[i] + j);
+            const float ka[4] = {k.x, k.y, k.z, k.w};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) sc[i] = mfma_f32(qa[e], ka[e], sc[i]);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) {
+                const float b = col0 + 16 * c < vd ? S[(size_t)(j + 4 * kg + e) * vd + 16 * c] : 0.f;
+                acc[c] = mfma_f32(qa[e] * qscale, b, acc[c]);
+            }
+    }
+    float* Pw = P[wave];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const int r = row0 + 4 * kg + v, t = 16 * i + m16;
+            Pw[(4 * kg + v) * PR + t] = (t <= r && t < n) ? sc[i][v] * pw[max(r - t, 0)] : 0.f;
+        }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); __builtin_amdgcn_wave_barrier();
+    for (int j = 0; j <= row0; j += 16) {
+        const float4 a4 = *reinterpret_cast<const float4*>(&Pw[m16 * PR + j + 4 * kg]);
+        const float a[4] = {a4.x, a4.y, a4.z, a4.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int t = j + 4 * kg + e;
+#pragma unroll
+            for (int c = 0; c < VT; ++c) {
+                const float b = (t < n && col0 + 16 * c < vd) ? V[(size_t)t * p.ldq + 16 * c] : 0.f;
+                acc[c] = mfma_f32(a[e], b, acc[c]);
+            }
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < VT; ++c) {
+        if (col0 + 16 * c >= vd) break;
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const int r = row0 + 4 * kg + v;
+            if (r < n) p.o[((size_t)(t0 + r) * p.H + h) * vd + col0 + 16 * c + m16] = acc[c][v];
+        }
+    }
 }
 
 inline unsigned blocks_of(int64_t n) { return (unsigned)((n + 255) / 256); }
@@ -373,15 +543,9 @@ int mi355_hyb_gate_group_norm(void* out, int32_t out_dtype, const float* y, cons
     LAUNCH_OK(); return 0;
 }
 
-int mi355_hyb_ssd_scan(float* y, float* state, int64_t state_stride, const float* xbc, int32_t ldx, const float* dt_in, int32_t ldd,
-                       const float* a_log, const float* dt_bias, const float* skip, const uint32_t* context_lens,
-                       const uint32_t* cu_seqlens_q, const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads,
-                       int32_t groups, int32_t n_state, int32_t vdim, int64_t stream) {
-    if (!y || !state || !xbc || !dt_in || !a_log || !dt_bias || !context_lens || !cu_seqlens_q || !state_slots) return -1;
-    if (heads <= 0 || groups <= 0 || heads % groups || n_state <= 0 || n_state > 512 || vdim <= 0) return -1;
-    if (ldx < heads * vdim + 2 * groups * n_state || ldd < heads) return -1;
-    if (num_seqs <= 0 || num_tokens <= 0) return 0;
-    SsdArgs p{y, state, state_stride, xbc, ldx, dt_in, ldd, a_log, dt_bias, skip, context_lens, cu_seqlens_q, state_slots, heads, groups, n_state, vdim};
+// (portions of prompts: 16 tokens per stage, so that the wait for a stage's rows is paid half as often; decoding batches: 8)
+static int ssd_launch(const SsdArgs& p, int num_seqs, int num_tokens, int64_t stream) {
+    const int n_state = p.N, vdim = p.vd, heads = p.H;
     hipStream_t s_ = to_stream(stream);
     if (n_state < 64) {
         const dim3 grid(num_seqs, heads, (vdim + 63) / 64);
@@ -390,13 +554,55 @@ int mi355_hyb_ssd_scan(float* y, float* state, int64_t state_stride, const float
         else ssd_scan_kernel<16, 4, 8><<<grid, 256, 0, s_>>>(p);
     } else {
         const dim3 grid(num_seqs, heads, (vdim + 15) / 16);
-        // portions of prompts: 16 tokens per stage (the wait for a stage's rows is paid half as often); decoding batches: 8
         const bool longer = num_tokens > 8 * num_seqs;
         if (n_state <= 64) { if (longer) ssd_scan_kernel<4, 16, 16><<<grid, 256, 0, s_>>>(p); else ssd_scan_kernel<4, 16, 8><<<grid, 256, 0, s_>>>(p); }
         else if (n_state <= 128) { if (longer) ssd_scan_kernel<8, 16, 16><<<grid, 256, 0, s_>>>(p); else ssd_scan_kernel<8, 16, 8><<<grid, 256, 0, s_>>>(p); }
         else if (n_state <= 256) ssd_scan_kernel<16, 16, 8><<<grid, 256, 0, s_>>>(p);
         else ssd_scan_kernel<32, 16, 4><<<grid, 256, 0, s_>>>(p);       // (stages of 4 tokens: two stages of B and C rows of 512 states fill LDS)
     }
+    LAUNCH_OK(); return 0;
+}
+
+int mi355_hyb_ssd_scan(float* y, float* state, int64_t state_stride, const float* xbc, int32_t ldx, const float* dt_in, int32_t ldd,
+                       const float* a_log, const float* dt_bias, const float* skip, const uint32_t* context_lens,
+                       const uint32_t* cu_seqlens_q, const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads,
+                       int32_t groups, int32_t n_state, int32_t vdim, int64_t stream) {
+    if (!y || !state || !xbc || !dt_in || !a_log || !dt_bias || !context_lens || !cu_seqlens_q || !state_slots) return -1;
+    if (heads <= 0 || groups <= 0 || heads % groups || n_state <= 0 || n_state > 512 || vdim <= 0) return -1;
+    if (ldx < heads * vdim + 2 * groups * n_state || ldd < heads) return -1;
+    if (num_seqs <= 0 || num_tokens <= 0) return 0;
+    SsdArgs p{y, state, state_stride, xbc, ldx, dt_in, ldd, a_log, dt_bias, skip, context_lens, cu_seqlens_q, state_slots, heads, groups, n_state, vdim,
+              0, heads * vdim, heads * vdim + groups * n_state, nullptr};
+    return ssd_launch(p, num_seqs, num_tokens, stream);
+}
+
+int64_t mi355_hyb_decay_attention_scratch(int32_t num_tokens, int32_t num_seqs, int32_t heads, int32_t dim, int32_t vdim) {
+    if (num_tokens < LC || num_tokens <= 8 * (int64_t)num_seqs || heads <= 0 || dim <= 0 || vdim <= 0 || dim % 16 || vdim % 16 || dim > 512) return 0;
+    return ((int64_t)num_tokens / LC + num_seqs) * heads * dim * vdim;
+}
+
+int mi355_hyb_decay_attention(float* o, float* state, int64_t state_stride, const float* qkv, int32_t ldq, int32_t q_off, int32_t k_off,
+                              int32_t v_off, const float* decay, const uint32_t* context_lens, const uint32_t* cu_seqlens_q,
+                              const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads, int32_t dim, int32_t vdim,
+                              float* scratch, int64_t stream) {
+    if (!o || !state || !qkv || !decay || !context_lens || !cu_seqlens_q || !state_slots) return -1;
+    if (heads <= 0 || heads > 65535 || dim <= 0 || dim > 512 || vdim <= 0 || q_off < 0 || k_off < 0 || v_off < 0) return -1;
+    if (ldq < q_off + heads * dim || ldq < k_off + heads * dim || ldq < v_off + heads * vdim) return -1;
+    if (num_seqs <= 0 || num_tokens <= 0) return 0;
+    const bool pieces = scratch && dim % 16 == 0 && vdim % 16 == 0;
+    if (!pieces || ldq % 4 || q_off % 4 || k_off % 4 || (uintptr_t)qkv % 16) {
+        SsdArgs p{o, state, state_stride, qkv, ldq, nullptr, 0, nullptr, nullptr, nullptr, context_lens, cu_seqlens_q, state_slots, heads, heads, dim, vdim,
+                  v_off, k_off, q_off, decay};
+        return ssd_launch(p, num_seqs, num_tokens, stream);
+    }
+    PieceArgs p{o, state, state_stride, qkv, ldq, q_off, k_off, v_off, decay, scratch, context_lens, cu_seqlens_q, state_slots, num_seqs, heads, dim, vdim};
+    hipStream_t s_ = to_stream(stream);
+    const unsigned np = (unsigned)(num_tokens / LC + num_seqs);
+    decay_piece_state_kernel<<<dim3(np, heads, (vdim + 63) / 64), 256, 0, s_>>>(p);
+    decay_piece_scan_kernel<<<dim3(num_seqs, heads, (dim * vdim + 255) / 256), 256, 0, s_>>>(p);
+    if (vdim <= 32) decay_piece_output_kernel<2><<<dim3(np, heads, 1), 256, 0, s_>>>(p);
+    else if (vdim <= 64) decay_piece_output_kernel<4><<<dim3(np, heads, 1), 256, 0, s_>>>(p);
+    else decay_piece_output_kernel<8><<<dim3(np, heads, (vdim + 127) / 128), 256, 0, s_>>>(p);
     LAUNCH_OK(); return 0;
 }
 

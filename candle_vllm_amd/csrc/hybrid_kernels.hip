@@ -51,7 +51,18 @@ struct LinArgs {
     // grouped product (blk != NULL): the rows come in blocks of blk_rows = the kernel's tile height; block b = blockIdx.y multiplies its
     // rows [b blk_rows, blk[2b + 1]) with matrix blk[2b] (w + blk[2b] w_bs); row r of `a` is read at row_src[r] when row_src != NULL
     const int32_t* blk; const int32_t* row_src; int blk_rows;
+    // epilogue: columns < act_cols pass an activation (MI355_HYB_ACT_*), out16: `out` holds bf16 instead of f32
+    int act, act_cols, out16;
 };
+__device__ __forceinline__ void lin_store(const LinArgs& p, int t, int n, float v) {
+    if (p.act && n < p.act_cols) {
+        if (p.act == MI355_HYB_ACT_SILU) v = siluf_(v);
+        else if (p.act == MI355_HYB_ACT_GELU) v = gelu_tanhf_(v);
+        else { v = fmaxf(v, 0.f); v *= v; }
+    }
+    if (p.out16) reinterpret_cast<uint16_t*>(p.out)[(size_t)t * p.ldo + n] = f32_to_bf16(v);
+    else p.out[(size_t)t * p.ldo + n] = v;
+}
 // the block's matrix and the end of its rows (one past the last); false = nothing to do
 __device__ __forceinline__ bool lin_group(LinArgs& p, int t0, int64_t& w_off) {
     w_off = (int64_t)blockIdx.z * p.w_bs;
@@ -109,7 +120,7 @@ template <typename TA, int MT> __global__ __launch_bounds__(256) void linear_bf1
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const int t = t0 + i * 16 + 4 * kg + v;
-            if (t < p.T) p.out[(size_t)t * p.ldo + n] = acc[i][v] + bias;
+            if (t < p.T) lin_store(p, t, n, acc[i][v] + bias);
         }
 }
 
@@ -187,7 +198,7 @@ __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(LinArgs p) {
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
                 const int t = t0 + wr * 64 + i * 16 + 4 * kg + v;
-                if (t < p.T) p.out[(size_t)t * p.ldo + n] = acc[i][j][v] + bias;
+                if (t < p.T) lin_store(p, t, n, acc[i][j][v] + bias);
             }
     }
 }
@@ -228,7 +239,7 @@ template <typename TA, int NW, int UNR> __global__ __launch_bounds__(64 * NW) vo
 #pragma unroll
             for (int w = 0; w < NW; ++w) s += part[w][v][lane];
             const int t = t0 + 4 * kg + v;
-            if (nok && t < p.T) p.out[(size_t)t * p.ldo + n] = s + bias;
+            if (nok && t < p.T) lin_store(p, t, n, s + bias);
         }
     }
 }
@@ -274,7 +285,7 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(LinArgs p) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < p.N) p.out[(size_t)t * p.ldo + n] = acc[i][j] + (p.bias ? p.bias[n] : 0.f);
+            if (n < p.N) lin_store(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
         }
     }
 }
@@ -392,9 +403,6 @@ template <typename TO> __global__ __launch_bounds__(256) void gather_group_norm_
     }
 }
 
-__device__ __forceinline__ float gelu_tanhf_(float z) {
-    return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
 template <typename TO> __global__ void gelu_glu_kernel(TO* out, const float* gu, int64_t n, int ff) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
@@ -490,6 +498,12 @@ struct AttnArgs {
     int cpk;                // lanes that share a key row when it is read 16 bytes a lane (power of two >= d / elements per 16 bytes)
     int keep;               // with a window: keys at positions < keep stay visible (the first tokens of the sequence)
     const float* dist;      // != NULL: [2, H] = r1, r2; score <- score - r1[h] ln(1 + r2[h] (query position - key position))
+    int chunked;            // the window is a chunk: a query sees the keys from the last multiple of `window` at or below its position on
+    // the lowest key that a query sees (beside the kept first tokens)
+    __device__ __forceinline__ int first_key(int pos) const {
+        if (window <= 0) return 0;
+        return chunked ? pos - pos % window : max(0, pos - window + 1);
+    }
 };
 // (the hardware's log2: the argument is at least 1, so the absolute error stays near the f32 rounding of the score it is taken from)
 __device__ __forceinline__ float dist_bias(float r1, float r2, int d) { return r1 * 0.6931471805599453f * __log2f(fmaf(r2, (float)d, 1.f)); }
@@ -531,7 +545,7 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
     const int s = p.tok_seq[t];
     const int n_new = (int)(p.cu_q[s + 1] - p.cu_q[s]);
     const int pos = (int)p.ctx[s] - n_new + (t - (int)p.cu_q[s]);
-    const int lo = p.window > 0 ? max(0, pos - p.window + 1) : 0;
+    const int lo = p.first_key(pos);
     // the visible keys in one run of indices: the kept first tokens below the window (nkeep of them), then the window [lo, pos]
     const int nkeep = min(p.keep, lo), n_vis = nkeep + pos - lo + 1;
     const int g = h / (p.H / p.G);
@@ -729,7 +743,10 @@ void window_attention_mfma_kernel(AttnArgs p) {
         for (int c = 0; c < VT; ++c) acc[n][c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     const int hi = pos0 + nq - 1;
     const float r1 = p.dist ? p.dist[h] : 0.f, r2 = p.dist ? p.dist[p.H + h] : 0.f;
-    const int lo = p.window > 0 ? max(0, pos0 - p.window + 1) : 0;
+    const int lo = p.first_key(pos0);
+    int low[4];                                                      // lowest key of this lane's four query rows
+#pragma unroll
+    for (int v = 0; v < 4; ++v) low[v] = p.first_key(pos0 + 4 * kg + v);
     // the keys any query of the tile may see, in one run of indices: the kept first tokens below the lowest window, then [lo, hi]
     const int nkeep = min(p.keep, lo), n_vis = nkeep + hi - lo + 1;
     auto key_at = [&](int i) { return i < nkeep ? i : (i < n_vis ? lo + (i - nkeep) : hi + 1); };
@@ -805,7 +822,7 @@ void window_attention_mfma_kernel(AttnArgs p) {
 #pragma unroll
             for (int kt = 0; kt < 4; ++kt) {
                 const int key = key_at(j0 + kt * 16 + m16);
-                const bool ok_ = r < nq && key <= qpos && (p.window == 0 || qpos - key < p.window || key < p.keep);
+                const bool ok_ = r < nq && key <= qpos && (key >= low[v] || key < p.keep);
                 sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - (p.dist ? dist_bias(r1, r2, qpos - key) : 0.f) : -INFINITY;
                 mx[v] = fmaxf(mx[v], sc[v][kt]);
             }
@@ -921,7 +938,10 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
     for (int c = 0; c < VT; ++c) acc[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     const int hi = pos0 + nq - 1;
     const float r1 = p.dist ? p.dist[h] : 0.f, r2 = p.dist ? p.dist[p.H + h] : 0.f;
-    const int lo = p.window > 0 ? max(0, pos0 - p.window + 1) : 0;
+    const int lo = p.first_key(pos0);
+    int low[4];                                                      // lowest key of this lane's four query rows
+#pragma unroll
+    for (int v = 0; v < 4; ++v) low[v] = p.first_key(pos0 + 4 * kg + v);
     const int nkeep = min(p.keep, lo), n_vis = nkeep + hi - lo + 1;
     auto key_at = [&](int i) { return i < nkeep ? i : (i < n_vis ? lo + (i - nkeep) : hi + 1); };
     auto page_row = [&](int key) { return (size_t)bt[key / p.bs] * p.bs + (key % p.bs); };
@@ -989,7 +1009,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
 #pragma unroll
             for (int kt = 0; kt < 4; ++kt) {
                 const int key = key_at(j0 + kt * 16 + m16);
-                const bool ok_ = r < nq && key <= qpos && (p.window == 0 || qpos - key < p.window || key < p.keep);
+                const bool ok_ = r < nq && key <= qpos && (key >= low[v] || key < p.keep);
                 sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - (p.dist ? dist_bias(r1, r2, qpos - key) : 0.f) : -INFINITY;
                 mx[v] = fmaxf(mx[v], sc[v][kt]);
             }
@@ -1518,7 +1538,8 @@ template <typename TO> __global__ void head_gate_kernel(TO* out, const float* in
 template <typename TO, int NW> __global__ __launch_bounds__(64 * NW) void moe_route_kernel(int32_t* ids, float* wts, float* sgate, TO* xn, const float* x,
                                                                                const float* norm_w, const float* router, const float* corr,
                                                                                const float* gate_row, int width, int E, int K, float scale,
-                                                                               float eps, int append, int sig, int groups, int keep, int normalise) {
+                                                                               float eps, int append, int sig, int groups, int keep, int normalise,
+                                                                               const float* bias) {
     extern __shared__ __align__(16) float rsm[];
     float* hs = rsm;                       // [width]
     float* logit = hs + width;             // [E + 1]
@@ -1561,27 +1582,31 @@ template <typename TO, int NW> __global__ __launch_bounds__(64 * NW) void moe_ro
             for (int i = lane; i < width; i += 64) acc = fmaf(hs[i], g[i], acc);
         }
         acc = wave_sum(acc);
-        if (lane == 0) logit[e] = acc;
+        if (lane == 0) logit[e] = (bias && e < E) ? acc + bias[e] : acc;
     }
     __syncthreads();
     if (wave != 0) return;
     const int KS = K + (append ? 1 : 0);                                // pairs per token: the shared expert as one more pair of every token
-    if (gate_row && lane == 0) {
-        const float sg = sigmoidf_(logit[E]);
+    if ((gate_row || append) && lane == 0) {
+        const float sg = gate_row ? sigmoidf_(logit[E]) : 1.f;
         if (sgate) sgate[t] = sg;
         if (append) { ids[(size_t)t * KS + K] = E; wts[(size_t)t * KS + K] = sg; }
     }
-    // scores s (softmax or sigmoid of the logits) and choice scores s + correction, in LDS
-    if (sig) {
+    // scores s (sig 0: softmax of the logits, 1: sigmoid, 2: softmax up to its denominator) and choice scores, in LDS
+    if (sig == 1) {
         for (int e = lane; e < E; e += 64) { const float v = sigmoidf_(logit[e]); sc[e] = v; cv[e] = v + (corr ? corr[e] : 0.f); }
     } else {
         float m = -INFINITY;
         for (int e = lane; e < E; e += 64) m = fmaxf(m, logit[e]);
         m = wave_max(m);
+        if (sig == 2) {                                                 // chosen by the logits themselves; normalised over the chosen ones below
+            for (int e = lane; e < E; e += 64) { sc[e] = expf(logit[e] - m); cv[e] = logit[e] + (corr ? corr[e] : 0.f); }
+        } else {
         float den = 0.f;
         for (int e = lane; e < E; e += 64) den += expf(logit[e] - m);
         den = wave_sum(den);
         for (int e = lane; e < E; e += 64) { const float v = expf(logit[e] - m) / den; sc[e] = v; cv[e] = v + (corr ? corr[e] : 0.f); }
+        }
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); __builtin_amdgcn_wave_barrier();
     if (groups > 0) {
@@ -1764,10 +1789,12 @@ int mi355_hyb_fill_f32(float* out, float v, int64_t n, int64_t stream) {
 }
 
 static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, int32_t a_dtype, int32_t lda, int64_t a_bs, const void* w,
-                         int64_t w_bs, const float* bias, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream) {
+                         int64_t w_bs, const float* bias, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream,
+                         int32_t act = 0, int32_t act_cols = 0, int32_t out16 = 0) {
     if (!out || !a || !w || T < 0 || n <= 0 || k <= 0 || ldo < n || lda < k || batch <= 0 || batch > 65535 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
     if (T == 0) return 0;
     LinArgs p{out, ldo, a, lda, w, bias, T, n, k, 0, 0, a_bs, w_bs, o_bs};
+    p.act = act; p.act_cols = act_cols; p.out16 = out16;
     hipStream_t st_ = to_stream(stream);
     const unsigned nz = (unsigned)batch;
     if (dtype == MI355_DTYPE_F32) {
@@ -1798,6 +1825,12 @@ static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, i
 int mi355_hyb_linear(float* out, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const void* w, const float* bias,
                      int32_t T, int32_t n, int32_t k, int32_t dtype, int64_t stream) {
     return linear_launch(out, ldo, 0, a, a_dtype, lda, 0, w, 0, bias, T, n, k, 1, dtype, stream);
+}
+int mi355_hyb_linear_act(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const void* w, const float* bias,
+                         int32_t T, int32_t n, int32_t k, int32_t act, int32_t act_cols, int32_t dtype, int64_t stream) {
+    if (act < 0 || act > MI355_HYB_ACT_RELU2 || act_cols < 0 || !is_dt(out_dtype)) return -1;
+    return linear_launch(static_cast<float*>(out), ldo, 0, a, a_dtype, lda, 0, w, 0, bias, T, n, k, 1, dtype, stream, act, act_cols,
+                         out_dtype == MI355_DTYPE_BF16);
 }
 int mi355_hyb_linear_batched(float* out, int32_t ldo, int64_t o_bs, const void* a, int32_t a_dtype, int32_t lda, int64_t a_bs,
                              const void* w, int64_t w_bs, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream) {
@@ -1907,7 +1940,18 @@ int mi355_hyb_biased_attention(void* out, int32_t out_dtype, int32_t ldo, int32_
                                int32_t num_seqs, int32_t T, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim,
                                int32_t block_size, int32_t max_blocks, int32_t window, int32_t keep_first, float scale, float out_scale,
                                int32_t k_ld, int32_t v_ld, float softcap, int32_t cross_values, int32_t dtype, int64_t stream) {
-    if (keep_first < 0) return -1;
+    return mi355_hyb_attention(out, out_dtype, ldo, out_off, q, k_pages, v_pages, block_tables, context_lens, cu_seqlens_q, tok_seq, sink, dist,
+                               num_seqs, T, heads, kv_heads, dim, vdim, block_size, max_blocks, MI355_HYB_MASK_SLIDING, window, keep_first, scale,
+                               out_scale, k_ld, v_ld, softcap, cross_values, dtype, stream);
+}
+
+int mi355_hyb_attention(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const void* q, const void* k_pages, const void* v_pages,
+                        const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_seqlens_q, const int32_t* tok_seq,
+                        const float* sink, const float* dist, int32_t num_seqs, int32_t T, int32_t heads, int32_t kv_heads, int32_t dim,
+                        int32_t vdim, int32_t block_size, int32_t max_blocks, int32_t mask_kind, int32_t window, int32_t keep_first,
+                        float scale, float out_scale, int32_t k_ld, int32_t v_ld, float softcap, int32_t cross_values, int32_t dtype,
+                        int64_t stream) {
+    if (keep_first < 0 || mask_kind < MI355_HYB_MASK_SLIDING || mask_kind > MI355_HYB_MASK_CHUNKED) return -1;
     if (!out || !q || !k_pages || !v_pages || !block_tables || !context_lens || !cu_seqlens_q || !tok_seq) return -1;
     if (!is_dt(dtype) || !is_dt(out_dtype) || heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || vdim <= 0) return -1;
     if (block_size <= 0 || max_blocks <= 0 || window < 0 || softcap < 0.f) return -1;
@@ -1927,6 +1971,7 @@ int mi355_hyb_biased_attention(void* out, int32_t out_dtype, int32_t ldo, int32_
     p.cpk = 64;
     p.keep = window > 0 ? keep_first : 0;
     p.dist = dist;
+    p.chunked = mask_kind == MI355_HYB_MASK_CHUNKED;
     if (vec) { int c = 1; while (c < vdim / epv) c <<= 1; p.cp2 = c; c = 1; while (c < dim / epv) c <<= 1; p.cpk = c; }
     else if (vdim > 512) return -1;
     // prompt-sized steps over bf16 pages: the matrix-core kernel (a tile of 16 tokens never spans two sequences)
@@ -2219,9 +2264,16 @@ int mi355_hyb_moe_route_ex(int32_t* expert_ids, float* weights, float* shared_ga
                            const float* norm_w, const float* router, const float* correction, const float* gate_row, int32_t T,
                            int32_t width, int32_t experts, int32_t top, float scale, float eps, int32_t append_shared,
                            int32_t sigmoid_scores, int32_t groups, int32_t keep_groups, int32_t normalise, int64_t stream) {
-    if (groups < 0 || (groups > 0 && (experts % groups || keep_groups < 1 || keep_groups > groups || (experts / groups) * keep_groups < top))) return -1;
+    return mi355_hyb_moe_route_biased(expert_ids, weights, shared_gate, xn, out_dtype, x, norm_w, router, nullptr, correction, gate_row, T, width,
+                                      experts, top, scale, eps, append_shared, sigmoid_scores ? 1 : 0, groups, keep_groups, normalise, stream);
+}
+int mi355_hyb_moe_route_biased(int32_t* expert_ids, float* weights, float* shared_gate, void* xn, int32_t out_dtype, const float* x,
+                               const float* norm_w, const float* router, const float* router_bias, const float* correction, const float* gate_row,
+                               int32_t T, int32_t width, int32_t experts, int32_t top, float scale, float eps, int32_t append_shared,
+                               int32_t score_kind, int32_t groups, int32_t keep_groups, int32_t normalise, int64_t stream) {
+    if (score_kind < 0 || score_kind > 2 || groups < 0 || (groups > 0 && (experts % groups || keep_groups < 1 || keep_groups > groups || (experts / groups) * keep_groups < top))) return -1;
     if (!expert_ids || !weights || !x || !router || width <= 0 || experts < 1 || experts > 4096 || top < 1 || top > experts) return -1;
-    if ((gate_row && !shared_gate && !append_shared) || (append_shared && !gate_row) || (xn && !is_dt(out_dtype))) return -1;
+    if ((gate_row && !shared_gate && !append_shared) || (xn && !is_dt(out_dtype))) return -1;
     if (T <= 0) return 0;
     const size_t lds = (size_t)(width + 4 * experts + 1) * sizeof(float);
     if (lds > 60000) return -1;
@@ -2229,7 +2281,7 @@ int mi355_hyb_moe_route_ex(int32_t* expert_ids, float* weights, float* shared_ga
     const bool bf = xn && out_dtype == MI355_DTYPE_BF16;
 #define ROUTE(TO, NW) moe_route_kernel<TO, NW><<<T, 64 * NW, lds, to_stream(stream)>>>(expert_ids, weights, shared_gate, (TO*)xn, x, norm_w, router, \
                                                                                        correction, gate_row, width, experts, top, scale, eps, append_shared ? 1 : 0, \
-                                                                                       sigmoid_scores ? 1 : 0, groups, keep_groups, normalise ? 1 : 0)
+                                                                                       score_kind, groups, keep_groups, normalise ? 1 : 0, router_bias)
     if (T <= 256) { if (bf) ROUTE(uint16_t, 16); else ROUTE(float, 16); }
     else { if (bf) ROUTE(uint16_t, 4); else ROUTE(float, 4); }
 #undef ROUTE
@@ -2258,10 +2310,19 @@ int mi355_hyb_moe_group(int32_t* pos, int32_t* row_token, int32_t* block_table, 
 int mi355_hyb_linear_grouped(float* out, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const int32_t* row_token, const void* w,
                              int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t n, int32_t k,
                              int32_t dtype, int64_t stream) {
+    return mi355_hyb_linear_grouped_act(out, MI355_DTYPE_F32, ldo, a, a_dtype, lda, row_token, w, w_bs, block_table, block_rows, n_blocks, n, k,
+                                        MI355_HYB_ACT_NONE, dtype, stream);
+}
+
+int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const int32_t* row_token,
+                                 const void* w, int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t n,
+                                 int32_t k, int32_t act, int32_t dtype, int64_t stream) {
+    if (act < 0 || act > MI355_HYB_ACT_RELU2 || !is_dt(out_dtype)) return -1;
     if (!out || !a || !w || !block_table || n <= 0 || k <= 0 || ldo < n || lda < k || w_bs < 0 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
     if (n_blocks <= 0) return 0;
     if (n_blocks > 65535) return -1;
-    LinArgs p{out, ldo, a, lda, w, nullptr, n_blocks * block_rows, n, k, 0, 0, 0, w_bs, 0, block_table, row_token, block_rows};
+    LinArgs p{static_cast<float*>(out), ldo, a, lda, w, nullptr, n_blocks * block_rows, n, k, 0, 0, 0, w_bs, 0, block_table, row_token, block_rows};
+    p.act = act; p.act_cols = n; p.out16 = out_dtype == MI355_DTYPE_BF16;
     hipStream_t st_ = to_stream(stream);
     if (dtype == MI355_DTYPE_F32) {
         if (a_dtype != MI355_DTYPE_F32 || block_rows != 64) return -1;

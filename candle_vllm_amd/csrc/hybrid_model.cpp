@@ -5,8 +5,10 @@
 // x itself; residual_form 2 puts a norm on both sides, x <- x + norm(sub(pre_norm(x))), optionally with a short causal convolution
 // added to the mixer's input; residual_form 3 has ONE norm per layer that mixer and feed-forward both read, x <- x + mixer(h) + ff(h),
 // then the token's side input and the average over the depth (a state-space mixer and an ungated feed-forward belong to that form's
-// design).  The feed-forward is a dense gate/up form or a mixture of experts (router, grouped expert products over
-// device-built blocks, shared expert).  A layer may run on another layer's weights (share_with) and still owns its pages and state.  Like the llama-family host layers
+// design); residual_form 4 carries the residual stream in several copies that every sublayer mixes (chunked attention and linear attention
+// with a constant decay belong to that form's design).  The feed-forward is a dense form with or without a gate or a mixture of experts
+// (router, grouped expert products over device-built blocks, shared expert).  A layer may run on another layer's weights (share_with)
+// and still owns its pages and state.  Like the llama-family host layers
 // (host_model.cpp, dense_model.cpp) it owns the weights, the K/V pages and the activation buffers and enqueues one step on a
 // stream; unlike them it owns a pool of recurrent state (one slot per live sequence, handed out by the block engine) and runs
 // prompts, portions of prompts and decoded tokens through the same launches.
@@ -57,6 +59,8 @@ struct HLayer {
     bool is_latent() const { return c.mixer == MI355_HYB_MIX_LATENT; }
     bool is_conv_attn() const { return c.mixer == MI355_HYB_MIX_CONV_ATTENTION; }
     bool is_ssd() const { return c.mixer == MI355_HYB_MIX_SSD; }
+    bool is_decay() const { return c.mixer == MI355_HYB_MIX_DECAY; }
+    int gate_up_rows() const { return (c.mlp_kind == 4 || c.mlp_kind == 5 || (c.mlp_kind == 3 && c.moe_relu2)) ? 1 : 2; }   // in units of the size
     bool uses_pages() const { return has_attn() || is_latent() || is_conv_attn(); }
     bool owns_pages() const { return uses_pages() && !c.kv_from; }       // a layer with kv_from reads another layer's pages
     int ssd_inner() const { return c.d_heads * c.d_vdim; }
@@ -89,6 +93,12 @@ struct HModel {
     float *y2 = nullptr, *hf = nullptr, *xs = nullptr, *side_g = nullptr;
     void *side_a = nullptr, *cq = nullptr;
     Weight side_table;
+    // form 4: the copies of the residual stream; embedding by pairs of tokens; scratch of the constant-decay attention by pieces
+    float *streams = nullptr, *pieces = nullptr;
+    int64_t cap_pieces = 0;
+    int32_t* bigram_rows = nullptr;
+    int64_t bigram_off = 0;
+    Weight bigram;
     bool need_hf = false, need_xs = false;
     int max_side = 0, max_q_rank = 0;
     float *moe_gu = nullptr, *moe_y = nullptr, *moe_wts = nullptr, *moe_sgate = nullptr;
@@ -132,10 +142,15 @@ int in_proj_parts(const mi355_hybrid_layer& c, int32_t* off) {
         off[P_G] = 0; off[P_DV] = inner; off[P_DK] = 2 * inner; off[P_DQ] = 2 * inner + gn; off[P_A] = 2 * inner + 2 * gn;
         return 2 * inner + 2 * gn + c.d_heads;
     }
+    if (c.mixer == MI355_HYB_MIX_DECAY) {                                // [q | k | v | gate]: silu on everything in front of the gate
+        off[P_DQ] = 0; off[P_DK] = c.d_heads * c.d_dim; off[P_DV] = 2 * c.d_heads * c.d_dim; off[P_G] = off[P_DV] + c.d_heads * c.d_vdim;
+        return off[P_G] + c.d_heads * c.d_vdim;
+    }
     if (c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION || c.mixer == MI355_HYB_MIX_CONV_ATTENTION) {
         off[P_AQ] = r; r += c.a_heads * c.a_dim;
         off[P_AK] = r; r += c.a_kv_heads * c.a_dim;
-        off[P_AV] = r; r += c.a_kv_heads * c.a_vdim;
+        if (c.a_v_is_k) off[P_AV] = off[P_AK];
+        else { off[P_AV] = r; r += c.a_kv_heads * c.a_vdim; }
     }
     if (c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_DELTA) {
         off[P_DQ] = r; r += c.d_kv_heads * c.d_dim;
@@ -151,7 +166,11 @@ int in_proj_parts(const mi355_hybrid_layer& c, int32_t* off) {
 bool layer_ok(const mi355_hybrid_layer& c) {
     const bool attn = c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION;
     const bool delta = c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_DELTA;
-    if (c.mixer < 0 || c.mixer > MI355_HYB_MIX_SSD || c.share_with < 0) return false;
+    if (c.mixer < 0 || c.mixer > MI355_HYB_MIX_DECAY || c.share_with < 0) return false;
+    if (c.mixer == MI355_HYB_MIX_DECAY && (c.d_heads <= 0 || c.d_dim <= 0 || c.d_dim > 512 || c.d_vdim <= 0)) return false;
+    if (c.a_mask_kind < MI355_HYB_MASK_SLIDING || c.a_mask_kind > MI355_HYB_MASK_CHUNKED || ((c.a_mask_kind || c.a_v_is_k) && !attn)) return false;
+    if (c.a_v_is_k && c.a_vdim != c.a_dim) return false;
+    if ((c.moe_relu2 || c.moe_bias || c.moe_shared_plain) && c.mlp_kind != 3) return false;
     if (c.mixer == MI355_HYB_MIX_SSD) {
         if (c.d_heads <= 0 || c.d_kv_heads <= 0 || c.d_heads % c.d_kv_heads || c.d_dim <= 0 || c.d_dim > 512 || c.d_vdim <= 0) return false;
         if (c.d_conv < 1 || c.d_conv > 16 || c.d_norm_groups < 1 || (c.d_heads * c.d_vdim) % c.d_norm_groups) return false;
@@ -183,7 +202,7 @@ bool layer_ok(const mi355_hybrid_layer& c) {
         if (c.d_gate != MI355_HYB_GATE_SIGMOID_LR && c.d_gate != MI355_HYB_GATE_SILU) return false;
     }
     if (c.mixer == MI355_HYB_MIX_MINGRU && c.g_width <= 0) return false;
-    if (c.mlp_kind < 0 || c.mlp_kind > 4 || (c.mlp_kind && c.mlp_ff <= 0)) return false;
+    if (c.mlp_kind < 0 || c.mlp_kind > 5 || (c.mlp_kind && c.mlp_ff <= 0)) return false;
     if (c.mlp_kind == 3 && (c.moe_experts < 1 || c.moe_experts > 4096 || c.moe_top < 1 || c.moe_top > c.moe_experts || c.moe_shared_ff < 0)) return false;
     if (c.a_keep_first < 0 || c.in_conv < 0 || c.in_conv > 16) return false;
     if ((c.a_keep_first || c.a_norm_after_rot || c.a_head_temp) && !attn) return false;      // switches of the plain attention branch
@@ -196,7 +215,7 @@ bool is_matrix(int which) {
         case MI355_HW_EMBED: case MI355_HW_HEAD: case MI355_HW_IN_PROJ: case MI355_HW_OUT_PROJ: case MI355_HW_D_A2: case MI355_HW_D_G2:
         case MI355_HW_MLP_GATE_UP: case MI355_HW_MLP_DOWN: case MI355_HW_L_UKT: case MI355_HW_L_UV:
         case MI355_HW_MOE_GATE_UP: case MI355_HW_MOE_DOWN: case MI355_HW_L_UQ: case MI355_HW_SIDE_GATE: case MI355_HW_SIDE_PROJ:
-        case MI355_HW_SIDE_TABLE: return true;
+        case MI355_HW_SIDE_TABLE: case MI355_HW_BIGRAM: return true;
         default: return false;
     }
 }
@@ -207,6 +226,7 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
         if (which == MI355_HW_EMBED) return (int64_t)m->cfg.vocab * W;
         if (which == MI355_HW_HEAD) return m->cfg.tie_head ? -1 : (int64_t)m->cfg.vocab * W;
         if (which == MI355_HW_FINAL_NORM) return W;
+        if (which == MI355_HW_BIGRAM) return m->cfg.bigram_buckets > 0 ? ((int64_t)m->cfg.bigram_buckets + 1) * W : -1;
         if (which == MI355_HW_SIDE_TABLE) return m->cfg.side_cols > 0 ? (int64_t)m->cfg.vocab * m->cfg.side_cols : -1;
         return -1;
     }
@@ -224,6 +244,12 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
         case MI355_HW_SIDE_GATE: case MI355_HW_SIDE_PROJ: return c.side_dim ? (int64_t)c.side_dim * W : -1;
         case MI355_HW_SIDE_NORM: return c.side_dim ? W : -1;
         case MI355_HW_DEPTH_W: return c.depth_terms ? c.depth_terms : -1;
+        case MI355_HW_HC1_IN: case MI355_HW_HC1_OUT: return m->cfg.residual_form == 4 ? m->cfg.streams : -1;
+        case MI355_HW_HC1_MIX: return m->cfg.residual_form == 4 ? m->cfg.streams * m->cfg.streams : -1;
+        case MI355_HW_HC2_IN: case MI355_HW_HC2_OUT: return m->cfg.residual_form == 4 && c.mlp_kind ? m->cfg.streams : -1;
+        case MI355_HW_HC2_MIX: return m->cfg.residual_form == 4 && c.mlp_kind ? m->cfg.streams * m->cfg.streams : -1;
+        case MI355_HW_MOE_BIAS: return c.moe_bias ? c.moe_experts : -1;
+        case MI355_HW_D_DECAY: return L.is_decay() ? c.d_heads : -1;
         case MI355_HW_IN_PROJ: return (int64_t)L.in_rows * W;
         case MI355_HW_IN_BIAS: return L.in_rows;
         case MI355_HW_OUT_PROJ: return (int64_t)W * L.out_k;
@@ -235,9 +261,9 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
         case MI355_HW_PRE_NORM1: return m->cfg.residual_form == 2 ? W : -1;
         case MI355_HW_PRE_NORM2: return m->cfg.residual_form == 2 && c.mlp_kind ? W : -1;
         case MI355_HW_IN_CONV: return c.in_conv ? (int64_t)W * c.in_conv : -1;
-        case MI355_HW_MOE_ROUTER: return c.mlp_kind == 3 ? (int64_t)(c.moe_experts + (c.moe_shared_ff ? 1 : 0)) * W : -1;
+        case MI355_HW_MOE_ROUTER: return c.mlp_kind == 3 ? (int64_t)(c.moe_experts + (c.moe_shared_ff && !c.moe_shared_plain ? 1 : 0)) * W : -1;
         case MI355_HW_MOE_CORRECTION: return c.mlp_kind == 3 ? c.moe_experts : -1;
-        case MI355_HW_MOE_GATE_UP: return c.mlp_kind == 3 ? (int64_t)(c.moe_experts + L.shared_merged()) * 2 * c.mlp_ff * W : -1;
+        case MI355_HW_MOE_GATE_UP: return c.mlp_kind == 3 ? (int64_t)(c.moe_experts + L.shared_merged()) * L.gate_up_rows() * c.mlp_ff * W : -1;
         case MI355_HW_MOE_DOWN: return c.mlp_kind == 3 ? (int64_t)(c.moe_experts + L.shared_merged()) * W * c.mlp_ff : -1;
         case MI355_HW_A_SINK: return (L.has_attn() || L.is_latent()) && c.a_has_sink ? c.a_heads : -1;
         case MI355_HW_A_CONV: return L.is_conv_attn() ? (int64_t)L.a_conv_channels() * c.a_conv : -1;
@@ -250,13 +276,12 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
         case MI355_HW_D_A_LOG: return L.has_delta() || L.is_ssd() ? c.d_heads : -1;
         case MI355_HW_D_DT_BIAS: if (L.is_ssd()) return c.d_heads;
                                  return L.has_delta() ? (c.d_decay_channels ? c.d_heads * c.d_dim : c.d_heads) : -1;
-        case MI355_HW_D_NORM: if (L.is_ssd()) return L.ssd_inner();
+        case MI355_HW_D_NORM: if (L.is_ssd() || L.is_decay()) return L.ssd_inner();
                               return L.has_delta() ? c.d_vdim : -1;
         case MI355_HW_D_A2: return L.has_delta() && c.d_decay_channels ? (int64_t)c.d_heads * c.d_dim * c.d_a_rank : -1;
         case MI355_HW_D_G2: return L.has_delta() && c.d_gate == MI355_HYB_GATE_SIGMOID_LR ? (int64_t)c.d_heads * c.d_vdim * c.d_g_rank : -1;
-        case MI355_HW_MLP_GATE_UP: if (c.mlp_kind == 3) return c.moe_shared_ff && !L.shared_merged() ? (int64_t)2 * c.moe_shared_ff * W : -1;
-                                   if (c.mlp_kind == 4) return (int64_t)c.mlp_ff * W;
-                                   return c.mlp_kind ? (int64_t)2 * c.mlp_ff * W : -1;
+        case MI355_HW_MLP_GATE_UP: if (c.mlp_kind == 3) return c.moe_shared_ff && !L.shared_merged() ? (int64_t)L.gate_up_rows() * c.moe_shared_ff * W : -1;
+                                   return c.mlp_kind ? (int64_t)L.gate_up_rows() * c.mlp_ff * W : -1;
         case MI355_HW_MLP_DOWN: if (c.mlp_kind == 3) return c.moe_shared_ff && !L.shared_merged() ? (int64_t)W * c.moe_shared_ff : -1;
                                 return c.mlp_kind ? (int64_t)W * c.mlp_ff : -1;
         default: return -1;
@@ -265,7 +290,7 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
 
 Weight* slot_of(HModel* m, int layer, int which) {
     if (layer < 0) return which == MI355_HW_EMBED ? &m->embed : which == MI355_HW_FINAL_NORM ? &m->final_norm : which == MI355_HW_HEAD ? &m->head :
-                          which == MI355_HW_SIDE_TABLE ? &m->side_table : nullptr;
+                          which == MI355_HW_SIDE_TABLE ? &m->side_table : which == MI355_HW_BIGRAM ? &m->bigram : nullptr;
     if (layer >= (int)m->layers.size() || which < MI355_HW_NORM1 || which >= MI355_HW_COUNT) return nullptr;
     return &m->layers[layer].w[which];
 }
@@ -294,7 +319,16 @@ template <typename T> int grow(T*& p, size_t bytes) {
     return 0;
 }
 
-int ensure_capacity(HModel* m, int T, int n_out) {
+int ensure_capacity(HModel* m, int T, int n_out, int n_seqs) {
+    int64_t pieces = 0;
+    for (const HLayer& L : m->layers)
+        if (L.is_decay()) pieces = std::max(pieces, mi355_hyb_decay_attention_scratch(T, n_seqs, L.c.d_heads, L.c.d_dim, L.c.d_vdim));
+    if (pieces > m->cap_pieces) {
+        HHIP(hipDeviceSynchronize());
+        drop_graphs(m);
+        HCHECK(grow(m->pieces, (size_t)pieces * 4));
+        m->cap_pieces = pieces;
+    }
     if (T > m->cap_t) {
         const size_t t = (size_t)T, W = (size_t)m->cfg.width;
         HHIP(hipDeviceSynchronize());
@@ -315,6 +349,8 @@ int ensure_capacity(HModel* m, int T, int n_out) {
         HCHECK(grow(m->att, t * (size_t)m->max_att * m->esize()));
         HCHECK(grow(m->tok_seq, t * 4));
         if (m->need_pre) HCHECK(grow(m->pre, t * W * m->esize()));
+        if (m->cfg.residual_form == 4) HCHECK(grow(m->streams, t * W * m->cfg.streams * 4));
+        if (m->cfg.bigram_buckets) HCHECK(grow(m->bigram_rows, t * 4));
         if (m->cfg.residual_form == 3) HCHECK(grow(m->y2, t * W * 4));
         if (m->need_hf) HCHECK(grow(m->hf, t * W * 4));
         if (m->need_xs) HCHECK(grow(m->xs, (m->layers.size() + 1) * t * W * 4));
@@ -374,7 +410,10 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
         const mi355_hybrid_layer& c = layers[i];
         if (c.side_dim && c.side_col + c.side_dim > cfg->side_cols) return nullptr;
         if (c.depth_terms && c.depth_terms != i + 2) return nullptr;
-        if (c.mlp_kind == 4 && cfg->residual_form != 3) return nullptr;
+        if (c.mlp_kind == 4 && cfg->residual_form != 3 && cfg->residual_form != 4) return nullptr;
+        if ((c.mlp_kind == 5 || c.moe_relu2 || c.moe_bias || c.moe_shared_plain || c.mixer == MI355_HYB_MIX_DECAY) && cfg->residual_form != 4) return nullptr;
+        if (cfg->residual_form == 4 && (c.in_conv || c.side_dim || c.depth_terms || c.mlp_kind == 1 || c.mlp_kind == 2)) return nullptr;
+        if (cfg->residual_form == 4 && c.mlp_kind == 3 && (!c.moe_relu2 || (c.moe_shared_ff && !c.moe_shared_plain))) return nullptr;
         if (cfg->residual_form == 3 && (c.in_conv || c.share_with || c.moe_shared_ff || c.mlp_kind == 1 || c.mlp_kind == 2)) return nullptr;
         if (c.kv_from) {                                            // the lender: an earlier latent layer with pages of its own and the same row
             if (c.kv_from > i) return nullptr;
@@ -382,12 +421,15 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
             if (b.mixer != MI355_HYB_MIX_LATENT || b.kv_from || b.a_kv_rank != c.a_kv_rank || b.a_rot_dim != c.a_rot_dim) return nullptr;
         }
     }
-    if (cfg->residual_form < 0 || cfg->residual_form > 3 || cfg->norm_groups < 0 || (cfg->norm_groups > 1 && cfg->width % cfg->norm_groups)) return nullptr;
+    if (cfg->residual_form == 4 && (cfg->streams < 1 || cfg->streams > 16 || cfg->width > 12288 || cfg->norm_groups > 1)) return nullptr;
+    if (cfg->residual_form != 4 && (cfg->streams || cfg->bigram_buckets)) return nullptr;
+    if (cfg->bigram_buckets < 0 || cfg->bigram_mul_prev < 0 || cfg->bigram_mul_cur < 0) return nullptr;
+    if (cfg->residual_form < 0 || cfg->residual_form > 4 || cfg->norm_groups < 0 || (cfg->norm_groups > 1 && cfg->width % cfg->norm_groups)) return nullptr;
     for (int i = 0; i < cfg->n_layers; ++i)                        // the experts' outputs are combined in front of an output norm
-        if (layers[i].mlp_kind == 3 && (cfg->residual_form == 1 || (cfg->residual_form != 3 && cfg->width > 4096))) return nullptr;
+        if (layers[i].mlp_kind == 3 && (cfg->residual_form == 1 || (cfg->residual_form < 3 && cfg->width > 4096))) return nullptr;
     HModel* m = new HModel();
     m->cfg = *cfg;
-    m->need_pre = cfg->residual_form == 2 || cfg->residual_form == 3;
+    m->need_pre = cfg->residual_form >= 2;
     m->layers.resize(cfg->n_layers);
     int64_t off = 0;
     for (int i = 0; i < cfg->n_layers; ++i) {
@@ -410,9 +452,15 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
             L.conv_off = off; off += (int64_t)L.ssd_channels() * (c.d_conv - 1);
             L.state_off = off; off += (int64_t)c.d_heads * c.d_dim * c.d_vdim;
         }
+        if (L.is_decay()) {
+            L.out_k = L.ssd_inner();
+            m->max_mix = std::max(m->max_mix, L.out_k);
+            m->max_o = std::max(m->max_o, L.ssd_inner());
+            L.state_off = off; off += (int64_t)c.d_heads * c.d_dim * c.d_vdim;
+        }
         if (c.side_dim) m->max_side = std::max(m->max_side, c.side_dim);
         if (c.depth_terms) m->need_xs = true;
-        if (c.mlp_kind == 3 && cfg->residual_form == 3 && cfg->dtype == MI355_DTYPE_BF16) m->need_hf = true;
+        if (c.mlp_kind == 3 && cfg->residual_form >= 3 && cfg->dtype == MI355_DTYPE_BF16) m->need_hf = true;
         if (L.is_latent() && c.a_q_rank) {
             m->max_q_rank = std::max(m->max_q_rank, c.a_q_rank);
             m->max_aux2 = std::max(m->max_aux2, c.a_heads * (c.a_dim + c.a_rot_dim));
@@ -446,6 +494,7 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
             m->max_ff = std::max(m->max_ff, c.moe_shared_ff);
         } else if (c.mlp_kind) m->max_ff = std::max(m->max_ff, c.mlp_ff);
     }
+    if (cfg->bigram_buckets) { m->bigram_off = off; ++off; }             // the previous token
     m->slot_floats = std::max<int64_t>(off, 1);
     return m;
 }
@@ -461,7 +510,8 @@ void mi355_hybrid_destroy(void* mp) {
     }
     for (void* p : {m->embed.p, m->final_norm.p, m->head.p, (void*)m->state, (void*)m->prep, (void*)m->x, (void*)m->proj, (void*)m->aux1, (void*)m->aux2,
                     (void*)m->conv, (void*)m->o, (void*)m->y, (void*)m->gu, m->xcopy, m->q, m->mix, m->act, m->xn, m->att, (void*)m->tok_seq,
-                    m->pre, m->moe_act, (void*)m->y2, (void*)m->hf, (void*)m->xs, (void*)m->side_g, m->side_a, m->cq, m->side_table.p, (void*)m->moe_gu, (void*)m->moe_y, (void*)m->moe_wts, (void*)m->moe_sgate, (void*)m->moe_ids,
+                    m->pre, m->moe_act, (void*)m->y2, (void*)m->hf, (void*)m->xs, (void*)m->side_g, m->side_a, m->cq, m->side_table.p,
+                    (void*)m->streams, (void*)m->pieces, (void*)m->bigram_rows, m->bigram.p, (void*)m->moe_gu, (void*)m->moe_y, (void*)m->moe_wts, (void*)m->moe_sgate, (void*)m->moe_ids,
                     (void*)m->moe_pos, (void*)m->moe_row_token, (void*)m->moe_table})
         if (p) (void)hipFree(p);
     delete m;
@@ -478,6 +528,18 @@ int mi355_hybrid_set_weight(void* mp, int32_t layer, int32_t which, const uint16
     if (rc == 0) rc = (int)hipDeviceSynchronize();
     (void)hipFree(tmp);
     return rc;
+}
+
+int mi355_hybrid_set_weight_f32(void* mp, int32_t layer, int32_t which, const float* host, int64_t n) {
+    HModel* m = static_cast<HModel*>(mp);
+    if (!m || !host || n <= 0) return -1;
+    Weight* w = slot_of(m, layer, which);
+    if (!w || is_matrix(which) || n != expected_elems(m, layer, which)) return -2;
+    HHIP(hipDeviceSynchronize());
+    drop_graphs(m);
+    HCHECK(grow(w->p, (size_t)n * 4));
+    w->n = n;
+    return (int)hipMemcpy(w->p, host, (size_t)n * 4, hipMemcpyHostToDevice);
 }
 
 int mi355_hybrid_set_weight_dev(void* mp, int32_t layer, int32_t which, const uint16_t* dev_bf16, int64_t n, int64_t stream) {
@@ -544,7 +606,8 @@ static int forward_check(HModel* m, const uint32_t* tokens, const int64_t* posit
                          int32_t max_blocks, int32_t max_context_len, float* logits) {
     if (!m || !tokens || !positions || !slot_mapping || !block_tables || !context_lens || !cu_seqlens_q || !state_slots) return -1;
     if (num_seqs <= 0 || T <= 0 || n_out < 0 || (n_out > 0 && (!out_rows || !logits)) || max_blocks <= 0) return -1;
-    if (!m->state || !m->embed.p || !m->final_norm.p || (!m->head.p && !m->cfg.tie_head) || (m->cfg.side_cols > 0 && !m->side_table.p)) return -3;
+    if (!m->state || !m->embed.p || !m->final_norm.p || (!m->head.p && !m->cfg.tie_head) || (m->cfg.side_cols > 0 && !m->side_table.p) ||
+        (m->cfg.bigram_buckets > 0 && !m->bigram.p)) return -3;
     if ((int64_t)max_blocks * m->cfg.block_size < max_context_len) return -4;
     for (const HLayer& L : m->layers) {
         const HLayer& WL = L.c.share_with ? m->layers[L.c.share_with - 1] : L;
@@ -556,7 +619,7 @@ static int forward_check(HModel* m, const uint32_t* tokens, const int64_t* posit
         }
         if (L.uses_pages() && (!L.k_pages || (L.rotates() && WL.n_pos < max_context_len))) return -4;
     }
-    return ensure_capacity(m, T, n_out);
+    return ensure_capacity(m, T, n_out, num_seqs);
 }
 
 static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* positions, const int64_t* slot_mapping,
@@ -568,12 +631,41 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
     const bool bf = m->bf16();
     const bool sandwich = m->cfg.residual_form == 2;                // a norm in front of every sublayer: nothing reads a copy of x
     const bool parallel = m->cfg.residual_form == 3;                // one norm per layer, both sublayers read it
-    void* xcopy = (bf && !sandwich && !parallel) ? m->xcopy : nullptr;
-    void* xin = (sandwich || parallel) ? m->pre : (bf ? m->xcopy : (void*)m->x);  // what the sublayers' first product reads
+    const bool copies = m->cfg.residual_form == 4;                  // several residual streams, a norm in front of every sublayer
+    void* xcopy = (bf && !sandwich && !parallel && !copies) ? m->xcopy : nullptr;
+    void* xin = (sandwich || parallel || copies) ? m->pre : (bf ? m->xcopy : (void*)m->x);  // what the sublayers' first product reads
     const int xin_dt = bf ? MI355_DTYPE_BF16 : MI355_DTYPE_F32;
     const int64_t TW = (int64_t)T * W;
     HCHECK(mi355_hyb_token_seq(m->tok_seq, cu_seqlens_q, num_seqs, stream));
-    if (m->cfg.embed_scale != 0.f && m->cfg.embed_scale != 1.f)
+    // form 4: what one sublayer hands to the next -- the copies behind sublayer (li, q) (q = 0: in front of the first one) with its output
+    // y (and, where its experts ran, their rows), the next sublayer's input and norm; behind the last one the sum of the copies
+    auto stream_step = [&](size_t li, int q, const float* y, bool experts, int top) -> int {
+        const size_t n = m->layers.size();
+        const size_t nl = (q == 1 && m->layers[li].c.mlp_kind) ? li : (q == 0 ? 0 : li + 1);
+        const int nq = (q == 1 && m->layers[li].c.mlp_kind) ? 2 : 1;
+        auto weights = [&](size_t l, int which) {
+            const int sw = m->layers[l].c.share_with;
+            return static_cast<const float*>(m->layers[sw ? sw - 1 : l].w[which].p);
+        };
+        const bool more = nl < n, layer_end = q > 0 && nl != li;
+        const float* norm = more ? weights(nl, nq == 1 ? MI355_HW_NORM1 : MI355_HW_NORM2) : nullptr;
+        const bool routes = more && nq == 2 && m->layers[nl].c.mlp_kind == 3 && bf;
+        return mi355_hyb_stream_step(m->streams, y, experts ? m->moe_y : nullptr, m->moe_pos, m->moe_wts, top,
+                                     q ? weights(li, q == 1 ? MI355_HW_HC1_MIX : MI355_HW_HC2_MIX) : nullptr,
+                                     q ? weights(li, q == 1 ? MI355_HW_HC1_OUT : MI355_HW_HC2_OUT) : nullptr,
+                                     (!more || (layer_trace && layer_end)) ? m->x : nullptr,
+                                     more ? weights(nl, nq == 1 ? MI355_HW_HC1_IN : MI355_HW_HC2_IN) : nullptr, norm, m->pre, dt,
+                                     routes ? m->hf : nullptr, T, m->cfg.streams, W, eps, stream);
+    };
+    if (copies) {
+        if (m->cfg.bigram_buckets)
+            HCHECK(mi355_hyb_bigram_rows(m->bigram_rows, reinterpret_cast<int32_t*>(m->state + m->bigram_off), m->slot_floats, tokens, context_lens,
+                                         cu_seqlens_q, state_slots, num_seqs, T, m->cfg.bigram_buckets, m->cfg.bigram_mul_prev,
+                                         m->cfg.bigram_mul_cur, stream));
+        HCHECK(mi355_hyb_embed_streams(m->streams, m->embed.p, m->bigram.p, m->bigram_rows, tokens, T, m->cfg.streams, W, m->cfg.vocab,
+                                       m->cfg.embed_scale != 0.f ? m->cfg.embed_scale : 1.f, dt, stream));
+        HCHECK(stream_step(0, 0, nullptr, false, 0));
+    } else if (m->cfg.embed_scale != 0.f && m->cfg.embed_scale != 1.f)
         HCHECK(mi355_hyb_embed_scaled(m->x, m->embed.p, tokens, T, W, m->cfg.vocab, m->cfg.embed_scale, dt, stream));
     else
         HCHECK(mi355_hyb_embed(m->x, xcopy, m->embed.p, tokens, T, W, m->cfg.vocab, dt, stream));
@@ -613,7 +705,9 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             HCHECK(mi355_hyb_pre_norm_ex(m->pre, dt, (c.mlp_kind == 3 && bf) ? m->hf : nullptr, m->x, W, f(MI355_HW_NORM1), T, W, m->cfg.norm_kind,
                                          eps, stream));
         }
-        HCHECK(mi355_hyb_linear(m->proj, ldp, min_, xin_dt, W, WL.w[MI355_HW_IN_PROJ].p, f(MI355_HW_IN_BIAS), T, L.in_rows, W, dt, stream));
+        // (constant-decay attention: silu on q, k, v, in the epilogue)
+        HCHECK(mi355_hyb_linear_act(m->proj, MI355_DTYPE_F32, ldp, min_, xin_dt, W, WL.w[MI355_HW_IN_PROJ].p, f(MI355_HW_IN_BIAS), T, L.in_rows, W,
+                                    L.is_decay() ? MI355_HYB_ACT_SILU : MI355_HYB_ACT_NONE, L.is_decay() ? L.off[P_G] : 0, dt, stream));
         int mix_col = 0;
         if (L.has_attn()) {
             const int norm_mode = c.a_qk_norm ? (c.a_norm_after_rot ? 2 : 1) : 0;
@@ -622,10 +716,11 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
                                              WL.cos_t, WL.sin_t, positions, slot_mapping, T, c.a_heads, c.a_kv_heads, c.a_dim, c.a_vdim,
                                              c.a_rot_dims, c.a_rot_interleaved, norm_mode, c.a_head_temp ? f(MI355_HW_A_TEMP) : nullptr, eps,
                                              dt, stream));
-            HCHECK(mi355_hyb_masked_attention(m->mix, dt, L.out_k, 0, m->q, L.k_pages, L.v_pages, block_tables, context_lens, cu_seqlens_q,
-                                              m->tok_seq, c.a_has_sink ? f(MI355_HW_A_SINK) : nullptr, num_seqs, T, c.a_heads,
-                                              c.a_kv_heads, c.a_dim, c.a_vdim, m->cfg.block_size, max_blocks, c.a_window, c.a_keep_first,
-                                              c.a_scale, c.mixer == MI355_HYB_MIX_PARALLEL ? c.a_out_scale : 1.f, 0, 0, 0.f, 0, dt, stream));
+            HCHECK(mi355_hyb_attention(m->mix, dt, L.out_k, 0, m->q, L.k_pages, L.v_pages, block_tables, context_lens, cu_seqlens_q,
+                                       m->tok_seq, c.a_has_sink ? f(MI355_HW_A_SINK) : nullptr, nullptr, num_seqs, T, c.a_heads,
+                                       c.a_kv_heads, c.a_dim, c.a_vdim, m->cfg.block_size, max_blocks, c.a_mask_kind, c.a_window,
+                                       c.a_keep_first, c.a_scale, c.mixer == MI355_HYB_MIX_PARALLEL ? c.a_out_scale : 1.f, 0, 0, 0.f, 0, dt,
+                                       stream));
             mix_col = c.a_heads * c.a_vdim;
         }
         if (L.is_latent()) {
@@ -693,6 +788,14 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             HCHECK(mi355_hyb_gate_group_norm(m->mix, dt, m->o, m->proj + L.off[P_G], ldp, f(MI355_HW_D_NORM), T, L.ssd_inner(), c.d_norm_groups,
                                              eps, stream));
         }
+        if (L.is_decay()) {
+            // q | k | v (behind silu) into the recurrence over the state slot, the norm over all heads, the gate
+            const bool by_pieces = mi355_hyb_decay_attention_scratch(T, num_seqs, c.d_heads, c.d_dim, c.d_vdim) > 0;
+            HCHECK(mi355_hyb_decay_attention(m->o, m->state + L.state_off, m->slot_floats, m->proj, ldp, L.off[P_DQ], L.off[P_DK], L.off[P_DV],
+                                             f(MI355_HW_D_DECAY), context_lens, cu_seqlens_q, state_slots, num_seqs, T, c.d_heads, c.d_dim,
+                                             c.d_vdim, by_pieces ? m->pieces : nullptr, stream));
+            HCHECK(mi355_hyb_norm_sigmoid_gate(m->mix, dt, m->o, m->proj + L.off[P_G], ldp, f(MI355_HW_D_NORM), T, L.ssd_inner(), 1, eps, stream));
+        }
         if (L.has_delta()) {
             const int C = L.conv_channels();
             float* conv_state = m->state + L.conv_off;
@@ -729,7 +832,38 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             return mi355_hyb_norm_add(m->x, xcopy, m->y, W, f(norm_slot), T, W, eps, stream);
         };
         HCHECK(mi355_hyb_linear(m->y, W, m->mix, dt, L.out_k, WL.w[MI355_HW_OUT_PROJ].p, nullptr, T, W, L.out_k, dt, stream));
-        if (parallel) {
+        if (copies) {
+            HCHECK(stream_step(li, 1, m->y, false, 0));
+            if (c.mlp_kind == 3) {
+                // router on the norm's f32 output, the (token, expert) pairs grouped, one grouped product per matrix of the experts with the
+                // activation in the first one's epilogue; the shared expert as one more group (of the experts' size) or as dense products
+                const bool merged = L.shared_merged();
+                const int E = c.moe_experts + merged, K = c.moe_top + merged, ff = c.mlp_ff, fs = merged ? 0 : c.moe_shared_ff, pairs = T * K;
+                HCHECK(mi355_hyb_moe_route_biased(m->moe_ids, m->moe_wts, nullptr, nullptr, dt, bf ? m->hf : static_cast<const float*>(m->pre), nullptr,
+                                                  f(MI355_HW_MOE_ROUTER), c.moe_bias ? f(MI355_HW_MOE_BIAS) : nullptr, f(MI355_HW_MOE_CORRECTION),
+                                                  nullptr, T, W, c.moe_experts, c.moe_top, c.moe_scale != 0.f ? c.moe_scale : 1.f, eps, merged,
+                                                  c.moe_sigmoid ? 1 : (c.moe_bias ? 2 : 0), c.moe_groups, c.moe_keep_groups,
+                                                  c.moe_bias || c.moe_normalise, stream));
+                const int bm = std::min(mi355_hyb_moe_block_rows(pairs, E, ff, W, dt), mi355_hyb_moe_block_rows(pairs, E, W, ff, dt));
+                const int nb = (pairs + bm - 1) / bm + E;
+                HCHECK(mi355_hyb_moe_group(m->moe_pos, m->moe_row_token, m->moe_table, m->moe_ids, pairs, K, E, bm, nb, stream));
+                HCHECK(mi355_hyb_linear_grouped_act(m->moe_act, dt, ff, xin, xin_dt, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)ff * W,
+                                                    m->moe_table, bm, nb, ff, W, MI355_HYB_ACT_RELU2, dt, stream));
+                HCHECK(mi355_hyb_linear_grouped(m->moe_y, W, m->moe_act, dt, ff, nullptr, WL.w[MI355_HW_MOE_DOWN].p, (int64_t)W * ff, m->moe_table, bm,
+                                                nb, W, ff, dt, stream));
+                if (fs) {
+                    HCHECK(mi355_hyb_linear_act(m->act, dt, fs, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, fs, W, MI355_HYB_ACT_RELU2, fs, dt,
+                                                stream));
+                    HCHECK(mi355_hyb_linear(m->y, W, m->act, dt, fs, WL.w[MI355_HW_MLP_DOWN].p, nullptr, T, W, fs, dt, stream));
+                }
+                HCHECK(stream_step(li, 2, fs ? m->y : nullptr, true, K));
+            } else if (c.mlp_kind) {
+                HCHECK(mi355_hyb_linear_act(m->act, dt, c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, c.mlp_ff, W,
+                                            c.mlp_kind == 5 ? MI355_HYB_ACT_GELU : MI355_HYB_ACT_RELU2, c.mlp_ff, dt, stream));
+                HCHECK(mi355_hyb_linear(m->y, W, m->act, dt, c.mlp_ff, WL.w[MI355_HW_MLP_DOWN].p, nullptr, T, W, c.mlp_ff, dt, stream));
+                HCHECK(stream_step(li, 2, m->y, false, 0));
+            }
+        } else if (parallel) {
             // x <- x + mixer(h) + ff(h): the feed-forward reads the same h (m->pre) the mixer's projections read
             if (c.mlp_kind == 3) {
                 const int E = c.moe_experts, K = c.moe_top, ff = c.mlp_ff, pairs = T * K;

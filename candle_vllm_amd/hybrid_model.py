@@ -1,7 +1,8 @@
 """Python harness over the `mi355_hybrid_*` handle (include/mi355_hybrid.h): layer-list models whose layers mix tokens by
-sliding-window attention with a sink, a gated delta rule, a minGRU, attention and delta rule side by side, latent attention, or
-attention behind a short convolution with mixed head weights, or a state-space mixer, with dense or mixture-of-experts
-feed-forwards.  The Sogodra, Vivazen, Kerolorn and Sabolorn designs are read here: a design's
+sliding-window attention with a sink, a gated delta rule, a minGRU, attention and delta rule side by side, latent attention,
+attention behind a short convolution with mixed head weights, a state-space mixer, chunked attention or linear attention with a
+constant decay, with dense or mixture-of-experts feed-forwards.  The Sogodra, Vivazen, Kerolorn, Sabolorn and Tosivik designs are read
+here: a design's
 config.json (`architecture`, `layers`, `norm`, `vocab`, `width`, ...) becomes the C structs, its tensors are concatenated into the
 host layer's slots.  No CPU fallback; torch only holds device buffers."""
 import ctypes
@@ -16,15 +17,16 @@ import torch
 from ._lib import lib, HybridConfig, HybridLayer, RopeScaling
 
 DT_F32, DT_BF16 = 0, 2
-MIX_PARALLEL, MIX_MINGRU, MIX_DELTA, MIX_ATTENTION, MIX_LATENT, MIX_CONV_ATTENTION, MIX_SSD = 0, 1, 2, 3, 4, 5, 6
+MIX_PARALLEL, MIX_MINGRU, MIX_DELTA, MIX_ATTENTION, MIX_LATENT, MIX_CONV_ATTENTION, MIX_SSD, MIX_DECAY = 0, 1, 2, 3, 4, 5, 6, 7
 GATE_SILU, GATE_SIGMOID_LR = 0, 1
 ROPE_DEFAULT, ROPE_LLAMA3, ROPE_YARN = 0, 2, 4
 (HW_EMBED, HW_FINAL_NORM, HW_HEAD, HW_NORM1, HW_NORM2, HW_IN_PROJ, HW_IN_BIAS, HW_OUT_PROJ, HW_A_QNORM, HW_A_KNORM, HW_A_SINK, HW_D_CONV,
  HW_D_A_LOG, HW_D_DT_BIAS, HW_D_NORM, HW_D_A2, HW_D_G2, HW_MLP_GATE_UP, HW_MLP_DOWN, HW_A_CONV, HW_A_TALK, HW_L_UKT, HW_L_UV,
  HW_L_CNORM, HW_PRE_NORM1, HW_PRE_NORM2, HW_IN_CONV, HW_A_TEMP, HW_MOE_ROUTER, HW_MOE_CORRECTION, HW_MOE_GATE_UP,
  HW_MOE_DOWN, HW_D_SKIP, HW_CONV_BIAS, HW_A_DIST, HW_L_QNORM, HW_L_UQ, HW_SIDE_GATE, HW_SIDE_PROJ, HW_SIDE_NORM, HW_DEPTH_W,
- HW_SIDE_TABLE) = range(42)
-MLP_CLAMPED_GLU, MLP_GELU_GLU, MLP_MOE, MLP_RELU2 = 1, 2, 3, 4
+ HW_SIDE_TABLE, HW_HC1_IN, HW_HC1_OUT, HW_HC1_MIX, HW_HC2_IN, HW_HC2_OUT, HW_HC2_MIX, HW_MOE_BIAS, HW_D_DECAY, HW_BIGRAM) = range(51)
+MLP_CLAMPED_GLU, MLP_GELU_GLU, MLP_MOE, MLP_RELU2, MLP_GELU = 1, 2, 3, 4, 5
+MASK_SLIDING, MASK_CHUNKED = 0, 1
 NORM_RMS, NORM_LAYER = 0, 1
 
 # constants the Sogodra design fixes
@@ -193,6 +195,16 @@ class SogodraSpec:
         return L, slots, rope
 
 
+def weights_layer(entries, i):
+    """the layer whose tensors layer i runs on (itself without `weights_of`)"""
+    src = i
+    for _ in entries:
+        if entries[src].get("weights_of") is None:
+            return src
+        src = int(entries[src]["weights_of"])
+    raise ValueError(f"layer {i}: weights_of runs in a circle")
+
+
 class VivazenSpec:
     """config.json of a Vivazen model -> layer structs + the tensor names behind every weight slot.  The design: the norm sits behind
     the residual sum, x <- N(alpha x + sub(x)), N = RMS norm over `norm.groups` parts of the vector; layers are latent attention
@@ -213,11 +225,7 @@ class VivazenSpec:
         self.layers, self.slots, self.rope = [], [], []
         entries = cfg["layers"]
         for i, lc in enumerate(entries):
-            src = i
-            while "weights_of" in entries[src]:                 # the layer whose tensors this one runs on
-                src = int(entries[src]["weights_of"])
-                if src == i:
-                    raise ValueError(f"layer {i}: weights_of runs in a circle")
+            src = weights_layer(entries, i)
             L, slots, rope = self._layer("l%d." % src, lc, shapes)
             if src != i:
                 L.share_with, slots, rope = src + 1, {}, None
@@ -470,7 +478,109 @@ class SabolornSpec:
         return L, slots, rope
 
 
-SPECS = {"Sogodra": SogodraSpec, "Vivazen": VivazenSpec, "Kerolorn": KerolornSpec, "Sabolorn": SabolornSpec}       # config.json `architecture` -> its reader
+class Constants:
+    """a slot entry: f32 constants of the configuration (the slot takes them as they are, not rounded to bf16)"""
+
+    def __init__(self, values):
+        self.values = np.asarray(values, np.float32).reshape(-1)
+
+
+class TosivikSpec:
+    """config.json of a Tosivik model -> layer structs + the tensor names behind every weight slot.  The design: the residual stream is
+    `streams` copies; a sublayer reads one learned mixture of them (RMS norm in front) and the copies are mixed again when its output
+    is added (`hc1` / `hc2`).  The embedding adds a row picked by the pair (previous token, token).  Mixers: attention inside chunks of
+    positions whose values are the unrotated keys (rotate-half pairs with yarn), linear attention with a constant decay per head behind
+    a norm over all heads and a sigmoid gate (`lightning`).  Feed-forward: gelu without a gate, or relu^2 experts with a biased router
+    (softmax over the chosen logits) and a plain shared expert.  A layer with `weights_of` runs on that layer's tensors with pages and
+    state of its own.  A config without `streams` is the plain pre-norm form: one copy, every weight of the mixing 1."""
+    residual_form, resid_alpha, norm_groups = 4, 1.0, 1
+    rope_scaling = staticmethod(yarn_scaling)
+
+    def __init__(self, cfg, shapes):
+        if cfg.get("architecture") != "Tosivik":
+            raise ValueError("not a Tosivik config")
+        self.cfg = cfg
+        self.width, self.vocab = int(cfg["width"]), int(cfg["vocab"])
+        self.eps = float(cfg["norm"]["eps"])
+        self.streams = int(cfg.get("streams") or 1)
+        self.logit_softcap = float(cfg.get("logit_softcap") or 0.0)
+        emb = cfg.get("embedding") or {}
+        self.embed_scale = float(emb.get("scale", 1.0))
+        b = emb.get("bigram")
+        self.bigram_buckets = int(b["buckets"]) if b else 0
+        self.bigram_mul_prev, self.bigram_mul_cur = (int(b["mul_prev"]), int(b["mul_cur"])) if b else (0, 0)
+        self.layers, self.slots, self.rope = [], [], []
+        entries = cfg["layers"]
+        for i, lc in enumerate(entries):
+            src = weights_layer(entries, i)
+            L, slots, rope = self._layer("l%d." % src, lc, shapes)
+            if src != i:
+                L.share_with, slots, rope = src + 1, {}, None
+            self.layers.append(L)
+            self.slots.append(slots)
+            self.rope.append(rope)
+
+    def globals_(self):
+        g = {HW_EMBED: "embed", HW_FINAL_NORM: "final.norm", HW_HEAD: "head"}
+        if self.bigram_buckets:
+            g[HW_BIGRAM] = "bigram"
+        return g
+
+    def _mixing(self, p, q, slots):
+        """the weights of the copies around sublayer q of the layer"""
+        hc = p + "hc%d." % q
+        names = (HW_HC1_IN, HW_HC1_OUT, HW_HC1_MIX) if q == 1 else (HW_HC2_IN, HW_HC2_OUT, HW_HC2_MIX)
+        for slot, n in zip(names, ("in", "out", "mix")):
+            slots[slot] = [hc + n] if self.cfg.get("streams") else [Ones(1)]
+
+    def _layer(self, p, lc, shapes):
+        L, slots, rope = HybridLayer(), {HW_NORM1: [p + "norm1"]}, None
+        c, kind, q = lc["mixer"], lc["type"], p + "mix."
+        self._mixing(p, 1, slots)
+        if kind == "attention":
+            L.mixer = MIX_ATTENTION
+            L.a_heads, L.a_kv_heads, L.a_dim, L.a_vdim = int(c["heads"]), int(c["kv_heads"]), int(c["dim"]), int(c["vdim"])
+            L.a_scale, L.a_out_scale, L.a_v_is_k = float(c["scale"]), 1.0, 1
+            L.a_window, L.a_mask_kind = (int(c["mask"]["size"]), MASK_CHUNKED) if c.get("mask") else (0, MASK_SLIDING)
+            rope = c.get("rot")
+            L.a_rot_dims = int(rope["dims"]) if rope else 0
+            slots[HW_IN_PROJ] = [q + "q", q + "k"]
+        elif kind == "lightning":
+            L.mixer = MIX_DECAY
+            L.d_heads, L.d_kv_heads, L.d_dim, L.d_vdim = int(c["heads"]), int(c["heads"]), int(c["dim"]), int(c["vdim"])
+            slots[HW_IN_PROJ], slots[HW_D_NORM] = [q + "q", q + "k", q + "v", q + "g"], [q + "norm"]
+            slots[HW_D_DECAY] = [Constants(np.broadcast_to(np.asarray(c["decay"], np.float64), (L.d_heads,)))]
+        else:
+            raise ValueError(f"layer type {kind!r} is not part of the design")
+        slots[HW_OUT_PROJ] = [q + "o"]
+        mlp = lc.get("mlp")
+        if mlp:
+            m = p + "mlp."
+            slots[HW_NORM2] = [p + "norm2"]
+            self._mixing(p, 2, slots)
+            if mlp.get("kind") == "dense":
+                L.mlp_kind, L.mlp_ff = MLP_GELU, int(mlp["ff"])
+                slots[HW_MLP_GATE_UP], slots[HW_MLP_DOWN] = [m + "up"], [m + "down"]
+            elif mlp.get("kind") == "moe":
+                r, shared = mlp["router"], mlp.get("shared")
+                L.mlp_kind, L.mlp_ff, L.moe_relu2, L.moe_bias, L.moe_shared_plain = MLP_MOE, int(mlp["expert"]["ff"]), 1, 1, 1
+                L.moe_experts, L.moe_top, L.moe_scale = int(r["experts"]), int(r["top"]), 1.0
+                L.moe_shared_ff = int(shared["ff"]) if shared else 0
+                slots[HW_MOE_ROUTER], slots[HW_MOE_BIAS] = [m + "router"], [m + "router.b"]
+                slots[HW_MOE_GATE_UP] = [m + "e%d.up" % e for e in range(L.moe_experts)]
+                slots[HW_MOE_DOWN] = [m + "e%d.down" % e for e in range(L.moe_experts)]
+                if shared and L.moe_shared_ff == L.mlp_ff:      # of the experts' size: one more matrix of the grouped products
+                    slots[HW_MOE_GATE_UP].append(m + "shared.up")
+                    slots[HW_MOE_DOWN].append(m + "shared.down")
+                elif shared:
+                    slots[HW_MLP_GATE_UP], slots[HW_MLP_DOWN] = [m + "shared.up"], [m + "shared.down"]
+            else:
+                raise ValueError(f"feed-forward kind {mlp.get('kind')!r} is not part of the design")
+        return L, slots, rope
+
+
+# config.json `architecture` -> its reader
+SPECS = {"Sogodra": SogodraSpec, "Vivazen": VivazenSpec, "Kerolorn": KerolornSpec, "Sabolorn": SabolornSpec, "Tosivik": TosivikSpec}
 
 
 class HybridModel:
@@ -487,7 +597,9 @@ class HybridModel:
                          residual_form=int(spec.residual_form), resid_alpha=float(spec.resid_alpha), norm_groups=int(spec.norm_groups),
                          logit_scale=float(getattr(spec, "logit_scale", 1.0)), norm_kind=int(getattr(spec, "norm_kind", NORM_RMS)),
                          embed_scale=float(getattr(spec, "embed_scale", 1.0)), logit_softcap=float(getattr(spec, "logit_softcap", 0.0)),
-                         tie_head=int(getattr(spec, "tie_head", 0)), side_cols=int(getattr(spec, "side_cols", 0)))
+                         tie_head=int(getattr(spec, "tie_head", 0)), side_cols=int(getattr(spec, "side_cols", 0)),
+                         streams=int(getattr(spec, "streams", 0)), bigram_buckets=int(getattr(spec, "bigram_buckets", 0)),
+                         bigram_mul_prev=int(getattr(spec, "bigram_mul_prev", 0)), bigram_mul_cur=int(getattr(spec, "bigram_mul_cur", 0)))
         self.h = lib.mi355_hybrid_create(ctypes.byref(c), self._layers)
         if not self.h:
             raise RuntimeError("mi355_hybrid_create refused the configuration")
@@ -540,6 +652,9 @@ class HybridModel:
                 elif which == HW_D_CONV:
                     mats = [np.asarray(bits[nm], np.uint16).reshape(shapes[nm]) for nm in names]
                     self._put(i, which, np.concatenate(mats, axis=0))
+                elif isinstance(names[0], Constants):
+                    v = np.ascontiguousarray(names[0].values)
+                    _check(lib.mi355_hybrid_set_weight_f32(self.h, i, which, v.ctypes.data, v.size), f"set_weight_f32 layer {i} slot {which}")
                 else:
                     self._put(i, which, np.concatenate([nm.bits(bits, shapes) if isinstance(nm, (HeadTranspose, Ones))
                                                         else np.asarray(bits[nm], np.uint16).reshape(-1) for nm in names]))

@@ -2,8 +2,9 @@
  * layer has -- sliding-window attention with a softmax sink, a gated delta rule (recurrent matrix state), a minGRU (recurrent vector
  * state), attention and delta rule side by side, latent attention (keys and values read off one cached latent vector per token), or
  * attention behind a short convolution whose heads' softmax weights are mixed -- and which feed-forward (dense gate/up forms or a
- * mixture of experts), or a state-space mixer with a scalar decay per head.  The Sogodra, Vivazen, Kerolorn and Sabolorn designs are
- * its users.
+ * mixture of experts), a state-space mixer with a scalar decay per head, or linear attention with one constant decay per head; the
+ * residual stream is one vector per token or several mixed copies of it.  The Sogodra, Vivazen, Kerolorn, Sabolorn and Tosivik designs
+ * are its users.
  *
  * What differs from the llama-family host layers (mi355_llama_*, mi355_dense_*):
  *   - the residual stream, norms, attention scores, decays, gates of a recurrence and the recurrent state are f32 in both dtypes;
@@ -37,6 +38,18 @@ extern "C" {
                                       step dt]; x, B, C pass a short causal convolution with bias and silu; per head S <- exp(-exp(a_log)
                                       dt) S + dt B x^T, y = S^T C + skip x; y silu(z), RMS norm in d_norm_groups parts, output projection.
                                       d_heads heads of d_vdim, state size d_dim, d_kv_heads groups of B / C, d_conv taps            */
+
+#define MI355_HYB_MIX_DECAY 7       /* linear attention with a constant decay per head: q, k, v = silu of their projections (d_heads heads of
+                                      d_dim | d_vdim, no sharing), S <- decay[h] S + k v^T, o = S^T q; RMS norm over all heads together,
+                                      times sigmoid(W_g h), output projection.  The decays are MI355_HW_D_DECAY                       */
+
+#define MI355_HYB_MASK_SLIDING 0    /* a query at position i sees keys j with 0 <= i - j < window                                      */
+#define MI355_HYB_MASK_CHUNKED 1    /* it sees keys j <= i with floor(i / window) = floor(j / window)                                  */
+
+#define MI355_HYB_ACT_NONE 0        /* activations in the epilogue of a product                                                        */
+#define MI355_HYB_ACT_SILU 1
+#define MI355_HYB_ACT_GELU 2        /* the tanh form                                                                                   */
+#define MI355_HYB_ACT_RELU2 3       /* relu(z)^2                                                                                       */
 
 #define MI355_HYB_GATE_SILU 0      /* output gate silu(W_g h), full rank                */
 #define MI355_HYB_GATE_SIGMOID_LR 1 /* output gate sigmoid(W_g2 (W_g1 h)), low rank     */
@@ -110,6 +123,15 @@ typedef struct mi355_hybrid_layer {
     int32_t side_col;
     int32_t depth_terms;           /* n > 0: behind the layer x <- sum_j w[j] X_j over the n earliest of (embedding output, results
                                       of the layers so far); n = layer index + 2 (MI355_HW_DEPTH_W [n])                        */
+    /* more switches of the plain attention mixers */
+    int32_t a_mask_kind;           /* MI355_HYB_MASK_*: what a_window means                                                  */
+    int32_t a_v_is_k;              /* no value projection: the cached value row is the key as projected, before the rotation
+                                      (a_vdim == a_dim); the v part of the input projection is its k part                    */
+    /* more forms of the feed-forward.  mlp_kind 5: dense without a gate, y = W_down gelu_tanh(W_up h) (up rows as in kind 4) */
+    int32_t moe_relu2;             /* kind 3: the experts (and the shared one) are y = W_down relu(W_up h)^2 without a gate; the
+                                      GATE_UP slots then hold [ff, width] up rows per expert                                 */
+    int32_t moe_bias;              /* kind 3: z = router . h + bias (MI355_HW_MOE_BIAS), softmax over the chosen logits only   */
+    int32_t moe_shared_plain;      /* kind 3: the shared expert is added as it is (no gate row in the router)                  */
 } mi355_hybrid_layer;
 
 typedef struct mi355_hybrid_config {
@@ -133,6 +155,15 @@ typedef struct mi355_hybrid_config {
     float logit_softcap;           /* > 0: logits <- cap tanh(logits / cap)                                                  */
     int32_t tie_head;              /* the logits are taken against the embedding table itself; MI355_HW_HEAD stays empty     */
     int32_t side_cols;             /* columns of the per-layer token table MI355_HW_SIDE_TABLE [vocab, side_cols] (0 = none) */
+    /* residual_form 4: the residual stream is `streams` copies X_i of the embedding output.  Every sublayer (norm in front:
+     * MI355_HW_NORM1 / 2) reads one mixture of them and writes to all: y = sub(norm(sum_i in[i] X_i)),
+     * X_j <- sum_i mix[i, j] X_i + out[j] y (MI355_HW_HC1_* in the mixer, _HC2_* in the feed-forward); the model's output is
+     * the sum of the copies                                                                                                  */
+    int32_t streams;
+    int32_t bigram_buckets;        /* > 0: the embedding also takes row (previous token mul_prev + token mul_cur) mod buckets of
+                                      MI355_HW_BIGRAM (row `buckets` at a sequence's first token); the previous token lives in
+                                      the state slot                                                                          */
+    int64_t bigram_mul_prev, bigram_mul_cur;
 } mi355_hybrid_config;
 
 /* weight slots: `layer` = -1 for the three global ones */
@@ -180,8 +211,17 @@ typedef struct mi355_hybrid_config {
 #define MI355_HW_SIDE_PROJ 38      /* [width, side_dim]                                                              */
 #define MI355_HW_SIDE_NORM 39      /* [width]                                                                        */
 #define MI355_HW_DEPTH_W 40        /* [depth_terms]                                                                  */
-#define MI355_HW_COUNT 41
 #define MI355_HW_SIDE_TABLE 41     /* global (layer -1): [vocab, side_cols]                                          */
+#define MI355_HW_HC1_IN 42         /* [streams]          residual form 4, mixer: what it reads of every copy         */
+#define MI355_HW_HC1_OUT 43        /* [streams]          how much of its output every copy takes                     */
+#define MI355_HW_HC1_MIX 44        /* [streams, streams] from copy i (row) to copy j                                 */
+#define MI355_HW_HC2_IN 45         /* the same three of the feed-forward                                             */
+#define MI355_HW_HC2_OUT 46
+#define MI355_HW_HC2_MIX 47
+#define MI355_HW_MOE_BIAS 48       /* [experts]                                                                      */
+#define MI355_HW_D_DECAY 49        /* [heads] f32, mi355_hybrid_set_weight_f32                                       */
+#define MI355_HW_COUNT 50
+#define MI355_HW_BIGRAM 50         /* global (layer -1): [bigram_buckets + 1, width]                                 */
 
 void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_layer* layers);
 void mi355_hybrid_destroy(void* model);
@@ -192,6 +232,8 @@ void mi355_hybrid_destroy(void* model);
 int32_t mi355_hybrid_in_proj_rows(const mi355_hybrid_layer* layer, int32_t* offsets);
 /* HOST bf16 bits (a checkpoint tensor), n elements; converted to the storage type of the slot */
 int mi355_hybrid_set_weight(void* model, int32_t layer, int32_t which, const uint16_t* host_bf16, int64_t n);
+/* HOST f32 values of a slot that is kept in f32 (constants of a configuration that bf16 cannot hold) */
+int mi355_hybrid_set_weight_f32(void* model, int32_t layer, int32_t which, const float* host, int64_t n);
 /* DEVICE bf16 bits (synthetic weights of a benchmark) */
 int mi355_hybrid_set_weight_dev(void* model, int32_t layer, int32_t which, const uint16_t* dev_bf16, int64_t n, int64_t stream);
 /* HOST f32 [n_positions, a_rot_dims / 2] cos and sin of a layer's rotary angles (mi355_rope_tables builds them) */
@@ -437,6 +479,58 @@ int mi355_hyb_moe_route_ex(int32_t* expert_ids, float* weights, float* shared_ga
                            const float* norm_w, const float* router, const float* correction, const float* gate_row, int32_t num_tokens,
                            int32_t width, int32_t experts, int32_t top, float scale, float eps, int32_t append_shared,
                            int32_t sigmoid_scores, int32_t groups, int32_t keep_groups, int32_t normalise, int64_t stream);
+/* ---- mechanisms of the designs with several residual streams */
+/* mi355_hyb_linear with an activation in the epilogue: columns < act_cols pass MI355_HYB_ACT_*; out (dt_out) [T, ldo] */
+int mi355_hyb_linear_act(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const void* w, const float* bias,
+                         int32_t num_tokens, int32_t n, int32_t k, int32_t act, int32_t act_cols, int32_t dtype, int64_t stream);
+/* mi355_hyb_linear_grouped with an activation on every column and the output type as an argument */
+int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const int32_t* row_token,
+                                 const void* w, int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t n,
+                                 int32_t k, int32_t act, int32_t dtype, int64_t stream);
+/* mi355_hyb_biased_attention with the kind of mask (MI355_HYB_MASK_*; the window is the chunk's size for the chunked one) */
+int mi355_hyb_attention(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const void* q, const void* k_pages, const void* v_pages,
+                        const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_seqlens_q, const int32_t* token_seq,
+                        const float* sink, const float* dist, int32_t num_seqs, int32_t num_tokens, int32_t heads, int32_t kv_heads, int32_t dim,
+                        int32_t vdim, int32_t block_size, int32_t max_blocks, int32_t mask_kind, int32_t window, int32_t keep_first,
+                        float scale, float out_scale, int32_t k_ld, int32_t v_ld, float softcap, int32_t cross_values, int32_t dtype,
+                        int64_t stream);
+/* mi355_hyb_moe_route_ex with a bias on the logits (router_bias f32 [experts] or NULL) and one more kind of scores: score_kind 0 =
+ * softmax, 1 = sigmoid, 2 = the experts are chosen by their logits (+ correction) and, with normalise, weighted by the softmax over the
+ * chosen logits.  append_shared without a gate_row: the appended pair has weight 1 */
+int mi355_hyb_moe_route_biased(int32_t* expert_ids, float* weights, float* shared_gate, void* xn, int32_t out_dtype, const float* x,
+                               const float* norm_w, const float* router, const float* router_bias, const float* correction, const float* gate_row,
+                               int32_t num_tokens, int32_t width, int32_t experts, int32_t top, float scale, float eps, int32_t append_shared,
+                               int32_t score_kind, int32_t groups, int32_t keep_groups, int32_t normalise, int64_t stream);
+/* rows i32 [T]: (previous token mul_prev + token mul_cur) mod buckets, or `buckets` at a sequence's first token; the last token of every
+ * sequence's portion is left in last_token (one 32-bit word per state slot, stride in words), where the next portion finds it */
+int mi355_hyb_bigram_rows(int32_t* rows, int32_t* last_token, int64_t state_stride, const uint32_t* tokens, const uint32_t* context_lens,
+                          const uint32_t* cu_seqlens_q, const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t buckets,
+                          int64_t mul_prev, int64_t mul_cur, int64_t stream);
+/* x f32 [T, copies, width]: every copy = table (dt) row ids[t] times scale + bigram (dt) row bigram_rows[t] (bigram NULL: nothing added) */
+int mi355_hyb_embed_streams(float* x, const void* table, const void* bigram, const int32_t* bigram_rows, const uint32_t* ids, int32_t num_tokens,
+                            int32_t copies, int32_t width, int32_t vocab, float scale, int32_t dtype, int64_t stream);
+/* the end of one sublayer and the start of the next in one launch, X f32 [T, streams, width]:
+ *   y = y_dense + sum_j moe_w[t, j] moe_rows[moe_pos[t top + j]]        (y_dense f32 [T, width] or NULL, moe_rows or NULL)
+ *   X_j <- sum_i mix[i, j] X_i + out_w[j] y                             (mix NULL: X stays, nothing was computed yet)
+ *   sum f32 [T, width] = sum_j X_j                                      (NULL = not written)
+ *   out (dt_out) [T, width] (and out_f32, NULL or f32) = RMSnorm(sum_i in_w[i] X_i) norm_w    (norm_w NULL: neither this nor X is written)
+ * streams <= 16, width <= 12288 */
+int mi355_hyb_stream_step(float* X, const float* y_dense, const float* moe_rows, const int32_t* moe_pos, const float* moe_w, int32_t top,
+                          const float* mix, const float* out_w, float* sum, const float* in_w, const float* norm_w, void* out,
+                          int32_t out_dtype, float* out_f32, int32_t num_tokens, int32_t streams, int32_t width, float eps, int64_t stream);
+/* out (dt_out) [T, n] = y / rms over each of `groups` equal parts * w[c] * sigmoid(gate_in[t, c]): the gate behind the norm */
+int mi355_hyb_norm_sigmoid_gate(void* out, int32_t out_dtype, const float* y, const float* gate_in, int32_t ldg, const float* w,
+                                int32_t num_tokens, int32_t n, int32_t groups, float eps, int64_t stream);
+/* linear attention with a constant decay per head over the new tokens of every sequence, state f32 [slots] x [heads, dim, vdim] (stride in
+ * floats): S <- decay[h] S + k v^T, o f32 [T, heads, vdim] = S^T q.  qkv f32 [T, ldq] holds q, k (heads x dim) and v (heads x vdim) at their
+ * offsets.  scratch != NULL: portions are cut into pieces of 64 tokens that are worked on side by side on the f32 matrix cores (needs
+ * dim and vdim that are multiples of 16, dim <= 512, and the floats below); NULL: one scan over the tokens.  dim <= 512 */
+int mi355_hyb_decay_attention(float* o, float* state, int64_t state_stride, const float* qkv, int32_t ldq, int32_t q_off, int32_t k_off,
+                              int32_t v_off, const float* decay, const uint32_t* context_lens, const uint32_t* cu_seqlens_q,
+                              const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads, int32_t dim, int32_t vdim,
+                              float* scratch, int64_t stream);
+/* floats of `scratch` that suit a step of this size; 0: the scan suits it (few tokens per sequence, or sizes that only the scan serves) */
+int64_t mi355_hyb_decay_attention_scratch(int32_t num_tokens, int32_t num_seqs, int32_t heads, int32_t dim, int32_t vdim);
 /* 0: prompt-sized steps over bf16 pages take the generic kernel instead of the matrix-core ones; 2: the matrix-core kernel with one
  * wave per head also where the query heads of a key/value head could share a workgroup (A/B switch, process-wide; default 1) */
 void mi355_hyb_set_attention_mfma(int32_t on);
