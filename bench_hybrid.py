@@ -1,5 +1,5 @@
 """`python bench.py --hybrid`: prompt and decode throughput of the layer-list host layer (Sogodra design, or Vivazen / Kerolorn /
-Sabolorn with `--hybrid-design vivazen|kerolorn|sabolorn`; random weights) at layer sizes of a real model, beside the framework's closest existing model -- the 16-bit llama host layer (dense_model.cpp) -- at equal
+Sabolorn / Tosivik with `--hybrid-design vivazen|kerolorn|sabolorn|tosivik`; random weights) at layer sizes of a real model, beside the framework's closest existing model -- the 16-bit llama host layer (dense_model.cpp) -- at equal
 width, depth, head geometry, feed-forward size and vocabulary.  One GPU, bf16, synthetic data.  The default workload of bench.py and
 its one-line contract are not touched: this option prints its own JSON line.
 
@@ -49,6 +49,62 @@ SABOLORN = {
     "8b": dict(s_heads=128, s_vdim=64, s_state=128, s_groups=8, l_heads=32, l_dim=128, l_rot=64, l_rank=192, l_vdim=128, q_rank=1536, taps=4,
                experts=16, top=4, groups=4, keep=2, side=256, layers="mall"),
 }
+
+
+# Tosivik at the same widths: linear attention with a constant decay (heads of 128 x 128) and attention with the llama geometry inside
+# chunks a little larger than the others' windows (a token behind 2048 cached ones sees 949 keys at 1b, 2049 at 3b and 8b), in turn; four residual streams; the first layer has a gelu feed-forward of the
+# llama size, the others relu^2 experts whose ACTIVE size equals it (`top` experts + the shared one, each ff / 4); the fourth layer runs
+# on the second one's weights
+TOSIVIK = {
+    "1b": dict(l_heads=16, l_dim=128, l_vdim=128, streams=4, experts=16, top=3, buckets=40009, layers="lala"),
+    "3b": dict(l_heads=24, l_dim=128, l_vdim=128, streams=4, experts=16, top=3, buckets=40009, layers="lala"),
+    "8b": dict(l_heads=32, l_dim=128, l_vdim=128, streams=4, experts=16, top=3, buckets=40009, layers="lala"),
+}
+
+
+def tosivik_config(s, v):
+    lin = {"decay": [float(np.exp(-2.0 ** (-8.0 * (i + 1) / v["l_heads"]))) for i in range(v["l_heads"])], "dim": v["l_dim"], "heads": v["l_heads"],
+           "vdim": v["l_vdim"]}
+    att = {"dim": s["dim"], "heads": s["heads"], "kv_heads": s["kv"], "mask": {"size": s["window"] + 76}, "scale": 1.1 * s["dim"] ** -0.5, "vdim": s["dim"],
+           "rot": {"base": 200000.0, "dims": s["dim"], "scaling": {"factor": 8.0, "fast": 24.0, "original": 4096, "slow": 2.0}}}
+    dense = {"ff": s["ff"], "kind": "dense"}
+    moe = {"expert": {"ff": s["ff"] // 4}, "kind": "moe", "router": {"experts": v["experts"], "top": v["top"]}, "shared": {"ff": s["ff"] // 4}}
+    layers, first = [], None
+    for i, c in enumerate(v["layers"]):
+        e = {"type": "lightning" if c == "l" else "attention", "mixer": lin if c == "l" else att, "mlp": dense if i == 0 else moe}
+        if c == "a" and first is not None:
+            e["weights_of"] = first
+        first = i if c == "a" and first is None else first
+        layers.append(e)
+    return {"architecture": "Tosivik", "embedding": {"bigram": {"buckets": v["buckets"], "mul_cur": 31, "mul_prev": 1009}, "scale": 2.0}, "layers": layers,
+            "logit_softcap": 30.0, "norm": {"eps": 1e-5}, "streams": v["streams"], "vocab": s["vocab"], "width": s["width"]}
+
+
+def tosivik_shapes(cfg):
+    W, sh, S = cfg["width"], {}, cfg["streams"]
+    sh["embed"], sh["final.norm"], sh["head"], sh["bigram"] = (cfg["vocab"], W), (W,), (cfg["vocab"], W), (cfg["embedding"]["bigram"]["buckets"] + 1, W)
+    for i, lc in enumerate(cfg["layers"]):
+        if "weights_of" in lc:
+            continue
+        p, c, mlp = "l%d." % i, lc["mixer"], lc["mlp"]
+        q, m = p + "mix.", p + "mlp."
+        for n in (1, 2):
+            sh[p + "norm%d" % n] = (W,)
+            sh[p + "hc%d.in" % n], sh[p + "hc%d.out" % n], sh[p + "hc%d.mix" % n] = (S,), (S,), (S, S)
+        H, d, vd = c["heads"], c["dim"], c["vdim"]
+        sh[q + "q"], sh[q + "o"] = (H * d, W), (W, H * vd)
+        if lc["type"] == "attention":
+            sh[q + "k"] = (c["kv_heads"] * d, W)
+        else:
+            sh[q + "k"], sh[q + "v"], sh[q + "g"], sh[q + "norm"] = (H * d, W), (H * vd, W), (H * vd, W), (H * vd,)
+        if mlp["kind"] == "dense":
+            sh[m + "up"], sh[m + "down"] = (mlp["ff"], W), (W, mlp["ff"])
+        else:
+            for e in ["e%d" % e for e in range(mlp["router"]["experts"])] + ["shared"]:
+                ff = mlp["shared" if e == "shared" else "expert"]["ff"]
+                sh[m + e + ".up"], sh[m + e + ".down"] = (ff, W), (W, ff)
+            sh[m + "router"], sh[m + "router.b"] = (mlp["router"]["experts"], W), (mlp["router"]["experts"],)
+    return sh
 
 
 def sabolorn_config(s, v):
@@ -225,7 +281,8 @@ def build_hybrid(cfg, max_tokens, slots):
     """random weights generated on the GPU, concatenated as the loader does it, handed over as device bf16"""
     import torch
     from candle_vllm_amd import hybrid_model as hm
-    shapes = {"Vivazen": vivazen_shapes, "Kerolorn": kerolorn_shapes, "Sogodra": sogodra_shapes, "Sabolorn": sabolorn_shapes}[cfg["architecture"]](cfg)
+    shapes = {"Vivazen": vivazen_shapes, "Kerolorn": kerolorn_shapes, "Sogodra": sogodra_shapes, "Sabolorn": sabolorn_shapes,
+              "Tosivik": tosivik_shapes}[cfg["architecture"]](cfg)
     spec = hm.SPECS[cfg["architecture"]](cfg, shapes)
     m = hm.HybridModel(spec, dtype="bfloat16", block_size=64, state_slots=slots)
     g = torch.Generator(device="cuda").manual_seed(7)
@@ -245,6 +302,10 @@ def build_hybrid(cfg, max_tokens, slots):
             return (0.1 + torch.rand(shape, generator=g, device="cuda")).to(torch.bfloat16)
         if name.endswith(".dwa"):
             return torch.full(shape, 1.0 / shape[0], device="cuda").to(torch.bfloat16)
+        if ".hc" in name:                                                 # mixing of the residual streams: near the identity, every stream takes part
+            n = shape[0]
+            base = 0.8 * torch.eye(n, device="cuda") + 0.2 / n if name.endswith(".mix") else torch.full(shape, 1.0 / n if name.endswith(".in") else 0.7, device="cuda")
+            return (base + 0.05 * torch.randn(shape, generator=g, device="cuda")).to(torch.bfloat16)
         if name.endswith(".talk"):
             return (torch.eye(shape[0], device="cuda") + 0.1 * torch.randn(shape, generator=g, device="cuda")).to(torch.bfloat16)
         s = 0.5 if name.endswith(".conv") else 0.3 if name.endswith("canon1") else (fan ** -0.5 if len(shape) > 1 else 0.3)
@@ -252,6 +313,10 @@ def build_hybrid(cfg, max_tokens, slots):
 
     def put(layer, which, names, axis=0):
         nonlocal nbytes
+        if isinstance(names[0], hm.Constants):
+            v = np.ascontiguousarray(names[0].values)
+            hm._check(hm.lib.mi355_hybrid_set_weight_f32(m.h, layer, which, v.ctypes.data, v.size), "set_weight_f32")
+            return
         names = [n.name if isinstance(n, hm.HeadTranspose) else n for n in names]       # random values: the transposed layout is as random
         ts = [rnd(shapes[n], n) if n else None for n in names]
         if which == hm.HW_IN_BIAS:
@@ -288,9 +353,9 @@ def run_size(name, T=2048, B=8, ctx=2048, dec_steps=16, design="sogodra"):
     from candle_vllm_amd.step_engine import StepEngine
     from oracle.dense_llama import DenseConfig
     s = SIZES[name]
-    extra = {"vivazen": VIVAZEN, "kerolorn": KEROLORN, "sabolorn": SABOLORN}.get(design, {}).get(name, {})
+    extra = {"vivazen": VIVAZEN, "kerolorn": KEROLORN, "sabolorn": SABOLORN, "tosivik": TOSIVIK}.get(design, {}).get(name, {})
     cfg = (vivazen_config(s, extra) if design == "vivazen" else kerolorn_config(s, extra) if design == "kerolorn" else
-           sabolorn_config(s, extra) if design == "sabolorn" else sogodra_config(s))
+           sabolorn_config(s, extra) if design == "sabolorn" else tosivik_config(s, extra) if design == "tosivik" else sogodra_config(s))
     rng = np.random.default_rng(5)
     out = {"size": name, "design": design, "shape": dict(s, **extra), "prompt_tokens": T, "decode_batch": B,
            "decode_ctx": ctx}
@@ -361,8 +426,8 @@ def run_size(name, T=2048, B=8, ctx=2048, dec_steps=16, design="sogodra"):
 
 
 def main(sizes="1b,3b", prompt_tokens=2048, batch=8, ctx=2048, design="sogodra"):
-    if design not in ("sogodra", "vivazen", "kerolorn", "sabolorn"):
-        raise SystemExit("--hybrid-design: sogodra, vivazen, kerolorn or sabolorn")
+    if design not in ("sogodra", "vivazen", "kerolorn", "sabolorn", "tosivik"):
+        raise SystemExit("--hybrid-design: sogodra, vivazen, kerolorn, sabolorn or tosivik")
     res = [run_size(n.strip(), T=prompt_tokens, B=batch, ctx=ctx, design=design) for n in sizes.split(",") if n.strip()]
     print(json.dumps({"metric": "hybrid_vs_llama_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
                       "note": "%s layer-list host layer beside the 16-bit llama host layer at equal sizes; the hybrid side's decode steps replay "

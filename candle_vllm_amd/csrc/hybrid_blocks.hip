@@ -298,7 +298,7 @@ __global__ __launch_bounds__(256) void decay_piece_state_kernel(PieceArgs p) {
         f32x4_t acc[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+#pragma unroll 4
         for (int t = 0; t < n; t += 4) {
             const bool on = t + kg < n;
             const float b = on ? V[(size_t)(t + kg) * p.ldq] * pw[n - 1 - t - kg] : 0.f;
@@ -373,24 +373,52 @@ template <int VT> __global__ __launch_bounds__(256) void decay_piece_output_kern
     const float* Kr[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) Kr[i] = K + (size_t)min(16 * i + m16, n - 1) * p.ldq;
+    // (the operands of the next 16 of the depth are requested before the current ones are multiplied)
+    float4 q, k[4], qn, kn[4];
+    float b[4][VT], bn[4][VT];
+    auto fetch = [&](int j) {
+        qn = *reinterpret_cast<const float4*>(Q + j);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) if (i <= wave) kn[i] = *reinterpret_cast<const float4*>(Kr[i] + j);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) bn[e][c] = col0 + 16 * c < vd ? S[(size_t)(j + 4 * kg + e) * vd + 16 * c] : 0.f;
+    };
+    auto fetch_values = [&](int j) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) {
+                const int t = j + 4 * kg + e;
+                bn[e][c] = (t < n && col0 + 16 * c < vd) ? V[(size_t)t * p.ldq + 16 * c] : 0.f;
+            }
+    };
+    auto take = [&]() {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) b[e][c] = bn[e][c];
+    };
+    fetch(0);
     for (int j = 0; j < d; j += 16) {
-        const float4 q = *reinterpret_cast<const float4*>(Q + j);
+        q = qn;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) k[i] = kn[i];
+        take();
+        if (j + 16 < d) fetch(j + 16); else fetch_values(0);
         const float qa[4] = {q.x, q.y, q.z, q.w};
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             if (i > wave) break;
-            const float4 k = *reinterpret_cast<const float4*>(Kr[i] + j);
-            const float ka[4] = {k.x, k.y, k.z, k.w};
+            const float ka[4] = {k[i].x, k[i].y, k[i].z, k[i].w};
 #pragma unroll
             for (int e = 0; e < 4; ++e) sc[i] = mfma_f32(qa[e], ka[e], sc[i]);
         }
 #pragma unroll
         for (int e = 0; e < 4; ++e)
 #pragma unroll
-            for (int c = 0; c < VT; ++c) {
-                const float b = col0 + 16 * c < vd ? S[(size_t)(j + 4 * kg + e) * vd + 16 * c] : 0.f;
-                acc[c] = mfma_f32(qa[e] * qscale, b, acc[c]);
-            }
+            for (int c = 0; c < VT; ++c) acc[c] = mfma_f32(qa[e] * qscale, b[e][c], acc[c]);
     }
     float* Pw = P[wave];
 #pragma unroll
@@ -402,17 +430,14 @@ template <int VT> __global__ __launch_bounds__(256) void decay_piece_output_kern
         }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); __builtin_amdgcn_wave_barrier();
     for (int j = 0; j <= row0; j += 16) {
+        take();
+        if (j + 16 <= row0) fetch_values(j + 16);
         const float4 a4 = *reinterpret_cast<const float4*>(&Pw[m16 * PR + j + 4 * kg]);
         const float a[4] = {a4.x, a4.y, a4.z, a4.w};
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int t = j + 4 * kg + e;
+        for (int e = 0; e < 4; ++e)
 #pragma unroll
-            for (int c = 0; c < VT; ++c) {
-                const float b = (t < n && col0 + 16 * c < vd) ? V[(size_t)t * p.ldq + 16 * c] : 0.f;
-                acc[c] = mfma_f32(a[e], b, acc[c]);
-            }
-        }
+            for (int c = 0; c < VT; ++c) acc[c] = mfma_f32(a[e], b[e][c], acc[c]);
     }
 #pragma unroll
     for (int c = 0; c < VT; ++c) {

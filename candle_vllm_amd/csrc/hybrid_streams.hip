@@ -28,7 +28,7 @@ __global__ __launch_bounds__(256) void bigram_rows_kernel(int32_t* rows, int32_t
     if (threadIdx.x == 0) *word = (int32_t)tokens[te - 1];
 }
 
-template <typename TW> __global__ void embed_streams_kernel(float* x, const TW* table, const TW* bigram, const int32_t* rows, const uint32_t* ids,
+template <typename TW> __global__ __launch_bounds__(1024) void embed_streams_kernel(float* x, const TW* table, const TW* bigram, const int32_t* rows, const uint32_t* ids,
                                                             int copies, int width, int vocab, float scale) {
     const int t = blockIdx.x;
     const uint32_t id = min(ids[t], (uint32_t)(vocab - 1));
@@ -196,8 +196,9 @@ int mi355_hyb_embed_streams(float* x, const void* table, const void* bigram, con
     if (!x || !table || !ids || (bigram && !bigram_rows) || copies < 1 || width <= 0 || vocab <= 0 || !is_dt(dtype)) return -1;
     if (T <= 0) return 0;
     hipStream_t s_ = to_stream(stream);
-    if (dtype == MI355_DTYPE_F32) embed_streams_kernel<float><<<T, 256, 0, s_>>>(x, (const float*)table, (const float*)bigram, bigram_rows, ids, copies, width, vocab, scale);
-    else embed_streams_kernel<uint16_t><<<T, 256, 0, s_>>>(x, (const uint16_t*)table, (const uint16_t*)bigram, bigram_rows, ids, copies, width, vocab, scale);
+    const int nt = (T <= 64 && width > 256) ? 1024 : 256;
+    if (dtype == MI355_DTYPE_F32) embed_streams_kernel<float><<<T, nt, 0, s_>>>(x, (const float*)table, (const float*)bigram, bigram_rows, ids, copies, width, vocab, scale);
+    else embed_streams_kernel<uint16_t><<<T, nt, 0, s_>>>(x, (const uint16_t*)table, (const uint16_t*)bigram, bigram_rows, ids, copies, width, vocab, scale);
     LAUNCH_OK(); return 0;
 }
 

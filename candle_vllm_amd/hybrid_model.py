@@ -526,17 +526,17 @@ class TosivikSpec:
             g[HW_BIGRAM] = "bigram"
         return g
 
-    def _mixing(self, p, q, slots):
+    def _mixing(self, p, q, slots, shapes):
         """the weights of the copies around sublayer q of the layer"""
         hc = p + "hc%d." % q
         names = (HW_HC1_IN, HW_HC1_OUT, HW_HC1_MIX) if q == 1 else (HW_HC2_IN, HW_HC2_OUT, HW_HC2_MIX)
         for slot, n in zip(names, ("in", "out", "mix")):
-            slots[slot] = [hc + n] if self.cfg.get("streams") else [Ones(1)]
+            slots[slot] = [hc + n] if self.streams > 1 or hc + n in shapes else [Ones(1)]
 
     def _layer(self, p, lc, shapes):
         L, slots, rope = HybridLayer(), {HW_NORM1: [p + "norm1"]}, None
         c, kind, q = lc["mixer"], lc["type"], p + "mix."
-        self._mixing(p, 1, slots)
+        self._mixing(p, 1, slots, shapes)
         if kind == "attention":
             L.mixer = MIX_ATTENTION
             L.a_heads, L.a_kv_heads, L.a_dim, L.a_vdim = int(c["heads"]), int(c["kv_heads"]), int(c["dim"]), int(c["vdim"])
@@ -557,7 +557,7 @@ class TosivikSpec:
         if mlp:
             m = p + "mlp."
             slots[HW_NORM2] = [p + "norm2"]
-            self._mixing(p, 2, slots)
+            self._mixing(p, 2, slots, shapes)
             if mlp.get("kind") == "dense":
                 L.mlp_kind, L.mlp_ff = MLP_GELU, int(mlp["ff"])
                 slots[HW_MLP_GATE_UP], slots[HW_MLP_DOWN] = [m + "up"], [m + "down"]

@@ -180,8 +180,9 @@ def weight_layer(layers, i):
     return i
 
 
-def forward(cfg, W, tokens, margins=None):
-    """-> logits [T, vocab], the sum of the copies behind every layer [n_layers, T, width]; margins: see route()"""
+def forward(cfg, W, tokens, margins=None, operand=None):
+    """-> logits [T, vocab], the sum of the copies behind every layer [n_layers, T, width]; margins: see route(); operand: what is done
+    to every sublayer's normed input (a rounding: how far it alone moves the logits)"""
     tokens = np.asarray(tokens, np.int64)
     eps, s = float(cfg["norm"]["eps"]), int(cfg.get("streams", 1))
     X = np.stack([embedding(cfg, W, tokens)] * s)
@@ -198,7 +199,8 @@ def forward(cfg, W, tokens, margins=None):
             if n == 2 and not m:
                 continue
             hc = "%shc%d." % (p, n)
-            y = f(rms_norm(stream_mixture(X, W[hc + "in"]), W[p + "norm%d" % n], eps))
+            h = rms_norm(stream_mixture(X, W[hc + "in"]), W[p + "norm%d" % n], eps)
+            y = f(operand(h) if operand else h)
             X = stream_update(X, W[hc + "mix"], W[hc + "out"], y)
         trace.append(X.sum(0))
     z = rms_norm(X.sum(0), W["final.norm"], eps) @ W["head"].T
