@@ -54,14 +54,17 @@ struct LinArgs {
     // epilogue: columns < act_cols pass an activation (MI355_HYB_ACT_*), out16: `out` holds bf16 instead of f32
     int act, act_cols, out16;
 };
-__device__ __forceinline__ void lin_store(const LinArgs& p, int t, int n, float v) {
-    if (p.act && n < p.act_cols) {
-        if (p.act == MI355_HYB_ACT_SILU) v = siluf_(v);
-        else if (p.act == MI355_HYB_ACT_GELU) v = gelu_tanhf_(v);
-        else { v = fmaxf(v, 0.f); v *= v; }
+// (EPI is a build of its own so that the plain products pay nothing for it)
+template <bool EPI> __device__ __forceinline__ void lin_store(const LinArgs& p, int t, int n, float v) {
+    if (EPI) {
+        if (p.act && n < p.act_cols) {
+            if (p.act == MI355_HYB_ACT_SILU) v = siluf_(v);
+            else if (p.act == MI355_HYB_ACT_GELU) v = gelu_tanhf_(v);
+            else { v = fmaxf(v, 0.f); v *= v; }
+        }
+        if (p.out16) { reinterpret_cast<uint16_t*>(p.out)[(size_t)t * p.ldo + n] = f32_to_bf16(v); return; }
     }
-    if (p.out16) reinterpret_cast<uint16_t*>(p.out)[(size_t)t * p.ldo + n] = f32_to_bf16(v);
-    else p.out[(size_t)t * p.ldo + n] = v;
+    p.out[(size_t)t * p.ldo + n] = v;
 }
 // the block's matrix and the end of its rows (one past the last); false = nothing to do
 __device__ __forceinline__ bool lin_group(LinArgs& p, int t0, int64_t& w_off) {
@@ -84,7 +87,7 @@ template <typename TA> __device__ __forceinline__ void lin_batch(LinArgs& p) {
 // Prompt-sized products, bf16 weights.  A workgroup of four waves owns 64 output columns (16 weight rows per wave) and 16 MT tokens;
 // fragments go from global memory / L2 straight into registers: lane (m16, kg) holds operands 8 kg .. 8 kg + 7 of row m16 of a
 // 32-wide K step on both sides, the accumulator holds tokens 4 kg + v of column m16.
-template <typename TA, int MT> __global__ __launch_bounds__(256) void linear_bf16_tile_kernel(LinArgs p) {
+template <typename TA, int MT, bool EPI> __global__ __launch_bounds__(256) void linear_bf16_tile_kernel(LinArgs p) {
     lin_batch<TA>(p);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4;
     const int n = blockIdx.x * 64 + wave * 16 + m16;
@@ -120,7 +123,7 @@ template <typename TA, int MT> __global__ __launch_bounds__(256) void linear_bf1
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const int t = t0 + i * 16 + 4 * kg + v;
-            if (t < p.T) lin_store(p, t, n, acc[i][v] + bias);
+            if (t < p.T) lin_store<EPI>(p, t, n, acc[i][v] + bias);
         }
 }
 
@@ -128,7 +131,7 @@ template <typename TA, int MT> __global__ __launch_bounds__(256) void linear_bf1
 // owns a 128-token x 128-column tile, each wave a 64 x 64 quarter (4 x 4 MFMA tiles).  The 128 x 32 slices of both operands go
 // through LDS (rows padded to 80 bytes so that the 16 rows a fragment read touches fall into different 16-byte banks), the slice
 // of the next K step is fetched into registers while the current one is multiplied: one barrier per K step.
-__global__ __launch_bounds__(256) void linear_bf16_lds_kernel(LinArgs p) {
+template <bool EPI> __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(LinArgs p) {
     constexpr int ROWB = 80;                                        // bytes per staged row: 64 of data + 16 of padding
     __shared__ __align__(16) uint8_t sa[2][128 * ROWB], sw[2][128 * ROWB];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m16 = lane & 15, kg = lane >> 4;
@@ -198,14 +201,14 @@ __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(LinArgs p) {
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
                 const int t = t0 + wr * 64 + i * 16 + 4 * kg + v;
-                if (t < p.T) lin_store(p, t, n, acc[i][j][v] + bias);
+                if (t < p.T) lin_store<EPI>(p, t, n, acc[i][j][v] + bias);
             }
     }
 }
 
 // Up to 16 tokens, bf16 weights: the product is a stream over the weights.  A workgroup owns 16 weight rows; its NW waves take the
 // 32-wide K steps in turn (UNR steps in flight per wave) and add their partial tiles through LDS.
-template <typename TA, int NW, int UNR> __global__ __launch_bounds__(64 * NW) void linear_bf16_stream_kernel(LinArgs p) {
+template <typename TA, int NW, int UNR, bool EPI> __global__ __launch_bounds__(64 * NW) void linear_bf16_stream_kernel(LinArgs p) {
     __shared__ float part[NW][4][64];
     lin_batch<TA>(p);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4;
@@ -239,14 +242,14 @@ template <typename TA, int NW, int UNR> __global__ __launch_bounds__(64 * NW) vo
 #pragma unroll
             for (int w = 0; w < NW; ++w) s += part[w][v][lane];
             const int t = t0 + 4 * kg + v;
-            if (nok && t < p.T) lin_store(p, t, n, s + bias);
+            if (nok && t < p.T) lin_store<EPI>(p, t, n, s + bias);
         }
     }
 }
 
 // f32 weights and operands: plain FMAs in f32 (no reduced-precision matrix mode).  64 x 64 tile, 16-wide K steps through LDS,
 // every thread owns 4 tokens x 4 columns.
-__global__ __launch_bounds__(256) void linear_f32_kernel(LinArgs p) {
+template <bool EPI> __global__ __launch_bounds__(256) void linear_f32_kernel(LinArgs p) {
     __shared__ float As[16][68], Ws[16][68];
     const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;
     const int n0 = blockIdx.x * 64, t0 = blockIdx.y * 64;
@@ -285,7 +288,7 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(LinArgs p) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < p.N) lin_store(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
+            if (n < p.N) lin_store<EPI>(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
         }
     }
 }
@@ -1788,6 +1791,8 @@ int mi355_hyb_fill_f32(float* out, float v, int64_t n, int64_t stream) {
     LAUNCH_OK(); return 0;
 }
 
+// which build of a product kernel: with an activation or a 16-bit result, or the plain one
+#define LIN_EPI(p, CALL) do { if ((p).act || (p).out16) { constexpr bool EPI = true; CALL; } else { constexpr bool EPI = false; CALL; } } while (0)
 static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, int32_t a_dtype, int32_t lda, int64_t a_bs, const void* w,
                          int64_t w_bs, const float* bias, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream,
                          int32_t act = 0, int32_t act_cols = 0, int32_t out16 = 0) {
@@ -1799,7 +1804,7 @@ static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, i
     const unsigned nz = (unsigned)batch;
     if (dtype == MI355_DTYPE_F32) {
         if (a_dtype != MI355_DTYPE_F32) return -1;
-        linear_f32_kernel<<<dim3((n + 63) / 64, (T + 63) / 64, nz), 256, 0, st_>>>(p);
+        LIN_EPI(p, (linear_f32_kernel<EPI><<<dim3((n + 63) / 64, (T + 63) / 64, nz), 256, 0, st_>>>(p)));
         LAUNCH_OK(); return 0;
     }
     const int a_bytes = a_dtype == MI355_DTYPE_F32 ? 4 : 2;
@@ -1808,16 +1813,16 @@ static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, i
     const bool af = a_dtype == MI355_DTYPE_F32;
     if (T <= 16) {
         const dim3 grid((n + 15) / 16, 1, nz);
-        if (k >= 2048) { if (af) linear_bf16_stream_kernel<float, 4, 4><<<grid, 256, 0, st_>>>(p); else linear_bf16_stream_kernel<uint16_t, 4, 4><<<grid, 256, 0, st_>>>(p); }
-        else { if (af) linear_bf16_stream_kernel<float, 2, 2><<<grid, 128, 0, st_>>>(p); else linear_bf16_stream_kernel<uint16_t, 2, 2><<<grid, 128, 0, st_>>>(p); }
+        if (k >= 2048) { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
+        else { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
     } else if (T > 32 && !af && p.a_vec && p.w_vec && k % 32 == 0) {
-        linear_bf16_lds_kernel<<<dim3((n + 127) / 128, (T + 127) / 128, nz), 256, 0, st_>>>(p);
+        LIN_EPI(p, (linear_bf16_lds_kernel<EPI><<<dim3((n + 127) / 128, (T + 127) / 128, nz), 256, 0, st_>>>(p)));
     } else if (T <= 32) {
         const dim3 grid((n + 63) / 64, (T + 31) / 32, nz);
-        if (af) linear_bf16_tile_kernel<float, 2><<<grid, 256, 0, st_>>>(p); else linear_bf16_tile_kernel<uint16_t, 2><<<grid, 256, 0, st_>>>(p);
+        if (af) LIN_EPI(p, (linear_bf16_tile_kernel<float, 2, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 2, EPI><<<grid, 256, 0, st_>>>(p)));
     } else {
         const dim3 grid((n + 63) / 64, (T + 63) / 64, nz);
-        if (af) linear_bf16_tile_kernel<float, 4><<<grid, 256, 0, st_>>>(p); else linear_bf16_tile_kernel<uint16_t, 4><<<grid, 256, 0, st_>>>(p);
+        if (af) LIN_EPI(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
     }
     LAUNCH_OK(); return 0;
 }
@@ -2326,7 +2331,7 @@ int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, cons
     hipStream_t st_ = to_stream(stream);
     if (dtype == MI355_DTYPE_F32) {
         if (a_dtype != MI355_DTYPE_F32 || block_rows != 64) return -1;
-        linear_f32_kernel<<<dim3((n + 63) / 64, n_blocks, 1), 256, 0, st_>>>(p);
+        LIN_EPI(p, (linear_f32_kernel<EPI><<<dim3((n + 63) / 64, n_blocks, 1), 256, 0, st_>>>(p)));
         LAUNCH_OK(); return 0;
     }
     const int a_bytes = a_dtype == MI355_DTYPE_F32 ? 4 : 2;
@@ -2335,13 +2340,13 @@ int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, cons
     const bool af = a_dtype == MI355_DTYPE_F32;
     if (block_rows == 16) {
         const dim3 grid((n + 15) / 16, n_blocks, 1);
-        if (k >= 2048) { if (af) linear_bf16_stream_kernel<float, 4, 4><<<grid, 256, 0, st_>>>(p); else linear_bf16_stream_kernel<uint16_t, 4, 4><<<grid, 256, 0, st_>>>(p); }
-        else { if (af) linear_bf16_stream_kernel<float, 2, 2><<<grid, 128, 0, st_>>>(p); else linear_bf16_stream_kernel<uint16_t, 2, 2><<<grid, 128, 0, st_>>>(p); }
+        if (k >= 2048) { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
+        else { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
     } else if (block_rows == 64) {
         const dim3 grid((n + 63) / 64, n_blocks, 1);
-        if (af) linear_bf16_tile_kernel<float, 4><<<grid, 256, 0, st_>>>(p); else linear_bf16_tile_kernel<uint16_t, 4><<<grid, 256, 0, st_>>>(p);
+        if (af) LIN_EPI(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
     } else if (block_rows == 128 && !af && p.a_vec && p.w_vec && k % 32 == 0) {
-        linear_bf16_lds_kernel<<<dim3((n + 127) / 128, n_blocks, 1), 256, 0, st_>>>(p);
+        LIN_EPI(p, (linear_bf16_lds_kernel<EPI><<<dim3((n + 127) / 128, n_blocks, 1), 256, 0, st_>>>(p)));
     } else {
         return -1;
     }

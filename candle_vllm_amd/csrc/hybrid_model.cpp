@@ -12,7 +12,7 @@
 // (host_model.cpp, dense_model.cpp) it owns the weights, the K/V pages and the activation buffers and enqueues one step on a
 // stream; unlike them it owns a pool of recurrent state (one slot per live sequence, handed out by the block engine) and runs
 // prompts, portions of prompts and decoded tokens through the same launches.
-// Kernels: hybrid_kernels.hip.  Every projection that reads a mixer's input is one matrix (rows concatenated at load time), the
+// Kernels: hybrid_kernels.hip, hybrid_blocks.hip, hybrid_streams.hip.  Every projection that reads a mixer's input is one matrix (rows concatenated at load time), the
 // output projections of a parallel mixer are one matrix along k (the branch scales are applied to the operands, not the weights).
 #include <hip/hip_runtime.h>
 #include <algorithm>
