@@ -349,7 +349,8 @@ class HybridLayer(ctypes.Structure):
                 ("moe_sigmoid", c_i32), ("moe_groups", c_i32), ("moe_keep_groups", c_i32), ("moe_normalise", c_i32),
                 ("d_norm_groups", c_i32), ("a_dist_bias", c_i32), ("a_q_rank", c_i32), ("a_out_gate", c_i32), ("kv_from", c_i32),
                 ("side_dim", c_i32), ("side_col", c_i32), ("depth_terms", c_i32),
-                ("a_mask_kind", c_i32), ("a_v_is_k", c_i32), ("moe_relu2", c_i32), ("moe_bias", c_i32), ("moe_shared_plain", c_i32)]
+                ("a_mask_kind", c_i32), ("a_v_is_k", c_i32), ("moe_relu2", c_i32), ("moe_bias", c_i32), ("moe_shared_plain", c_i32),
+                ("a_temp_coef", c_f32), ("a_temp_every", c_f32)]
 
 
 class HybridConfig(ctypes.Structure):
@@ -454,6 +455,17 @@ _sig("mi355_hyb_stream_step", ctypes.c_int, [c_vp] * 5 + [c_i32] + [c_vp] * 6 + 
 _sig("mi355_hyb_norm_sigmoid_gate", ctypes.c_int, [c_vp, c_i32, c_vp, c_vp, c_i32, c_vp, c_i32, c_i32, c_i32, c_f32, c_i64])
 _sig("mi355_hyb_decay_attention", ctypes.c_int, [c_vp, c_vp, c_i64, c_vp, c_i32, c_i32, c_i32, c_i32] + [c_vp] * 4 + [c_i32] * 5 + [c_vp, c_i64])
 _sig("mi355_hyb_decay_attention_scratch", c_i64, [c_i32] * 5)
+_sig("mi355_hyb_linear_segments", ctypes.c_int, [c_vp, c_i32, c_vp, c_i32, c_i32, c_i64, c_i32, c_vp, c_vp, c_vp] + [c_i32] * 5 + [c_i64])
+_sig("mi355_hyb_pair_step", ctypes.c_int, [c_vp] * 6 + [c_i32] + [c_vp] * 4 + [c_i64, c_vp, c_i32, c_vp, c_vp, c_i32, c_vp, c_i64] + [c_vp] * 5 +
+     [c_i32, c_i32, c_f32, c_i64])
+_sig("mi355_hyb_lowrank_decay", ctypes.c_int, [c_vp, c_i32, c_vp, c_i32, c_vp, c_vp, c_i32, c_i32, c_i32, c_i64])
+_sig("mi355_hyb_bonus_recurrence", ctypes.c_int, [c_vp, c_vp, c_i64, c_vp, c_i32, c_i32, c_i32, c_i32, c_vp, c_i32] + [c_vp] * 4 + [c_i32] * 5 +
+     [c_vp, c_vp, c_i32, c_vp, c_i64])
+_sig("mi355_hyb_gated_norm_heads", ctypes.c_int, [c_vp, c_i32, c_i32, c_i32, c_vp, c_vp, c_i32, c_vp, c_i32, c_i32, c_i32, c_i32, c_i32, c_f32, c_f32, c_i64])
+_sig("mi355_hyb_attn_prepare_temp", ctypes.c_int, [c_vp] * 4 + [c_i32] * 4 + [c_vp] * 6 + [c_i32] * 8 + [c_vp, c_f32, c_f32, c_f32, c_i32, c_i64])
+_sig("mi355_hyb_attn_prepare_whole_temp", ctypes.c_int, [c_vp] * 4 + [c_i32] * 4 + [c_vp] * 4 + [c_i32] * 6 + [c_f32, c_f32, c_f32, c_i32, c_i64])
+_sig("mi355_hyb_attention_ex", ctypes.c_int, [c_vp, c_i32, c_i32, c_i32] + [c_vp] * 9 + [c_i32, c_vp, c_i32] + [c_i32] * 11 +
+     [c_f32, c_f32, c_i32, c_i32, c_f32, c_i32, c_i32, c_i64])
 
 # the hand-written ctypes mirrors must have the layout the library was built with
 for _id, _cls in ((0, QmmDesc), (1, LlamaConfig), (2, DenseConfig), (3, RopeScaling), (4, HybridConfig), (5, HybridLayer)):

@@ -41,6 +41,7 @@ __device__ __forceinline__ f32x4_t mfma_bf16(const uint4& a, const uint4& b, con
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
+constexpr int LIN_MAX_SEG = 8;
 struct LinArgs {
     float* out; int ldo;
     const void* a; int lda;
@@ -53,10 +54,13 @@ struct LinArgs {
     const int32_t* blk; const int32_t* row_src; int blk_rows;
     // epilogue: columns < act_cols pass an activation (MI355_HYB_ACT_*), out16: `out` holds bf16 instead of f32
     int act, act_cols, out16;
+    // segments: columns [.., seg_end[i]) are a product of their own left operand, a + (seg0 + i) seg_a elements (ends are multiples of 128)
+    int n_seg, seg0; int64_t seg_a; int seg_end[LIN_MAX_SEG];
 };
-// (EPI is a build of its own so that the plain products pay nothing for it)
-template <bool EPI> __device__ __forceinline__ void lin_store(const LinArgs& p, int t, int n, float v) {
-    if (EPI) {
+// (what a product can do beyond the plain one is a build of its own, so that the plain products pay nothing for it)
+enum { LIN_PLAIN = 0, LIN_EPI_BUILD = 1, LIN_SEG_BUILD = 2 };
+template <int B> __device__ __forceinline__ void lin_store(const LinArgs& p, int t, int n, float v) {
+    if (B == LIN_EPI_BUILD) {
         if (p.act && n < p.act_cols) {
             if (p.act == MI355_HYB_ACT_SILU) v = siluf_(v);
             else if (p.act == MI355_HYB_ACT_GELU) v = gelu_tanhf_(v);
@@ -78,7 +82,14 @@ __device__ __forceinline__ bool lin_group(LinArgs& p, int t0, int64_t& w_off) {
     return true;
 }
 __device__ __forceinline__ int lin_row(const LinArgs& p, int t) { return p.row_src ? p.row_src[t] : t; }
-template <typename TA> __device__ __forceinline__ void lin_batch(LinArgs& p) {
+// n0: the tile's first column
+template <typename TA, int B> __device__ __forceinline__ void lin_batch(LinArgs& p, int n0) {
+    if (B == LIN_SEG_BUILD) {
+        int i = 0;
+        while (i + 1 < p.n_seg && n0 >= p.seg_end[i]) ++i;
+        p.a = static_cast<const TA*>(p.a) + (p.seg0 + i) * p.seg_a;
+        return;
+    }
     const int64_t z = blockIdx.z;
     p.a = static_cast<const TA*>(p.a) + z * p.a_bs;
     p.out += z * p.o_bs;
@@ -87,8 +98,8 @@ template <typename TA> __device__ __forceinline__ void lin_batch(LinArgs& p) {
 // Prompt-sized products, bf16 weights.  A workgroup of four waves owns 64 output columns (16 weight rows per wave) and 16 MT tokens;
 // fragments go from global memory / L2 straight into registers: lane (m16, kg) holds operands 8 kg .. 8 kg + 7 of row m16 of a
 // 32-wide K step on both sides, the accumulator holds tokens 4 kg + v of column m16.
-template <typename TA, int MT, bool EPI> __global__ __launch_bounds__(256) void linear_bf16_tile_kernel(LinArgs p) {
-    lin_batch<TA>(p);
+template <typename TA, int MT, int B> __global__ __launch_bounds__(256) void linear_bf16_tile_kernel(LinArgs p) {
+    lin_batch<TA, B>(p, blockIdx.x * 64);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4;
     const int n = blockIdx.x * 64 + wave * 16 + m16;
     const int t0 = blockIdx.y * (16 * MT);
@@ -123,7 +134,7 @@ template <typename TA, int MT, bool EPI> __global__ __launch_bounds__(256) void 
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const int t = t0 + i * 16 + 4 * kg + v;
-            if (t < p.T) lin_store<EPI>(p, t, n, acc[i][v] + bias);
+            if (t < p.T) lin_store<B>(p, t, n, acc[i][v] + bias);
         }
 }
 
@@ -131,13 +142,13 @@ template <typename TA, int MT, bool EPI> __global__ __launch_bounds__(256) void 
 // owns a 128-token x 128-column tile, each wave a 64 x 64 quarter (4 x 4 MFMA tiles).  The 128 x 32 slices of both operands go
 // through LDS (rows padded to 80 bytes so that the 16 rows a fragment read touches fall into different 16-byte banks), the slice
 // of the next K step is fetched into registers while the current one is multiplied: one barrier per K step.
-template <bool EPI> __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(LinArgs p) {
+template <int B> __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(LinArgs p) {
     constexpr int ROWB = 80;                                        // bytes per staged row: 64 of data + 16 of padding
     __shared__ __align__(16) uint8_t sa[2][128 * ROWB], sw[2][128 * ROWB];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m16 = lane & 15, kg = lane >> 4;
     const int wr = wave >> 1, wc = wave & 1;
     const int n0 = blockIdx.x * 128, t0 = blockIdx.y * 128;
-    lin_batch<uint16_t>(p);
+    lin_batch<uint16_t, B>(p, n0);
     int64_t w_off;
     if (!lin_group(p, t0, w_off)) return;
     const uint16_t* A = static_cast<const uint16_t*>(p.a);
@@ -201,16 +212,16 @@ template <bool EPI> __global__ __launch_bounds__(256) void linear_bf16_lds_kerne
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
                 const int t = t0 + wr * 64 + i * 16 + 4 * kg + v;
-                if (t < p.T) lin_store<EPI>(p, t, n, acc[i][j][v] + bias);
+                if (t < p.T) lin_store<B>(p, t, n, acc[i][j][v] + bias);
             }
     }
 }
 
 // Up to 16 tokens, bf16 weights: the product is a stream over the weights.  A workgroup owns 16 weight rows; its NW waves take the
 // 32-wide K steps in turn (UNR steps in flight per wave) and add their partial tiles through LDS.
-template <typename TA, int NW, int UNR, bool EPI> __global__ __launch_bounds__(64 * NW) void linear_bf16_stream_kernel(LinArgs p) {
+template <typename TA, int NW, int UNR, int B> __global__ __launch_bounds__(64 * NW) void linear_bf16_stream_kernel(LinArgs p) {
     __shared__ float part[NW][4][64];
-    lin_batch<TA>(p);
+    lin_batch<TA, B>(p, blockIdx.x * 16);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4;
     const int n = blockIdx.x * 16 + m16;
     const int t0 = blockIdx.y * 16;                                  // a grouped product: block blockIdx.y of 16 rows; else 0
@@ -242,18 +253,18 @@ template <typename TA, int NW, int UNR, bool EPI> __global__ __launch_bounds__(6
 #pragma unroll
             for (int w = 0; w < NW; ++w) s += part[w][v][lane];
             const int t = t0 + 4 * kg + v;
-            if (nok && t < p.T) lin_store<EPI>(p, t, n, s + bias);
+            if (nok && t < p.T) lin_store<B>(p, t, n, s + bias);
         }
     }
 }
 
 // f32 weights and operands: plain FMAs in f32 (no reduced-precision matrix mode).  64 x 64 tile, 16-wide K steps through LDS,
 // every thread owns 4 tokens x 4 columns.
-template <bool EPI> __global__ __launch_bounds__(256) void linear_f32_kernel(LinArgs p) {
+template <int B> __global__ __launch_bounds__(256) void linear_f32_kernel(LinArgs p) {
     __shared__ float As[16][68], Ws[16][68];
     const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;
     const int n0 = blockIdx.x * 64, t0 = blockIdx.y * 64;
-    lin_batch<float>(p);
+    lin_batch<float, B>(p, n0);
     int64_t w_off;
     if (!lin_group(p, t0, w_off)) return;
     const float* A = static_cast<const float*>(p.a);
@@ -288,7 +299,7 @@ template <bool EPI> __global__ __launch_bounds__(256) void linear_f32_kernel(Lin
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < p.N) lin_store<EPI>(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
+            if (n < p.N) lin_store<B>(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
         }
     }
 }
@@ -432,7 +443,11 @@ struct PrepArgs {
     int interleaved;        // rotated pairs are (2i, 2i + 1) instead of (i, i + rot / 2)
     int norm_mode;          // 0 none, 1 RMS norm (weights qw / kw or none) before the rotation, 2 weightless RMS norm after it
     const float* q_scale;   // [H] or NULL: head h's query times q_scale[h]
+    float temp_coef, temp_every;  // temp_coef != 0: the query at position p times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
 };
+__device__ __forceinline__ float query_temp(float coef, float every, int64_t pos) {
+    return coef != 0.f ? 1.f + coef * logf((float)floor((double)(pos + 1) / (double)every) + 1.f) : 1.f;
+}
 // one wave per (token, vector): query heads 0 .. H-1, key heads H .. H+G-1, value heads H+G .. H+2G-1
 template <typename TC> __global__ __launch_bounds__(64) void attn_prepare_kernel(PrepArgs p) {
     extern __shared__ float vec[];
@@ -487,6 +502,7 @@ template <typename TC> __global__ __launch_bounds__(64) void attn_prepare_kernel
     float mul = 1.f;
     if (p.norm_mode == 2) mul = 1.f / sqrtf(wave_sum(s2) / (float)p.d + p.eps);
     if (is_q && p.q_scale) mul *= p.q_scale[h];
+    if (is_q) mul *= query_temp(p.temp_coef, p.temp_every, pos);
     for (int i = lane; i < p.d; i += 64) st<TC>(dst, i, rotated[i] * mul);
 }
 
@@ -502,6 +518,8 @@ struct AttnArgs {
     int keep;               // with a window: keys at positions < keep stay visible (the first tokens of the sequence)
     const float* dist;      // != NULL: [2, H] = r1, r2; score <- score - r1[h] ln(1 + r2[h] (query position - key position))
     int chunked;            // the window is a chunk: a query sees the keys from the last multiple of `window` at or below its position on
+    int dist_linear;        // the distance bias is r1[h] (query position - key position)
+    const float* gate; int ldg;   // != NULL: head h's output times sigmoid(gate[t ldg + h])
     // the lowest key that a query sees (beside the kept first tokens)
     __device__ __forceinline__ int first_key(int pos) const {
         if (window <= 0) return 0;
@@ -510,6 +528,12 @@ struct AttnArgs {
 };
 // (the hardware's log2: the argument is at least 1, so the absolute error stays near the f32 rounding of the score it is taken from)
 __device__ __forceinline__ float dist_bias(float r1, float r2, int d) { return r1 * 0.6931471805599453f * __log2f(fmaf(r2, (float)d, 1.f)); }
+__device__ __forceinline__ float distance_off(const AttnArgs& p, float r1, float r2, int d) {
+    return !p.dist ? 0.f : p.dist_linear ? r1 * (float)d : dist_bias(r1, r2, d);
+}
+__device__ __forceinline__ float head_out_scale(const AttnArgs& p, int t, int h) {
+    return p.gate ? p.out_scale * sigmoidf_(p.gate[(size_t)t * p.ldg + h]) : p.out_scale;
+}
 __device__ __forceinline__ float cap_score(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
 // 16 bytes of a page row as floats (EPV = 8 bf16 or 4 f32)
 template <typename TC> struct Vec16;
@@ -606,12 +630,12 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
                     if (lane / kq == u0 + u) dot = v;
                 }
             }
-            if (j <= pos) sc = cap_score(dot * p.scale, p.softcap) - (p.dist ? dist_bias(r1, r2, pos - j) : 0.f);
+            if (j <= pos) sc = cap_score(dot * p.scale, p.softcap) - distance_off(p, r1, r2, pos - j);
         } else if (j <= pos) {
             const TC* kr = static_cast<const TC*>(p.k_pages) + (size_t)page_row * p.k_ld + g * p.d;
             float dot = 0.f;
             for (int i = 0; i < p.d; ++i) dot = fmaf(qs[i], ld<TC>(kr, i), dot);
-            sc = cap_score(dot * p.scale, p.softcap) - (p.dist ? dist_bias(r1, r2, pos - j) : 0.f);
+            sc = cap_score(dot * p.scale, p.softcap) - distance_off(p, r1, r2, pos - j);
         }
         const float mn = fmaxf(m, wave_max(sc));
         const float pj = (j <= pos) ? expf(sc - mn) : 0.f;
@@ -685,14 +709,15 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
         for (int w = 0; w < NW; ++w) M = fmaxf(M, pm[w]);
         float L = p.sink ? expf(p.sink[h] - M) : 0.f;
         float cw[NW];
+        const float os = head_out_scale(p, t, h);
         for (int w = 0; w < NW; ++w) { cw[w] = pm[w] == -INFINITY ? 0.f : expf(pm[w] - M); L += pl[w] * cw[w]; }
         for (int n = 0; n < NV; ++n) {
             const size_t base = (size_t)t * p.ldo + p.out_off + (size_t)(oh0 + n) * p.vd;
             for (int col = lane; col < p.vd; col += 64) {
                 float o = 0.f;
                 for (int w = 0; w < NW; ++w) o += pacc[(w * NV + n) * p.vd + col] * cw[w];
-                if (p.out_f32) st<float>(static_cast<float*>(p.out), base + col, o / L * p.out_scale);
-                else st<uint16_t>(static_cast<uint16_t*>(p.out), base + col, o / L * p.out_scale);
+                if (p.out_f32) st<float>(static_cast<float*>(p.out), base + col, o / L * os);
+                else st<uint16_t>(static_cast<uint16_t*>(p.out), base + col, o / L * os);
             }
         }
     }
@@ -826,7 +851,7 @@ void window_attention_mfma_kernel(AttnArgs p) {
             for (int kt = 0; kt < 4; ++kt) {
                 const int key = key_at(j0 + kt * 16 + m16);
                 const bool ok_ = r < nq && key <= qpos && (key >= low[v] || key < p.keep);
-                sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - (p.dist ? dist_bias(r1, r2, qpos - key) : 0.f) : -INFINITY;
+                sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - distance_off(p, r1, r2, qpos - key) : -INFINITY;
                 mx[v] = fmaxf(mx[v], sc[v][kt]);
             }
 #pragma unroll
@@ -887,7 +912,7 @@ void window_attention_mfma_kernel(AttnArgs p) {
         const float M = fmaxf(mrow[v], sink);
         const float cm = expf(mrow[v] - M);
         const float L = lrow[v] * cm + (p.sink ? expf(sink - M) : 0.f);
-        const float f = cm / L * p.out_scale;
+        const float f = cm / L * head_out_scale(p, t0 + r, h);
 #pragma unroll
         for (int n = 0; n < NV; ++n) {
             const size_t base = (size_t)(t0 + r) * p.ldo + p.out_off + (size_t)(oh0 + n) * vd;
@@ -1013,7 +1038,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
             for (int kt = 0; kt < 4; ++kt) {
                 const int key = key_at(j0 + kt * 16 + m16);
                 const bool ok_ = r < nq && key <= qpos && (key >= low[v] || key < p.keep);
-                sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - (p.dist ? dist_bias(r1, r2, qpos - key) : 0.f) : -INFINITY;
+                sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - distance_off(p, r1, r2, qpos - key) : -INFINITY;
                 mx[v] = fmaxf(mx[v], sc[v][kt]);
             }
 #pragma unroll
@@ -1060,7 +1085,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
         const float M = fmaxf(mrow[v], sink);
         const float cm = expf(mrow[v] - M);
         const float L = lrow[v] * cm + (p.sink ? expf(sink - M) : 0.f);
-        const float f = cm / L * p.out_scale;
+        const float f = cm / L * head_out_scale(p, t0 + r, h);
         const size_t base = (size_t)(t0 + r) * p.ldo + p.out_off + (size_t)h * vd;
 #pragma unroll
         for (int c = 0; c < VT; ++c) {
@@ -1312,9 +1337,9 @@ template <int DP, int LPC, int CH> __global__ __launch_bounds__(256) void delta_
         for (int r = 0; r < DP; ++r) { const int i = part * DP + r; if (i < d) stt[(size_t)i * vd + col] = S[r]; }
 }
 
-// out = o / rms(o) * w * gate * out_scale, one wave per (token, head)
+// out = o / rms(o) * w * gate * out_scale, one wave per (token, head); head h's weights start at w + h w_ld
 template <typename TO> __global__ __launch_bounds__(64) void gated_norm_kernel(TO* out, int ldo, int out_off, const float* o, const float* w,
-                                                                              const float* gate_in, int ldg, int gate, int H, int vd,
+                                                                              const float* gate_in, int ldg, int gate, int H, int vd, int w_ld,
                                                                               float eps, float out_scale) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const float* orow = o + ((size_t)t * H + h) * vd;
@@ -1325,7 +1350,7 @@ template <typename TO> __global__ __launch_bounds__(64) void gated_norm_kernel(T
     for (int i = lane; i < vd; i += 64) {
         const float gi = gate_in[(size_t)t * ldg + h * vd + i];
         const float gt = gate == MI355_HYB_GATE_SILU ? siluf_(gi) : sigmoidf_(gi);
-        st<TO>(out, (size_t)t * ldo + out_off + h * vd + i, orow[i] * inv * w[i] * gt * out_scale);
+        st<TO>(out, (size_t)t * ldo + out_off + h * vd + i, orow[i] * inv * w[h * w_ld + i] * gt * out_scale);
     }
 }
 
@@ -1435,24 +1460,26 @@ struct WholePrepArgs {
     const float* src; int ld, q_off, k_off, v_off;
     const float* qw; const float* kw; const int64_t* slots;
     int H, G, d, vd, v_unit; float eps;
+    const int64_t* positions; float temp_coef, temp_every;   // as in PrepArgs
 };
 // One workgroup per token.  q and k: ONE RMS norm over the whole row part (all heads at once), weights of that size; v: every head
-// divided by its own root mean square (no weight).  q -> q_out, k and v -> the token's page row.  No rotation.
-template <typename TC> __global__ __launch_bounds__(256) void attn_prepare_whole_kernel(WholePrepArgs p) {
-    __shared__ float red[4];
+// divided by its own root mean square (no weight).  q -> q_out, k and v -> the token's page row (k_pages NULL: nothing is cached).  No
+// rotation.
+template <typename TC> __global__ __launch_bounds__(1024) void attn_prepare_whole_kernel(WholePrepArgs p) {
+    __shared__ float red[16];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const float* row = p.src + (size_t)t * p.ld;
     const int nq = p.H * p.d, nk = p.G * p.d;
     const int64_t slot = p.slots[t];
     float sq = 0.f, sk = 0.f;
     if (p.qw) for (int i = threadIdx.x; i < nq; i += blockDim.x) { const float v = row[p.q_off + i]; sq = fmaf(v, v, sq); }
-    if (p.kw) for (int i = threadIdx.x; i < nk; i += blockDim.x) { const float v = row[p.k_off + i]; sk = fmaf(v, v, sk); }
+    if (p.kw && p.k_pages) for (int i = threadIdx.x; i < nk; i += blockDim.x) { const float v = row[p.k_off + i]; sk = fmaf(v, v, sk); }
     sq = block_sum(sq, red);
     sk = block_sum(sk, red);
-    const float iq = p.qw ? 1.f / sqrtf(sq / (float)nq + p.eps) : 1.f, ik = p.kw ? 1.f / sqrtf(sk / (float)nk + p.eps) : 1.f;
+    const float iq = (p.qw ? 1.f / sqrtf(sq / (float)nq + p.eps) : 1.f) * (p.temp_coef != 0.f ? query_temp(p.temp_coef, p.temp_every, p.positions[t]) : 1.f), ik = p.kw ? 1.f / sqrtf(sk / (float)nk + p.eps) : 1.f;
     TC* qd = static_cast<TC*>(p.q_out) + (size_t)t * nq;
     for (int i = threadIdx.x; i < nq; i += blockDim.x) st<TC>(qd, i, row[p.q_off + i] * iq * (p.qw ? p.qw[i] : 1.f));
-    if (slot < 0) return;
+    if (slot < 0 || !p.k_pages) return;
     TC* kd = static_cast<TC*>(p.k_pages) + (size_t)slot * nk;
     for (int i = threadIdx.x; i < nk; i += blockDim.x) st<TC>(kd, i, row[p.k_off + i] * ik * (p.kw ? p.kw[i] : 1.f));
     TC* vdst = static_cast<TC*>(p.v_pages) + (size_t)slot * p.G * p.vd;
@@ -1792,14 +1819,26 @@ int mi355_hyb_fill_f32(float* out, float v, int64_t n, int64_t stream) {
 }
 
 // which build of a product kernel: with an activation or a 16-bit result, or the plain one
-#define LIN_EPI(p, CALL) do { if ((p).act || (p).out16) { constexpr bool EPI = true; CALL; } else { constexpr bool EPI = false; CALL; } } while (0)
+#define LIN_EPI(p, CALL) do { if ((p).n_seg) { constexpr int EPI = LIN_SEG_BUILD; CALL; } else if ((p).act || (p).out16) { constexpr int EPI = LIN_EPI_BUILD; CALL; } \
+                              else { constexpr int EPI = LIN_PLAIN; CALL; } } while (0)
+// (the experts' products have no segments)
+#define LIN_EPI2(p, CALL) do { if ((p).act || (p).out16) { constexpr int EPI = LIN_EPI_BUILD; CALL; } else { constexpr int EPI = LIN_PLAIN; CALL; } } while (0)
+struct LinSegments { int32_t n, first; int64_t a_stride; const int32_t* rows; };
 static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, int32_t a_dtype, int32_t lda, int64_t a_bs, const void* w,
                          int64_t w_bs, const float* bias, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream,
-                         int32_t act = 0, int32_t act_cols = 0, int32_t out16 = 0) {
+                         int32_t act = 0, int32_t act_cols = 0, int32_t out16 = 0, const LinSegments* seg = nullptr) {
     if (!out || !a || !w || T < 0 || n <= 0 || k <= 0 || ldo < n || lda < k || batch <= 0 || batch > 65535 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
     if (T == 0) return 0;
     LinArgs p{out, ldo, a, lda, w, bias, T, n, k, 0, 0, a_bs, w_bs, o_bs};
     p.act = act; p.act_cols = act_cols; p.out16 = out16;
+    if (seg) {
+        if (seg->n < 1 || seg->n > LIN_MAX_SEG || seg->first < 0 || seg->a_stride < 0 || !seg->rows || batch != 1 || act || out16) return -1;
+        int end = 0;
+        for (int i = 0; i < seg->n; ++i) { if (seg->rows[i] <= 0 || seg->rows[i] % 128) return -1; end += seg->rows[i]; p.seg_end[i] = end; }
+        if (end != n) return -1;
+        p.n_seg = seg->n; p.seg0 = seg->first; p.seg_a = seg->a_stride;
+        a_bs = seg->a_stride;                                           // (its alignment counts like a batch's)
+    }
     hipStream_t st_ = to_stream(stream);
     const unsigned nz = (unsigned)batch;
     if (dtype == MI355_DTYPE_F32) {
@@ -1841,6 +1880,12 @@ int mi355_hyb_linear_batched(float* out, int32_t ldo, int64_t o_bs, const void* 
                              const void* w, int64_t w_bs, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream) {
     if (o_bs < 0 || a_bs < 0 || w_bs < 0) return -1;
     return linear_launch(out, ldo, o_bs, a, a_dtype, lda, a_bs, w, w_bs, nullptr, T, n, k, batch, dtype, stream);
+}
+
+int mi355_hyb_linear_segments(float* out, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, int64_t a_stride, int32_t first, const void* w,
+                              const float* bias, const int32_t* seg_rows, int32_t n_seg, int32_t T, int32_t n, int32_t k, int32_t dtype, int64_t stream) {
+    const LinSegments seg{n_seg, first, a_stride, seg_rows};
+    return linear_launch(out, ldo, 0, a, a_dtype, lda, 0, w, 0, bias, T, n, k, 1, dtype, stream, 0, 0, 0, &seg);
 }
 
 int mi355_hyb_embed(float* x, void* xcopy, const void* table, const uint32_t* ids, int32_t T, int32_t width, int32_t vocab, int32_t dtype,
@@ -1894,14 +1939,24 @@ int mi355_hyb_attn_prepare_ex(void* q_out, void* k_pages, void* v_pages, const f
                               const int64_t* positions, const int64_t* slot_mapping, int32_t T, int32_t heads, int32_t kv_heads,
                               int32_t dim, int32_t vdim, int32_t rot_dims, int32_t interleaved, int32_t norm_mode,
                               const float* q_head_scale, float eps, int32_t dtype, int64_t stream) {
-    if (norm_mode < 0 || norm_mode > 2) return -1;
-    if (!q_out || !k_pages || !v_pages || !proj || !positions || !slot_mapping || !is_dt(dtype)) return -1;
+    if (!k_pages || !v_pages) return -1;
+    return mi355_hyb_attn_prepare_temp(q_out, k_pages, v_pages, proj, ldp, q_off, k_off, v_off, q_norm_w, k_norm_w, cos_t, sin_t, positions, slot_mapping,
+                                       T, heads, kv_heads, dim, vdim, rot_dims, interleaved, norm_mode, q_head_scale, 0.f, 1.f, eps, dtype, stream);
+}
+
+int mi355_hyb_attn_prepare_temp(void* q_out, void* k_pages, void* v_pages, const float* proj, int32_t ldp, int32_t q_off, int32_t k_off,
+                                int32_t v_off, const float* q_norm_w, const float* k_norm_w, const float* cos_t, const float* sin_t,
+                                const int64_t* positions, const int64_t* slot_mapping, int32_t T, int32_t heads, int32_t kv_heads,
+                                int32_t dim, int32_t vdim, int32_t rot_dims, int32_t interleaved, int32_t norm_mode, const float* q_head_scale,
+                                float temp_coef, float temp_every, float eps, int32_t dtype, int64_t stream) {
+    if (norm_mode < 0 || norm_mode > 2 || (temp_coef != 0.f && !(temp_every > 0.f)) || (!k_pages != !v_pages)) return -1;
+    if (!q_out || !proj || !positions || !slot_mapping || !is_dt(dtype)) return -1;
     if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || vdim <= 0 || rot_dims < 0 || rot_dims > dim || (rot_dims & 1)) return -1;
     if (rot_dims > 0 && (!cos_t || !sin_t)) return -1;
     if (T <= 0) return 0;
     PrepArgs p{q_out, k_pages, v_pages, proj, ldp, q_off, k_off, v_off, q_norm_w, k_norm_w, cos_t, sin_t, positions, slot_mapping,
-               heads, kv_heads, dim, vdim, rot_dims, eps, interleaved, norm_mode, q_head_scale};
-    const dim3 grid(T, heads + 2 * kv_heads);
+               heads, kv_heads, dim, vdim, rot_dims, eps, interleaved, norm_mode, q_head_scale, temp_coef, temp_every};
+    const dim3 grid(T, heads + (k_pages ? 2 * kv_heads : 0));      // (no pages: the queries only)
     if (dtype == MI355_DTYPE_F32) attn_prepare_kernel<float><<<grid, 64, 2 * dim * sizeof(float), to_stream(stream)>>>(p);
     else attn_prepare_kernel<uint16_t><<<grid, 64, 2 * dim * sizeof(float), to_stream(stream)>>>(p);
     LAUNCH_OK(); return 0;
@@ -1956,6 +2011,18 @@ int mi355_hyb_attention(void* out, int32_t out_dtype, int32_t ldo, int32_t out_o
                         int32_t vdim, int32_t block_size, int32_t max_blocks, int32_t mask_kind, int32_t window, int32_t keep_first,
                         float scale, float out_scale, int32_t k_ld, int32_t v_ld, float softcap, int32_t cross_values, int32_t dtype,
                         int64_t stream) {
+    return mi355_hyb_attention_ex(out, out_dtype, ldo, out_off, q, k_pages, v_pages, block_tables, context_lens, cu_seqlens_q, tok_seq, sink, dist, 0,
+                                  nullptr, 0, num_seqs, T, heads, kv_heads, dim, vdim, block_size, max_blocks, mask_kind, window, keep_first, scale,
+                                  out_scale, k_ld, v_ld, softcap, cross_values, dtype, stream);
+}
+
+int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const void* q, const void* k_pages, const void* v_pages,
+                           const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_seqlens_q, const int32_t* tok_seq,
+                           const float* sink, const float* dist, int32_t dist_linear, const float* gate, int32_t ldg, int32_t num_seqs, int32_t T,
+                           int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int32_t max_blocks, int32_t mask_kind,
+                           int32_t window, int32_t keep_first, float scale, float out_scale, int32_t k_ld, int32_t v_ld, float softcap,
+                           int32_t cross_values, int32_t dtype, int64_t stream) {
+    if (gate && ldg < heads) return -1;
     if (keep_first < 0 || mask_kind < MI355_HYB_MASK_SLIDING || mask_kind > MI355_HYB_MASK_CHUNKED) return -1;
     if (!out || !q || !k_pages || !v_pages || !block_tables || !context_lens || !cu_seqlens_q || !tok_seq) return -1;
     if (!is_dt(dtype) || !is_dt(out_dtype) || heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || vdim <= 0) return -1;
@@ -1977,6 +2044,8 @@ int mi355_hyb_attention(void* out, int32_t out_dtype, int32_t ldo, int32_t out_o
     p.keep = window > 0 ? keep_first : 0;
     p.dist = dist;
     p.chunked = mask_kind == MI355_HYB_MASK_CHUNKED;
+    p.dist_linear = dist_linear ? 1 : 0;
+    p.gate = gate; p.ldg = ldg;
     if (vec) { int c = 1; while (c < vdim / epv) c <<= 1; p.cp2 = c; c = 1; while (c < dim / epv) c <<= 1; p.cpk = c; }
     else if (vdim > 512) return -1;
     // prompt-sized steps over bf16 pages: the matrix-core kernel (a tile of 16 tokens never spans two sequences)
@@ -2010,7 +2079,7 @@ int mi355_hyb_attention(void* out, int32_t out_dtype, int32_t ldo, int32_t out_o
                                    default: ok_shape = false; } } while (0)
         bool ok_shape = true;
         if (vt > 8) {
-            switch (dk) { case 4: WMW(4); break; case 5: WMW(5); break; case 6: WMW(6); break; case 7: WMW(7); break; case 8: WMW(8); break;
+            switch (dk) { case 1: WMW(1); break; case 2: WMW(2); break; case 3: WMW(3); break; case 4: WMW(4); break; case 5: WMW(5); break; case 6: WMW(6); break; case 7: WMW(7); break; case 8: WMW(8); break;
                           default: ok_shape = false; }
         } else {
             switch (dk) { case 1: WMV(1, WMN); break; case 2: WMV(2, WMN); break; case 3: WMV(3, WMN); break; case 4: WMV(4, WMN); break;
@@ -2130,11 +2199,17 @@ int mi355_hyb_delta_rule(float* o, float* state, int64_t state_stride, const flo
 int mi355_hyb_gated_norm(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const float* o, const float* w,
                          const float* gate_in, int32_t ldg, int32_t gate, int32_t T, int32_t heads, int32_t vdim, float eps,
                          float out_scale, int64_t stream) {
-    if (!out || !o || !w || !gate_in || !is_dt(out_dtype) || heads <= 0 || vdim <= 0) return -1;
+    return mi355_hyb_gated_norm_heads(out, out_dtype, ldo, out_off, o, w, 0, gate_in, ldg, gate, T, heads, vdim, eps, out_scale, stream);
+}
+
+int mi355_hyb_gated_norm_heads(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const float* o, const float* w, int32_t w_ld,
+                               const float* gate_in, int32_t ldg, int32_t gate, int32_t T, int32_t heads, int32_t vdim, float eps,
+                               float out_scale, int64_t stream) {
+    if (!out || !o || !w || !gate_in || !is_dt(out_dtype) || heads <= 0 || vdim <= 0 || w_ld < 0) return -1;
     if (T <= 0) return 0;
     const dim3 grid(T, heads);
-    if (out_dtype == MI355_DTYPE_F32) gated_norm_kernel<float><<<grid, 64, 0, to_stream(stream)>>>((float*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, eps, out_scale);
-    else gated_norm_kernel<uint16_t><<<grid, 64, 0, to_stream(stream)>>>((uint16_t*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, eps, out_scale);
+    if (out_dtype == MI355_DTYPE_F32) gated_norm_kernel<float><<<grid, 64, 0, to_stream(stream)>>>((float*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, w_ld, eps, out_scale);
+    else gated_norm_kernel<uint16_t><<<grid, 64, 0, to_stream(stream)>>>((uint16_t*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, w_ld, eps, out_scale);
     LAUNCH_OK(); return 0;
 }
 
@@ -2188,13 +2263,25 @@ int mi355_hyb_attn_prepare_whole(void* q_out, void* k_pages, void* v_pages, cons
                                  int32_t v_off, const float* q_norm_w, const float* k_norm_w, const int64_t* slot_mapping, int32_t T,
                                  int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t v_unit, float eps, int32_t dtype,
                                  int64_t stream) {
-    if (!q_out || !k_pages || !v_pages || !src || !slot_mapping || !is_dt(dtype)) return -1;
+    if (!k_pages || !v_pages) return -1;
+    return mi355_hyb_attn_prepare_whole_temp(q_out, k_pages, v_pages, src, ld, q_off, k_off, v_off, q_norm_w, k_norm_w, nullptr, slot_mapping, T, heads,
+                                             kv_heads, dim, vdim, v_unit, 0.f, 1.f, eps, dtype, stream);
+}
+
+int mi355_hyb_attn_prepare_whole_temp(void* q_out, void* k_pages, void* v_pages, const float* src, int32_t ld, int32_t q_off, int32_t k_off,
+                                      int32_t v_off, const float* q_norm_w, const float* k_norm_w, const int64_t* positions,
+                                      const int64_t* slot_mapping, int32_t T, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim,
+                                      int32_t v_unit, float temp_coef, float temp_every, float eps, int32_t dtype, int64_t stream) {
+    if (!q_out || (!k_pages != !v_pages) || !src || !slot_mapping || !is_dt(dtype)) return -1;
+    if (temp_coef != 0.f && (!positions || !(temp_every > 0.f))) return -1;
     if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || vdim <= 0) return -1;
     if (T <= 0) return 0;
     WholePrepArgs p{q_out, k_pages, v_pages, src, ld, q_off, k_off, v_off, q_norm_w, k_norm_w, slot_mapping, heads, kv_heads, dim, vdim,
-                    v_unit ? 1 : 0, eps};
-    if (dtype == MI355_DTYPE_F32) attn_prepare_whole_kernel<float><<<T, 256, 0, to_stream(stream)>>>(p);
-    else attn_prepare_whole_kernel<uint16_t><<<T, 256, 0, to_stream(stream)>>>(p);
+                    v_unit ? 1 : 0, eps, positions, temp_coef, temp_every};
+    // few tokens (decoding batches): sixteen waves per token
+    const int nt = (T <= 64 && (heads + kv_heads) * dim > 1024) ? 1024 : 256;
+    if (dtype == MI355_DTYPE_F32) attn_prepare_whole_kernel<float><<<T, nt, 0, to_stream(stream)>>>(p);
+    else attn_prepare_whole_kernel<uint16_t><<<T, nt, 0, to_stream(stream)>>>(p);
     LAUNCH_OK(); return 0;
 }
 
@@ -2331,7 +2418,7 @@ int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, cons
     hipStream_t st_ = to_stream(stream);
     if (dtype == MI355_DTYPE_F32) {
         if (a_dtype != MI355_DTYPE_F32 || block_rows != 64) return -1;
-        LIN_EPI(p, (linear_f32_kernel<EPI><<<dim3((n + 63) / 64, n_blocks, 1), 256, 0, st_>>>(p)));
+        LIN_EPI2(p, (linear_f32_kernel<EPI><<<dim3((n + 63) / 64, n_blocks, 1), 256, 0, st_>>>(p)));
         LAUNCH_OK(); return 0;
     }
     const int a_bytes = a_dtype == MI355_DTYPE_F32 ? 4 : 2;
@@ -2340,13 +2427,13 @@ int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, cons
     const bool af = a_dtype == MI355_DTYPE_F32;
     if (block_rows == 16) {
         const dim3 grid((n + 15) / 16, n_blocks, 1);
-        if (k >= 2048) { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
-        else { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
+        if (k >= 2048) { if (af) LIN_EPI2(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
+        else { if (af) LIN_EPI2(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
     } else if (block_rows == 64) {
         const dim3 grid((n + 63) / 64, n_blocks, 1);
-        if (af) LIN_EPI(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
+        if (af) LIN_EPI2(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
     } else if (block_rows == 128 && !af && p.a_vec && p.w_vec && k % 32 == 0) {
-        LIN_EPI(p, (linear_bf16_lds_kernel<EPI><<<dim3((n + 127) / 128, n_blocks, 1), 256, 0, st_>>>(p)));
+        LIN_EPI2(p, (linear_bf16_lds_kernel<EPI><<<dim3((n + 127) / 128, n_blocks, 1), 256, 0, st_>>>(p)));
     } else {
         return -1;
     }

@@ -6,14 +6,17 @@
 // added to the mixer's input; residual_form 3 has ONE norm per layer that mixer and feed-forward both read, x <- x + mixer(h) + ff(h),
 // then the token's side input and the average over the depth (a state-space mixer and an ungated feed-forward belong to that form's
 // design); residual_form 4 carries the residual stream in several copies that every sublayer mixes (chunked attention and linear attention
-// with a constant decay belong to that form's design).  The feed-forward is a dense form with or without a gate or a mixture of experts
+// with a constant decay belong to that form's design); residual_form 5 gives both sublayers a norm of their own of the same x,
+// x <- x + (mixer(norm1(x)) + ff(norm2(x))) (time mixing beside attention belongs to that form's design).  The feed-forward is a dense form with or without a gate or a mixture of experts
 // (router, grouped expert products over device-built blocks, shared expert).  A layer may run on another layer's weights (share_with)
 // and still owns its pages and state.  Like the llama-family host layers
 // (host_model.cpp, dense_model.cpp) it owns the weights, the K/V pages and the activation buffers and enqueues one step on a
 // stream; unlike them it owns a pool of recurrent state (one slot per live sequence, handed out by the block engine) and runs
 // prompts, portions of prompts and decoded tokens through the same launches.
-// Kernels: hybrid_kernels.hip, hybrid_blocks.hip, hybrid_streams.hip.  Every projection that reads a mixer's input is one matrix (rows concatenated at load time), the
+// Kernels: hybrid_kernels.hip, hybrid_blocks.hip, hybrid_streams.hip, hybrid_timemix.hip.  Every projection that reads a mixer's input is one matrix (rows concatenated at load time), the
 // output projections of a parallel mixer are one matrix along k (the branch scales are applied to the operands, not the weights).
+// Time mixing reads a different mixture per projection: its rows follow in the same matrix in segments of whole 128-row tiles, one left
+// operand per segment, so that the layer's projections are still one launch.
 #include <hip/hip_runtime.h>
 #include <algorithm>
 #include <cmath>
@@ -41,6 +44,9 @@ namespace {
 #define HCHECK(expr) do { const int rc_ = (expr); if (rc_ != 0) return rc_; } while (0)
 #define HHIP(expr) do { const hipError_t e_ = (expr); if (e_ != hipSuccess) return (int)e_; } while (0)
 
+// time mixing: what a segment of the input projection reads -- h itself, then its mixtures for r, k, v, gate, decay
+constexpr int TIMEMIX_MIXES = 5, TIMEMIX_SEGMENTS = TIMEMIX_MIXES + 1;
+
 enum { P_AQ = 0, P_AK, P_AV, P_DQ, P_DK, P_DV, P_B, P_A, P_G, P_COUNT };   // parts of the input projection (minGRU: z, x, g in 0..2)
 
 struct Weight { void* p = nullptr; int64_t n = 0; };
@@ -54,11 +60,15 @@ struct HLayer {
     void *k_pages = nullptr, *v_pages = nullptr;
     int64_t conv_off = 0, state_off = 0;          // floats from the start of a slot
     int64_t in_conv_off = 0;                      // the input convolution's last rows
-    bool has_attn() const { return c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION; }
+    int64_t row_off = 0;                          // time mixing: the last token's h
+    int32_t seg_rows[TIMEMIX_SEGMENTS] = {}, n_seg = 0;   // segments of the input projection (has_timemix)
+    bool has_attn() const { return c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX; }
+    bool side_by_side() const { return c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX; }
     bool has_delta() const { return c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_DELTA; }
     bool is_latent() const { return c.mixer == MI355_HYB_MIX_LATENT; }
     bool is_conv_attn() const { return c.mixer == MI355_HYB_MIX_CONV_ATTENTION; }
     bool is_ssd() const { return c.mixer == MI355_HYB_MIX_SSD; }
+    bool has_timemix() const { return c.mixer == MI355_HYB_MIX_TIMEMIX || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX; }
     bool is_decay() const { return c.mixer == MI355_HYB_MIX_DECAY; }
     int gate_up_rows() const { return (c.mlp_kind == 4 || c.mlp_kind == 5 || (c.mlp_kind == 3 && c.moe_relu2)) ? 1 : 2; }   // in units of the size
     bool uses_pages() const { return has_attn() || is_latent() || is_conv_attn(); }
@@ -100,6 +110,12 @@ struct HModel {
     int64_t bigram_off = 0;
     Weight bigram;
     bool need_hf = false, need_xs = false;
+    // form 5: the residual's second buffer (a layer reads one and writes the other), what the mixer reads (h and its mixtures), the last
+    // tokens' h on their way into the slots, the decays' logarithms
+    float *x2 = nullptr, *h_last = nullptr, *log_w = nullptr;
+    void* mix_in = nullptr;
+    bool need_mixes = false;
+    int max_log_w = 0, cap_seqs = 0;
     int max_side = 0, max_q_rank = 0;
     float *moe_gu = nullptr, *moe_y = nullptr, *moe_wts = nullptr, *moe_sgate = nullptr;
     int32_t *moe_ids = nullptr, *moe_pos = nullptr, *moe_row_token = nullptr, *moe_table = nullptr;
@@ -123,9 +139,10 @@ void drop_graphs(HModel* m) {
     m->graphs.clear();
 }
 
-int in_proj_parts(const mi355_hybrid_layer& c, int32_t* off) {
+// segments: NULL, or receives the rows of every segment of a time-mixing layer's projection (n_seg of them)
+int in_proj_parts(const mi355_hybrid_layer& c, int32_t* off, int32_t* segments = nullptr, int32_t* n_seg = nullptr) {
     for (int i = 0; i < P_COUNT; ++i) off[i] = -1;
-    int r = 0;
+    int r = 0, ns = 0;
     if (c.mixer == MI355_HYB_MIX_MINGRU) {
         off[0] = 0; off[1] = c.g_width; off[2] = 2 * c.g_width;
         return 3 * c.g_width;
@@ -146,12 +163,28 @@ int in_proj_parts(const mi355_hybrid_layer& c, int32_t* off) {
         off[P_DQ] = 0; off[P_DK] = c.d_heads * c.d_dim; off[P_DV] = 2 * c.d_heads * c.d_dim; off[P_G] = off[P_DV] + c.d_heads * c.d_vdim;
         return off[P_G] + c.d_heads * c.d_vdim;
     }
-    if (c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION || c.mixer == MI355_HYB_MIX_CONV_ATTENTION) {
+    if (c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION || c.mixer == MI355_HYB_MIX_CONV_ATTENTION ||
+        c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX) {
         off[P_AQ] = r; r += c.a_heads * c.a_dim;
-        off[P_AK] = r; r += c.a_kv_heads * c.a_dim;
-        if (c.a_v_is_k) off[P_AV] = off[P_AK];
-        else { off[P_AV] = r; r += c.a_kv_heads * c.a_vdim; }
+        if (!c.kv_from) {
+            off[P_AK] = r; r += c.a_kv_heads * c.a_dim;
+            if (c.a_v_is_k) off[P_AV] = off[P_AK];
+            else { off[P_AV] = r; r += c.a_kv_heads * c.a_vdim; }
+        }
+        if (c.a_head_gate) { off[P_G] = r; r += c.a_heads; }
     }
+    if (c.mixer == MI355_HYB_MIX_TIMEMIX || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX) {   // every part ends on a whole 128-row tile
+        const int part[TIMEMIX_MIXES] = {P_DQ, P_DK, P_DV, P_B, P_A};
+        const int rows[TIMEMIX_MIXES] = {c.d_heads * c.d_dim, c.d_heads * c.d_dim, c.d_heads * c.d_vdim, c.d_heads * c.d_vdim, c.d_a_rank};
+        if (r) { const int n = (r + 127) / 128 * 128; if (segments) segments[ns] = n; ++ns; r = n; }
+        for (int i = 0; i < TIMEMIX_MIXES; ++i) {
+            const int n = (rows[i] + 127) / 128 * 128;
+            off[part[i]] = r; r += n;
+            if (segments) segments[ns] = n;
+            ++ns;
+        }
+    }
+    if (n_seg) *n_seg = ns;
     if (c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_DELTA) {
         off[P_DQ] = r; r += c.d_kv_heads * c.d_dim;
         off[P_DK] = r; r += c.d_kv_heads * c.d_dim;
@@ -164,9 +197,13 @@ int in_proj_parts(const mi355_hybrid_layer& c, int32_t* off) {
 }
 
 bool layer_ok(const mi355_hybrid_layer& c) {
-    const bool attn = c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION;
+    const bool timemix = c.mixer == MI355_HYB_MIX_TIMEMIX || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX;
+    const bool attn = c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_ATTENTION || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX;
     const bool delta = c.mixer == MI355_HYB_MIX_PARALLEL || c.mixer == MI355_HYB_MIX_DELTA;
-    if (c.mixer < 0 || c.mixer > MI355_HYB_MIX_DECAY || c.share_with < 0) return false;
+    if (c.mixer < 0 || c.mixer > MI355_HYB_MIX_PARALLEL_TIMEMIX || c.share_with < 0) return false;
+    if (timemix && (c.d_heads <= 0 || c.d_dim <= 0 || c.d_dim > 512 || c.d_vdim <= 0 || c.d_a_rank <= 0)) return false;
+    if (c.a_temp_coef != 0.f && (!attn || !(c.a_temp_every > 0.f))) return false;
+    if (attn && c.a_norm_whole && (c.a_rot_dims || c.a_norm_after_rot || c.a_head_temp || c.a_v_is_k)) return false;   // (that form does not rotate)
     if (c.mixer == MI355_HYB_MIX_DECAY && (c.d_heads <= 0 || c.d_dim <= 0 || c.d_dim > 512 || c.d_vdim <= 0)) return false;
     if (c.a_mask_kind < MI355_HYB_MASK_SLIDING || c.a_mask_kind > MI355_HYB_MASK_CHUNKED || ((c.a_mask_kind || c.a_v_is_k) && !attn)) return false;
     if (c.a_v_is_k && c.a_vdim != c.a_dim) return false;
@@ -176,9 +213,12 @@ bool layer_ok(const mi355_hybrid_layer& c) {
         if (c.d_conv < 1 || c.d_conv > 16 || c.d_norm_groups < 1 || (c.d_heads * c.d_vdim) % c.d_norm_groups) return false;
     }
     if (c.a_q_rank < 0 || c.kv_from < 0 || c.side_dim < 0 || c.side_col < 0 || c.depth_terms < 0 || c.moe_groups < 0) return false;
-    if ((c.a_q_rank || c.a_out_gate || c.kv_from) && c.mixer != MI355_HYB_MIX_LATENT) return false;
+    if ((c.a_q_rank || c.a_out_gate) && c.mixer != MI355_HYB_MIX_LATENT) return false;
+    if (c.kv_from && c.mixer != MI355_HYB_MIX_LATENT && !attn) return false;
+    if (c.a_head_gate && c.mixer != MI355_HYB_MIX_LATENT && !attn) return false;
     if (c.a_out_gate && c.a_head_gate) return false;
-    if (c.a_dist_bias && c.mixer != MI355_HYB_MIX_CONV_ATTENTION) return false;
+    if (c.mixer == MI355_HYB_MIX_PARALLEL && c.a_head_gate) return false;                // (the gate part is the delta rule's)
+    if (c.a_dist_bias < 0 || c.a_dist_bias > 2 || (c.a_dist_bias && c.mixer != MI355_HYB_MIX_CONV_ATTENTION && !attn)) return false;
     if (c.moe_groups > 0 && (c.mlp_kind != 3 || c.moe_experts % c.moe_groups || c.moe_keep_groups < 1 || c.moe_keep_groups > c.moe_groups ||
                              (c.moe_experts / c.moe_groups) * c.moe_keep_groups < c.moe_top)) return false;
     if (c.mixer == MI355_HYB_MIX_LATENT) {
@@ -202,7 +242,7 @@ bool layer_ok(const mi355_hybrid_layer& c) {
         if (c.d_gate != MI355_HYB_GATE_SIGMOID_LR && c.d_gate != MI355_HYB_GATE_SILU) return false;
     }
     if (c.mixer == MI355_HYB_MIX_MINGRU && c.g_width <= 0) return false;
-    if (c.mlp_kind < 0 || c.mlp_kind > 5 || (c.mlp_kind && c.mlp_ff <= 0)) return false;
+    if (c.mlp_kind < 0 || c.mlp_kind > 6 || (c.mlp_kind && c.mlp_ff <= 0)) return false;
     if (c.mlp_kind == 3 && (c.moe_experts < 1 || c.moe_experts > 4096 || c.moe_top < 1 || c.moe_top > c.moe_experts || c.moe_shared_ff < 0)) return false;
     if (c.a_keep_first < 0 || c.in_conv < 0 || c.in_conv > 16) return false;
     if ((c.a_keep_first || c.a_norm_after_rot || c.a_head_temp) && !attn) return false;      // switches of the plain attention branch
@@ -235,10 +275,13 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
     if (c.share_with) return -1;                               // a layer that runs on another layer's weights holds none
     switch (which) {
         case MI355_HW_NORM1: return W;
+        case MI355_HW_T_MU: return L.has_timemix() ? (int64_t)TIMEMIX_MIXES * W : -1;
+        case MI355_HW_T_W2: return L.has_timemix() ? (int64_t)c.d_a_rank * c.d_heads * c.d_dim : -1;
+        case MI355_HW_T_W0: case MI355_HW_T_BONUS: return L.has_timemix() ? c.d_heads * c.d_dim : -1;
         case MI355_HW_NORM2: return c.mlp_kind && m->cfg.residual_form != 3 ? W : -1;
         case MI355_HW_D_SKIP: return L.is_ssd() ? c.d_heads : -1;
         case MI355_HW_CONV_BIAS: return L.is_ssd() ? L.ssd_channels() : -1;
-        case MI355_HW_A_DIST: return L.is_conv_attn() && c.a_dist_bias ? 2 * c.a_heads : -1;
+        case MI355_HW_A_DIST: return (L.is_conv_attn() || L.has_attn()) && c.a_dist_bias ? 2 * c.a_heads : -1;
         case MI355_HW_L_QNORM: return L.is_latent() && c.a_q_rank ? c.a_q_rank : -1;
         case MI355_HW_L_UQ: return L.is_latent() && c.a_q_rank ? (int64_t)c.a_heads * (c.a_dim + c.a_rot_dim) * c.a_q_rank : -1;
         case MI355_HW_SIDE_GATE: case MI355_HW_SIDE_PROJ: return c.side_dim ? (int64_t)c.side_dim * W : -1;
@@ -253,9 +296,10 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
         case MI355_HW_IN_PROJ: return (int64_t)L.in_rows * W;
         case MI355_HW_IN_BIAS: return L.in_rows;
         case MI355_HW_OUT_PROJ: return (int64_t)W * L.out_k;
-        case MI355_HW_A_QNORM: if (L.is_conv_attn()) return c.a_qk_norm ? c.a_heads * c.a_dim : -1;
+        case MI355_HW_A_QNORM: if (L.is_conv_attn() || (L.has_attn() && c.a_norm_whole)) return c.a_qk_norm ? c.a_heads * c.a_dim : -1;
                                return L.has_attn() && c.a_qk_norm && !c.a_norm_after_rot ? c.a_dim : -1;
-        case MI355_HW_A_KNORM: if (L.is_conv_attn()) return c.a_qk_norm ? c.a_kv_heads * c.a_dim : -1;
+        case MI355_HW_A_KNORM: if (c.kv_from) return -1;
+                               if (L.is_conv_attn() || (L.has_attn() && c.a_norm_whole)) return c.a_qk_norm ? c.a_kv_heads * c.a_dim : -1;
                                return L.has_attn() && c.a_qk_norm && !c.a_norm_after_rot ? c.a_dim : -1;
         case MI355_HW_A_TEMP: return L.has_attn() && c.a_head_temp ? c.a_heads : -1;
         case MI355_HW_PRE_NORM1: return m->cfg.residual_form == 2 ? W : -1;
@@ -276,7 +320,7 @@ int64_t expected_elems(const HModel* m, int layer, int which) {
         case MI355_HW_D_A_LOG: return L.has_delta() || L.is_ssd() ? c.d_heads : -1;
         case MI355_HW_D_DT_BIAS: if (L.is_ssd()) return c.d_heads;
                                  return L.has_delta() ? (c.d_decay_channels ? c.d_heads * c.d_dim : c.d_heads) : -1;
-        case MI355_HW_D_NORM: if (L.is_ssd() || L.is_decay()) return L.ssd_inner();
+        case MI355_HW_D_NORM: if (L.is_ssd() || L.is_decay() || L.has_timemix()) return L.ssd_inner();
                               return L.has_delta() ? c.d_vdim : -1;
         case MI355_HW_D_A2: return L.has_delta() && c.d_decay_channels ? (int64_t)c.d_heads * c.d_dim * c.d_a_rank : -1;
         case MI355_HW_D_G2: return L.has_delta() && c.d_gate == MI355_HYB_GATE_SIGMOID_LR ? (int64_t)c.d_heads * c.d_vdim * c.d_g_rank : -1;
@@ -329,6 +373,12 @@ int ensure_capacity(HModel* m, int T, int n_out, int n_seqs) {
         HCHECK(grow(m->pieces, (size_t)pieces * 4));
         m->cap_pieces = pieces;
     }
+    if (m->need_mixes && n_seqs > m->cap_seqs) {
+        HHIP(hipDeviceSynchronize());
+        drop_graphs(m);
+        HCHECK(grow(m->h_last, (size_t)n_seqs * m->cfg.width * 4));
+        m->cap_seqs = n_seqs;
+    }
     if (T > m->cap_t) {
         const size_t t = (size_t)T, W = (size_t)m->cfg.width;
         HHIP(hipDeviceSynchronize());
@@ -351,7 +401,12 @@ int ensure_capacity(HModel* m, int T, int n_out, int n_seqs) {
         if (m->need_pre) HCHECK(grow(m->pre, t * W * m->esize()));
         if (m->cfg.residual_form == 4) HCHECK(grow(m->streams, t * W * m->cfg.streams * 4));
         if (m->cfg.bigram_buckets) HCHECK(grow(m->bigram_rows, t * 4));
-        if (m->cfg.residual_form == 3) HCHECK(grow(m->y2, t * W * 4));
+        if (m->cfg.residual_form == 3 || m->cfg.residual_form == 5) HCHECK(grow(m->y2, t * W * 4));
+        if (m->cfg.residual_form == 5) {
+            HCHECK(grow(m->x2, t * W * 4));
+            HCHECK(grow(m->mix_in, t * W * m->esize() * (m->need_mixes ? TIMEMIX_SEGMENTS : 1)));
+            if (m->need_mixes) HCHECK(grow(m->log_w, t * (size_t)m->max_log_w * 4));
+        }
         if (m->need_hf) HCHECK(grow(m->hf, t * W * 4));
         if (m->need_xs) HCHECK(grow(m->xs, (m->layers.size() + 1) * t * W * 4));
         if (m->max_side) { HCHECK(grow(m->side_g, t * (size_t)m->max_side * 4)); HCHECK(grow(m->side_a, t * (size_t)m->max_side * m->esize())); }
@@ -410,25 +465,34 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
         const mi355_hybrid_layer& c = layers[i];
         if (c.side_dim && c.side_col + c.side_dim > cfg->side_cols) return nullptr;
         if (c.depth_terms && c.depth_terms != i + 2) return nullptr;
-        if (c.mlp_kind == 4 && cfg->residual_form != 3 && cfg->residual_form != 4) return nullptr;
-        if ((c.mlp_kind == 5 || c.moe_relu2 || c.moe_bias || c.moe_shared_plain || c.mixer == MI355_HYB_MIX_DECAY) && cfg->residual_form != 4) return nullptr;
+        if (c.mlp_kind == 4 && cfg->residual_form < 3) return nullptr;
+        if ((c.moe_relu2 || c.moe_bias || c.moe_shared_plain || c.mixer == MI355_HYB_MIX_DECAY) && cfg->residual_form != 4) return nullptr;
+        if (c.mlp_kind == 5 && cfg->residual_form < 4) return nullptr;
         if (cfg->residual_form == 4 && (c.in_conv || c.side_dim || c.depth_terms || c.mlp_kind == 1 || c.mlp_kind == 2)) return nullptr;
         if (cfg->residual_form == 4 && c.mlp_kind == 3 && (!c.moe_relu2 || (c.moe_shared_ff && !c.moe_shared_plain))) return nullptr;
+        const bool timemix = c.mixer == MI355_HYB_MIX_TIMEMIX || c.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX;
+        if ((timemix || c.mlp_kind == 6) && cfg->residual_form != 5) return nullptr;
+        if (cfg->residual_form == 5 && (c.in_conv || c.side_dim || c.depth_terms || c.share_with || c.mlp_kind == 1 || c.moe_shared_ff || c.moe_relu2 || c.moe_bias ||
+                                        c.moe_shared_plain)) return nullptr;
         if (cfg->residual_form == 3 && (c.in_conv || c.share_with || c.moe_shared_ff || c.mlp_kind == 1 || c.mlp_kind == 2)) return nullptr;
-        if (c.kv_from) {                                            // the lender: an earlier latent layer with pages of its own and the same row
+        if (c.kv_from) {                                            // the lender: an earlier layer of the kind with pages of its own and the same rows
             if (c.kv_from > i) return nullptr;
             const mi355_hybrid_layer& b = layers[c.kv_from - 1];
-            if (b.mixer != MI355_HYB_MIX_LATENT || b.kv_from || b.a_kv_rank != c.a_kv_rank || b.a_rot_dim != c.a_rot_dim) return nullptr;
+            if (c.mixer != MI355_HYB_MIX_LATENT) {
+                const bool battn = b.mixer == MI355_HYB_MIX_PARALLEL || b.mixer == MI355_HYB_MIX_ATTENTION || b.mixer == MI355_HYB_MIX_PARALLEL_TIMEMIX;
+                if (!battn || b.kv_from || b.a_kv_heads != c.a_kv_heads || b.a_dim != c.a_dim || b.a_vdim != c.a_vdim || c.a_v_is_k) return nullptr;
+            } else if (b.mixer != MI355_HYB_MIX_LATENT || b.kv_from || b.a_kv_rank != c.a_kv_rank || b.a_rot_dim != c.a_rot_dim) return nullptr;
         }
     }
     if (cfg->residual_form == 4 && (cfg->streams < 1 || cfg->streams > 16 || cfg->width > 12288 || cfg->norm_groups > 1)) return nullptr;
     if (cfg->residual_form != 4 && (cfg->streams || cfg->bigram_buckets)) return nullptr;
     if (cfg->bigram_buckets < 0 || cfg->bigram_mul_prev < 0 || cfg->bigram_mul_cur < 0) return nullptr;
-    if (cfg->residual_form < 0 || cfg->residual_form > 4 || cfg->norm_groups < 0 || (cfg->norm_groups > 1 && cfg->width % cfg->norm_groups)) return nullptr;
+    if (cfg->residual_form < 0 || cfg->residual_form > 5 || cfg->norm_groups < 0 || (cfg->norm_groups > 1 && cfg->width % cfg->norm_groups)) return nullptr;
     for (int i = 0; i < cfg->n_layers; ++i)                        // the experts' outputs are combined in front of an output norm
         if (layers[i].mlp_kind == 3 && (cfg->residual_form == 1 || (cfg->residual_form < 3 && cfg->width > 4096))) return nullptr;
     HModel* m = new HModel();
     m->cfg = *cfg;
+    if (cfg->residual_form == 5 && (cfg->width > 16384 || cfg->norm_groups > 1)) { delete m; return nullptr; }
     m->need_pre = cfg->residual_form >= 2;
     m->layers.resize(cfg->n_layers);
     int64_t off = 0;
@@ -436,7 +500,7 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
         HLayer& L = m->layers[i];
         L.c = layers[i];
         const mi355_hybrid_layer& c = L.c;
-        L.in_rows = in_proj_parts(c, L.off);
+        L.in_rows = in_proj_parts(c, L.off, L.seg_rows, &L.n_seg);
         L.out_k = 0;
         if (L.uses_pages()) L.out_k += c.a_heads * c.a_vdim;
         if (L.has_delta()) L.out_k += c.d_heads * c.d_vdim;
@@ -457,6 +521,15 @@ void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_lay
             m->max_mix = std::max(m->max_mix, L.out_k);
             m->max_o = std::max(m->max_o, L.ssd_inner());
             L.state_off = off; off += (int64_t)c.d_heads * c.d_dim * c.d_vdim;
+        }
+        if (L.has_timemix()) {
+            L.out_k += L.ssd_inner();
+            m->max_mix = std::max(m->max_mix, L.out_k);
+            m->max_o = std::max(m->max_o, L.ssd_inner());
+            m->max_log_w = std::max(m->max_log_w, c.d_heads * c.d_dim);
+            m->need_mixes = true;
+            L.state_off = off; off += (int64_t)c.d_heads * c.d_dim * c.d_vdim;
+            L.row_off = off; off += cfg->width;
         }
         if (c.side_dim) m->max_side = std::max(m->max_side, c.side_dim);
         if (c.depth_terms) m->need_xs = true;
@@ -511,7 +584,7 @@ void mi355_hybrid_destroy(void* mp) {
     for (void* p : {m->embed.p, m->final_norm.p, m->head.p, (void*)m->state, (void*)m->prep, (void*)m->x, (void*)m->proj, (void*)m->aux1, (void*)m->aux2,
                     (void*)m->conv, (void*)m->o, (void*)m->y, (void*)m->gu, m->xcopy, m->q, m->mix, m->act, m->xn, m->att, (void*)m->tok_seq,
                     m->pre, m->moe_act, (void*)m->y2, (void*)m->hf, (void*)m->xs, (void*)m->side_g, m->side_a, m->cq, m->side_table.p,
-                    (void*)m->streams, (void*)m->pieces, (void*)m->bigram_rows, m->bigram.p, (void*)m->moe_gu, (void*)m->moe_y, (void*)m->moe_wts, (void*)m->moe_sgate, (void*)m->moe_ids,
+                    (void*)m->x2, (void*)m->h_last, (void*)m->log_w, m->mix_in, (void*)m->streams, (void*)m->pieces, (void*)m->bigram_rows, m->bigram.p, (void*)m->moe_gu, (void*)m->moe_y, (void*)m->moe_wts, (void*)m->moe_sgate, (void*)m->moe_ids,
                     (void*)m->moe_pos, (void*)m->moe_row_token, (void*)m->moe_table})
         if (p) (void)hipFree(p);
     delete m;
@@ -591,7 +664,7 @@ int mi355_hybrid_alloc_cache(void* mp, int32_t num_blocks) {
             HHIP(hipMemset(L.v_pages, 0, rows * L.v_row() * m->esize()));
         }
     }
-    for (HLayer& L : m->layers) if (L.c.kv_from) L.k_pages = m->layers[L.c.kv_from - 1].k_pages;
+    for (HLayer& L : m->layers) if (L.c.kv_from) { L.k_pages = m->layers[L.c.kv_from - 1].k_pages; L.v_pages = m->layers[L.c.kv_from - 1].v_pages; }
     const size_t sb = (size_t)m->slot_floats * 4 * m->cfg.state_slots;
     HCHECK(grow(m->state, sb));
     HHIP(hipMemset(m->state, 0, sb));
@@ -632,8 +705,9 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
     const bool sandwich = m->cfg.residual_form == 2;                // a norm in front of every sublayer: nothing reads a copy of x
     const bool parallel = m->cfg.residual_form == 3;                // one norm per layer, both sublayers read it
     const bool copies = m->cfg.residual_form == 4;                  // several residual streams, a norm in front of every sublayer
-    void* xcopy = (bf && !sandwich && !parallel && !copies) ? m->xcopy : nullptr;
-    void* xin = (sandwich || parallel || copies) ? m->pre : (bf ? m->xcopy : (void*)m->x);  // what the sublayers' first product reads
+    const bool pair = m->cfg.residual_form == 5;                    // a norm for the mixer and one for the feed-forward, both of the same x
+    void* xcopy = (bf && !sandwich && !parallel && !copies && !pair) ? m->xcopy : nullptr;
+    void* xin = (sandwich || parallel || copies || pair) ? m->pre : (bf ? m->xcopy : (void*)m->x);  // what the sublayers' first product reads
     const int xin_dt = bf ? MI355_DTYPE_BF16 : MI355_DTYPE_F32;
     const int64_t TW = (int64_t)T * W;
     HCHECK(mi355_hyb_token_seq(m->tok_seq, cu_seqlens_q, num_seqs, stream));
@@ -657,6 +731,38 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
                                      more ? weights(nl, nq == 1 ? MI355_HW_HC1_IN : MI355_HW_HC2_IN) : nullptr, norm, m->pre, dt,
                                      routes ? m->hf : nullptr, T, m->cfg.streams, W, eps, stream);
     };
+    // form 5: the end of layer li (-1: none yet) and the start of the next -- the residual moves from one buffer to the other, the next
+    // layer's two norms, and what its mixer reads: h alone, or h and its mixtures with the token before
+    float* xcur = m->x;
+    auto pair_step = [&](int li, const float* y1, const float* y2, bool experts, int top) -> int {
+        const bool more = li + 1 < (int)m->layers.size();
+        const HLayer* N = more ? &m->layers[li + 1] : nullptr;
+        const bool mixes = more && N->has_timemix(), ff = more && N->c.mlp_kind;
+        auto w = [&](int which) { return more ? static_cast<const float*>(N->w[which].p) : nullptr; };
+        float* to = li < 0 ? nullptr : (xcur == m->x ? m->x2 : m->x);
+        HCHECK(mi355_hyb_pair_step(xcur, y1, y2, experts ? m->moe_y : nullptr, m->moe_pos, m->moe_wts, top, to, w(MI355_HW_NORM1),
+                                   ff ? w(MI355_HW_NORM2) : nullptr, m->mix_in, TW, m->pre, dt, (ff && N->c.mlp_kind == 3 && bf) ? m->hf : nullptr,
+                                   mixes ? w(MI355_HW_T_MU) : nullptr, mixes ? TIMEMIX_MIXES : 0, mixes ? m->state + N->row_off : nullptr,
+                                   m->slot_floats, m->h_last, context_lens, cu_seqlens_q, state_slots, m->tok_seq, T, W, eps, stream));
+        if (to) xcur = to;
+        return 0;
+    };
+    // the experts of a feed-forward without an output norm: routing on the f32 norm output, the pairs grouped, gate/up, silu, down -> moe_y
+    auto run_experts = [&](const mi355_hybrid_layer& c, const HLayer& WL) -> int {
+        const int E = c.moe_experts, K = c.moe_top, ff = c.mlp_ff, pairs = T * K;
+        HCHECK(mi355_hyb_moe_route_ex(m->moe_ids, m->moe_wts, nullptr, nullptr, dt, bf ? m->hf : static_cast<const float*>(m->pre), nullptr,
+                                      static_cast<const float*>(WL.w[MI355_HW_MOE_ROUTER].p), static_cast<const float*>(WL.w[MI355_HW_MOE_CORRECTION].p),
+                                      nullptr, T, W, E, K, c.moe_scale != 0.f ? c.moe_scale : 1.f, eps, 0, c.moe_sigmoid, c.moe_groups,
+                                      c.moe_keep_groups, c.moe_normalise, stream));
+        const int bm = std::min(mi355_hyb_moe_block_rows(pairs, E, 2 * ff, W, dt), mi355_hyb_moe_block_rows(pairs, E, W, ff, dt));
+        const int nb = (pairs + bm - 1) / bm + E;
+        HCHECK(mi355_hyb_moe_group(m->moe_pos, m->moe_row_token, m->moe_table, m->moe_ids, pairs, K, E, bm, nb, stream));
+        HCHECK(mi355_hyb_linear_grouped(m->moe_gu, 2 * ff, xin, xin_dt, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)2 * ff * W,
+                                        m->moe_table, bm, nb, 2 * ff, W, dt, stream));
+        HCHECK(mi355_hyb_silu_glu(m->moe_act, dt, m->moe_gu, nb * bm, ff, m->moe_table, bm, stream));
+        return mi355_hyb_linear_grouped(m->moe_y, W, m->moe_act, dt, ff, nullptr, WL.w[MI355_HW_MOE_DOWN].p, (int64_t)W * ff, m->moe_table, bm,
+                                        nb, W, ff, dt, stream);
+    };
     if (copies) {
         if (m->cfg.bigram_buckets)
             HCHECK(mi355_hyb_bigram_rows(m->bigram_rows, reinterpret_cast<int32_t*>(m->state + m->bigram_off), m->slot_floats, tokens, context_lens,
@@ -669,6 +775,7 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
         HCHECK(mi355_hyb_embed_scaled(m->x, m->embed.p, tokens, T, W, m->cfg.vocab, m->cfg.embed_scale, dt, stream));
     else
         HCHECK(mi355_hyb_embed(m->x, xcopy, m->embed.p, tokens, T, W, m->cfg.vocab, dt, stream));
+    if (pair) HCHECK(pair_step(-1, nullptr, nullptr, false, 0));
     if (m->need_xs) HCHECK(mi355_hyb_copy_f32(m->xs, m->x, TW, stream));         // X_0 of the depth average
     for (size_t li = 0; li < m->layers.size(); ++li) {
         HLayer& L = m->layers[li];
@@ -676,7 +783,7 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
         const HLayer& WL = c.share_with ? m->layers[c.share_with - 1] : L;          // whose weights (and rope tables) the layer runs on
         auto f = [&](int which) { return static_cast<const float*>(WL.w[which].p); };
         const int ldp = L.in_rows;
-        const void* min_ = xin;                                         // the mixer's input
+        const void* min_ = pair ? m->mix_in : xin;                      // the mixer's input
         if (c.in_conv) {
             // h + conv(h): h = the normed x (form 2) or x itself.  Up to 8 taps: norm, convolution (and, when every sequence brings one
             // token, the move of the slot's rows) are one launch; else the normed rows go through m->y (free until the output projection)
@@ -705,22 +812,31 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             HCHECK(mi355_hyb_pre_norm_ex(m->pre, dt, (c.mlp_kind == 3 && bf) ? m->hf : nullptr, m->x, W, f(MI355_HW_NORM1), T, W, m->cfg.norm_kind,
                                          eps, stream));
         }
-        // (constant-decay attention: silu on q, k, v, in the epilogue)
+        if (L.n_seg)                                                    // every segment of the projection reads its own mixture
+            HCHECK(mi355_hyb_linear_segments(m->proj, ldp, min_, xin_dt, W, TW, L.n_seg == TIMEMIX_SEGMENTS ? 0 : 1, WL.w[MI355_HW_IN_PROJ].p, nullptr,
+                                             L.seg_rows, L.n_seg, T, L.in_rows, W, dt, stream));
+        else                                                            // (constant-decay attention: silu on q, k, v, in the epilogue)
         HCHECK(mi355_hyb_linear_act(m->proj, MI355_DTYPE_F32, ldp, min_, xin_dt, W, WL.w[MI355_HW_IN_PROJ].p, f(MI355_HW_IN_BIAS), T, L.in_rows, W,
                                     L.is_decay() ? MI355_HYB_ACT_SILU : MI355_HYB_ACT_NONE, L.is_decay() ? L.off[P_G] : 0, dt, stream));
         int mix_col = 0;
         if (L.has_attn()) {
             const int norm_mode = c.a_qk_norm ? (c.a_norm_after_rot ? 2 : 1) : 0;
-            HCHECK(mi355_hyb_attn_prepare_ex(m->q, L.k_pages, L.v_pages, m->proj, ldp, L.off[P_AQ], L.off[P_AK], L.off[P_AV],
-                                             norm_mode == 1 ? f(MI355_HW_A_QNORM) : nullptr, norm_mode == 1 ? f(MI355_HW_A_KNORM) : nullptr,
-                                             WL.cos_t, WL.sin_t, positions, slot_mapping, T, c.a_heads, c.a_kv_heads, c.a_dim, c.a_vdim,
-                                             c.a_rot_dims, c.a_rot_interleaved, norm_mode, c.a_head_temp ? f(MI355_HW_A_TEMP) : nullptr, eps,
-                                             dt, stream));
-            HCHECK(mi355_hyb_attention(m->mix, dt, L.out_k, 0, m->q, L.k_pages, L.v_pages, block_tables, context_lens, cu_seqlens_q,
-                                       m->tok_seq, c.a_has_sink ? f(MI355_HW_A_SINK) : nullptr, nullptr, num_seqs, T, c.a_heads,
-                                       c.a_kv_heads, c.a_dim, c.a_vdim, m->cfg.block_size, max_blocks, c.a_mask_kind, c.a_window,
-                                       c.a_keep_first, c.a_scale, c.mixer == MI355_HYB_MIX_PARALLEL ? c.a_out_scale : 1.f, 0, 0, 0.f, 0, dt,
-                                       stream));
+            void *kp = c.kv_from ? nullptr : L.k_pages, *vp = c.kv_from ? nullptr : L.v_pages;      // (another layer's pages are read, not written)
+            const int k_off = c.kv_from ? 0 : L.off[P_AK], v_off = c.kv_from ? 0 : L.off[P_AV];
+            if (c.a_norm_whole)
+                HCHECK(mi355_hyb_attn_prepare_whole_temp(m->q, kp, vp, m->proj, ldp, L.off[P_AQ], k_off, v_off, f(MI355_HW_A_QNORM), f(MI355_HW_A_KNORM),
+                                                         positions, slot_mapping, T, c.a_heads, c.a_kv_heads, c.a_dim, c.a_vdim, c.a_v_unit, c.a_temp_coef,
+                                                         c.a_temp_every, eps, dt, stream));
+            else
+                HCHECK(mi355_hyb_attn_prepare_temp(m->q, kp, vp, m->proj, ldp, L.off[P_AQ], k_off, v_off, norm_mode == 1 ? f(MI355_HW_A_QNORM) : nullptr,
+                                                   norm_mode == 1 ? f(MI355_HW_A_KNORM) : nullptr, WL.cos_t, WL.sin_t, positions, slot_mapping, T,
+                                                   c.a_heads, c.a_kv_heads, c.a_dim, c.a_vdim, c.a_rot_dims, c.a_rot_interleaved, norm_mode,
+                                                   c.a_head_temp ? f(MI355_HW_A_TEMP) : nullptr, c.a_temp_coef, c.a_temp_every, eps, dt, stream));
+            HCHECK(mi355_hyb_attention_ex(m->mix, dt, L.out_k, 0, m->q, L.k_pages, L.v_pages, block_tables, context_lens, cu_seqlens_q,
+                                          m->tok_seq, c.a_has_sink ? f(MI355_HW_A_SINK) : nullptr, c.a_dist_bias ? f(MI355_HW_A_DIST) : nullptr,
+                                          c.a_dist_bias == 2, c.a_head_gate ? m->proj + L.off[P_G] : nullptr, ldp, num_seqs, T, c.a_heads,
+                                          c.a_kv_heads, c.a_dim, c.a_vdim, m->cfg.block_size, max_blocks, c.a_mask_kind, c.a_window,
+                                          c.a_keep_first, c.a_scale, L.side_by_side() ? c.a_out_scale : 1.f, 0, 0, c.a_softcap, 0, dt, stream));
             mix_col = c.a_heads * c.a_vdim;
         }
         if (L.is_latent()) {
@@ -796,6 +912,17 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
                                              c.d_vdim, by_pieces ? m->pieces : nullptr, stream));
             HCHECK(mi355_hyb_norm_sigmoid_gate(m->mix, dt, m->o, m->proj + L.off[P_G], ldp, f(MI355_HW_D_NORM), T, L.ssd_inner(), 1, eps, stream));
         }
+        if (L.has_timemix()) {
+            // the decays of the low-rank map, the recurrence over the state slot (which also takes the portions' last h), the norm per head
+            // with the gate
+            const int C = c.d_heads * c.d_dim;
+            HCHECK(mi355_hyb_lowrank_decay(m->log_w, C, m->proj + L.off[P_A], ldp, f(MI355_HW_T_W2), f(MI355_HW_T_W0), T, c.d_a_rank, C, stream));
+            HCHECK(mi355_hyb_bonus_recurrence(m->o, m->state + L.state_off, m->slot_floats, m->proj, ldp, L.off[P_DQ], L.off[P_DK], L.off[P_DV], m->log_w,
+                                              C, f(MI355_HW_T_BONUS), context_lens, cu_seqlens_q, state_slots, num_seqs, T, c.d_heads, c.d_dim, c.d_vdim,
+                                              m->h_last, m->state + L.row_off, W, nullptr, stream));
+            HCHECK(mi355_hyb_gated_norm_heads(m->mix, dt, L.out_k, mix_col, m->o, f(MI355_HW_D_NORM), c.d_vdim, m->proj + L.off[P_B], ldp,
+                                              MI355_HYB_GATE_SILU, T, c.d_heads, c.d_vdim, eps, L.side_by_side() ? c.d_out_scale : 1.f, stream));
+        }
         if (L.has_delta()) {
             const int C = L.conv_channels();
             float* conv_state = m->state + L.conv_off;
@@ -832,7 +959,20 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             return mi355_hyb_norm_add(m->x, xcopy, m->y, W, f(norm_slot), T, W, eps, stream);
         };
         HCHECK(mi355_hyb_linear(m->y, W, m->mix, dt, L.out_k, WL.w[MI355_HW_OUT_PROJ].p, nullptr, T, W, L.out_k, dt, stream));
-        if (copies) {
+        if (pair) {
+            if (c.mlp_kind == 3) HCHECK(run_experts(c, WL));
+            else if (c.mlp_kind == 4 || c.mlp_kind == 5) {
+                HCHECK(mi355_hyb_linear_act(m->act, dt, c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, c.mlp_ff, W,
+                                            c.mlp_kind == 5 ? MI355_HYB_ACT_GELU : MI355_HYB_ACT_RELU2, c.mlp_ff, dt, stream));
+            } else if (c.mlp_kind) {
+                HCHECK(mi355_hyb_linear(m->gu, 2 * c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, 2 * c.mlp_ff, W, dt, stream));
+                if (c.mlp_kind == 2) HCHECK(mi355_hyb_gelu_glu(m->act, dt, m->gu, T, c.mlp_ff, stream));
+                else HCHECK(mi355_hyb_silu_glu(m->act, dt, m->gu, T, c.mlp_ff, nullptr, 0, stream));
+            }
+            const bool dense = c.mlp_kind && c.mlp_kind != 3;
+            if (dense) HCHECK(mi355_hyb_linear(m->y2, W, m->act, dt, c.mlp_ff, WL.w[MI355_HW_MLP_DOWN].p, nullptr, T, W, c.mlp_ff, dt, stream));
+            HCHECK(pair_step((int)li, m->y, dense ? m->y2 : nullptr, c.mlp_kind == 3, c.moe_top));
+        } else if (copies) {
             HCHECK(stream_step(li, 1, m->y, false, 0));
             if (c.mlp_kind == 3) {
                 // router on the norm's f32 output, the (token, expert) pairs grouped, one grouped product per matrix of the experts with the
@@ -866,20 +1006,8 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
         } else if (parallel) {
             // x <- x + mixer(h) + ff(h): the feed-forward reads the same h (m->pre) the mixer's projections read
             if (c.mlp_kind == 3) {
-                const int E = c.moe_experts, K = c.moe_top, ff = c.mlp_ff, pairs = T * K;
-                HCHECK(mi355_hyb_moe_route_ex(m->moe_ids, m->moe_wts, nullptr, nullptr, dt, bf ? m->hf : static_cast<const float*>(m->pre), nullptr,
-                                              f(MI355_HW_MOE_ROUTER), f(MI355_HW_MOE_CORRECTION), nullptr, T, W, E, K,
-                                              c.moe_scale != 0.f ? c.moe_scale : 1.f, eps, 0, c.moe_sigmoid, c.moe_groups, c.moe_keep_groups,
-                                              c.moe_normalise, stream));
-                const int bm = std::min(mi355_hyb_moe_block_rows(pairs, E, 2 * ff, W, dt), mi355_hyb_moe_block_rows(pairs, E, W, ff, dt));
-                const int nb = (pairs + bm - 1) / bm + E;
-                HCHECK(mi355_hyb_moe_group(m->moe_pos, m->moe_row_token, m->moe_table, m->moe_ids, pairs, K, E, bm, nb, stream));
-                HCHECK(mi355_hyb_linear_grouped(m->moe_gu, 2 * ff, xin, xin_dt, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)2 * ff * W,
-                                                m->moe_table, bm, nb, 2 * ff, W, dt, stream));
-                HCHECK(mi355_hyb_silu_glu(m->moe_act, dt, m->moe_gu, nb * bm, ff, m->moe_table, bm, stream));
-                HCHECK(mi355_hyb_linear_grouped(m->moe_y, W, m->moe_act, dt, ff, nullptr, WL.w[MI355_HW_MOE_DOWN].p, (int64_t)W * ff, m->moe_table, bm,
-                                                nb, W, ff, dt, stream));
-                HCHECK(mi355_hyb_moe_combine_add(m->x, m->y, m->moe_y, m->moe_pos, m->moe_wts, T, W, K, stream));
+                HCHECK(run_experts(c, WL));
+                HCHECK(mi355_hyb_moe_combine_add(m->x, m->y, m->moe_y, m->moe_pos, m->moe_wts, T, W, c.moe_top, stream));
             } else if (c.mlp_kind == 4) {
                 HCHECK(mi355_hyb_linear(m->gu, c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, c.mlp_ff, W, dt, stream));
                 HCHECK(mi355_hyb_relu2(m->act, dt, m->gu, (int64_t)T * c.mlp_ff, stream));
@@ -949,13 +1077,13 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             else if (m->need_xs) HCHECK(mi355_hyb_copy_f32(m->xs + (li + 1) * (size_t)TW, m->x, TW, stream));
         }
         if (layer_trace)
-            HHIP(hipMemcpyAsync(layer_trace + li * (size_t)T * W, m->x, (size_t)T * W * 4, hipMemcpyDeviceToDevice, reinterpret_cast<hipStream_t>(stream)));
+            HHIP(hipMemcpyAsync(layer_trace + li * (size_t)T * W, xcur, (size_t)T * W * 4, hipMemcpyDeviceToDevice, reinterpret_cast<hipStream_t>(stream)));
     }
     if (n_out > 0) {
         if (m->cfg.norm_kind == 1)
-            HCHECK(mi355_hyb_gather_norm_ex(m->xn, dt, m->x, out_rows, static_cast<const float*>(m->final_norm.p), n_out, W, 1, eps, stream));
+            HCHECK(mi355_hyb_gather_norm_ex(m->xn, dt, xcur, out_rows, static_cast<const float*>(m->final_norm.p), n_out, W, 1, eps, stream));
         else
-            HCHECK(mi355_hyb_gather_group_norm(m->xn, dt, m->x, out_rows, static_cast<const float*>(m->final_norm.p), n_out, W,
+            HCHECK(mi355_hyb_gather_group_norm(m->xn, dt, xcur, out_rows, static_cast<const float*>(m->final_norm.p), n_out, W,
                                                m->cfg.norm_groups, eps, stream));
         HCHECK(mi355_hyb_linear(logits, m->cfg.vocab, m->xn, dt, W, m->cfg.tie_head ? m->embed.p : m->head.p, nullptr, n_out, m->cfg.vocab, W, dt,
                                 stream));

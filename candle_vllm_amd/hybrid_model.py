@@ -1,9 +1,8 @@
 """Python harness over the `mi355_hybrid_*` handle (include/mi355_hybrid.h): layer-list models whose layers mix tokens by
 sliding-window attention with a sink, a gated delta rule, a minGRU, attention and delta rule side by side, latent attention,
 attention behind a short convolution with mixed head weights, a state-space mixer, chunked attention or linear attention with a
-constant decay, with dense or mixture-of-experts feed-forwards.  The Sogodra, Vivazen, Kerolorn, Sabolorn and Tosivik designs are read
-here: a design's
-config.json (`architecture`, `layers`, `norm`, `vocab`, `width`, ...) becomes the C structs, its tensors are concatenated into the
+constant decay, or time mixing (beside attention), with dense or mixture-of-experts feed-forwards.  The Sogodra, Vivazen, Kerolorn,
+Sabolorn, Tosivik and Devalorn designs are read here: a design's config.json (`architecture`, `layers`, `norm`, `vocab`, `width`, ...) becomes the C structs, its tensors are concatenated into the
 host layer's slots.  No CPU fallback; torch only holds device buffers."""
 import ctypes
 import json
@@ -18,14 +17,18 @@ from ._lib import lib, HybridConfig, HybridLayer, RopeScaling
 
 DT_F32, DT_BF16 = 0, 2
 MIX_PARALLEL, MIX_MINGRU, MIX_DELTA, MIX_ATTENTION, MIX_LATENT, MIX_CONV_ATTENTION, MIX_SSD, MIX_DECAY = 0, 1, 2, 3, 4, 5, 6, 7
+MIX_TIMEMIX, MIX_PARALLEL_TIMEMIX = 8, 9
 GATE_SILU, GATE_SIGMOID_LR = 0, 1
 ROPE_DEFAULT, ROPE_LLAMA3, ROPE_YARN = 0, 2, 4
 (HW_EMBED, HW_FINAL_NORM, HW_HEAD, HW_NORM1, HW_NORM2, HW_IN_PROJ, HW_IN_BIAS, HW_OUT_PROJ, HW_A_QNORM, HW_A_KNORM, HW_A_SINK, HW_D_CONV,
  HW_D_A_LOG, HW_D_DT_BIAS, HW_D_NORM, HW_D_A2, HW_D_G2, HW_MLP_GATE_UP, HW_MLP_DOWN, HW_A_CONV, HW_A_TALK, HW_L_UKT, HW_L_UV,
  HW_L_CNORM, HW_PRE_NORM1, HW_PRE_NORM2, HW_IN_CONV, HW_A_TEMP, HW_MOE_ROUTER, HW_MOE_CORRECTION, HW_MOE_GATE_UP,
  HW_MOE_DOWN, HW_D_SKIP, HW_CONV_BIAS, HW_A_DIST, HW_L_QNORM, HW_L_UQ, HW_SIDE_GATE, HW_SIDE_PROJ, HW_SIDE_NORM, HW_DEPTH_W,
- HW_SIDE_TABLE, HW_HC1_IN, HW_HC1_OUT, HW_HC1_MIX, HW_HC2_IN, HW_HC2_OUT, HW_HC2_MIX, HW_MOE_BIAS, HW_D_DECAY, HW_BIGRAM) = range(51)
-MLP_CLAMPED_GLU, MLP_GELU_GLU, MLP_MOE, MLP_RELU2, MLP_GELU = 1, 2, 3, 4, 5
+ HW_SIDE_TABLE, HW_HC1_IN, HW_HC1_OUT, HW_HC1_MIX, HW_HC2_IN, HW_HC2_OUT, HW_HC2_MIX, HW_MOE_BIAS, HW_D_DECAY, HW_BIGRAM, HW_T_MU,
+ HW_T_W2, HW_T_W0, HW_T_BONUS) = range(55)
+MLP_CLAMPED_GLU, MLP_GELU_GLU, MLP_MOE, MLP_RELU2, MLP_GELU, MLP_SILU_GLU = 1, 2, 3, 4, 5, 6
+DIST_LOG, DIST_LINEAR = 1, 2
+SEGMENT_ROWS = 128                 # a segment of a time-mixing layer's input projection is whole tiles of this many rows
 MASK_SLIDING, MASK_CHUNKED = 0, 1
 NORM_RMS, NORM_LAYER = 0, 1
 
@@ -579,8 +582,118 @@ class TosivikSpec:
         return L, slots, rope
 
 
+class ZeroRows:
+    """a slot entry: rows of zeros (what fills a segment of a projection up to whole tiles)"""
+
+    def __init__(self, rows, cols):
+        self.rows, self.cols = int(rows), int(cols)
+
+    def bits(self, bits, shapes):
+        return np.zeros(self.rows * self.cols, np.uint16)
+
+
+class DevalornSpec:
+    """config.json of a Devalorn model -> layer structs + the tensor names behind every weight slot.  The design: both sublayers read the
+    same residual through a norm of their own, x <- x + (mixer(N1(x)) + ff(N2(x))).  Mixers: attention with one norm over the whole q
+    and k projections, a query temperature that grows with the position, a linear distance bias and a window, optionally on an earlier
+    layer's keys and values (`attention`, `kv_from`); windowed attention with kept first tokens, rotate-half pairs and a gate per head
+    beside time mixing, the outputs scaled and added (`parallel`).  Feed-forward: silu gate/up, dense or a mixture of experts (softmax
+    router, scaled weights)."""
+    residual_form, resid_alpha, norm_groups = 5, 1.0, 1
+    rope_scaling = staticmethod(yarn_scaling)
+
+    def __init__(self, cfg, shapes):
+        if cfg.get("architecture") != "Devalorn":
+            raise ValueError("not a Devalorn config")
+        self.cfg = cfg
+        self.width, self.vocab = int(cfg["width"]), int(cfg["vocab"])
+        self.eps = float(cfg["norm"]["eps"])
+        self.layers, self.slots, self.rope = [], [], []
+        for i, lc in enumerate(cfg["layers"]):
+            L, slots, rope = self._layer("l%d." % i, lc, shapes)
+            self.layers.append(L)
+            self.slots.append(slots)
+            self.rope.append(rope)
+
+    def _attention(self, L, q, c, shapes, slots):
+        """the fields both kinds of attention share -> (tensors that read the mixer's input, rotation)"""
+        L.a_heads, L.a_kv_heads, L.a_dim, L.a_vdim = int(c["heads"]), int(c["kv_heads"]), int(c["dim"]), int(c["vdim"])
+        L.a_scale = float(c["scale"])
+        mask = c.get("mask") or {}
+        L.a_window, L.a_keep_first = int(mask.get("size") or 0), int(mask.get("keep_first") or 0)
+        qt = c.get("q_temp")
+        if qt:
+            L.a_temp_coef, L.a_temp_every = float(qt["coef"]), float(qt["every"])
+        rope = c.get("rot")
+        L.a_rot_dims = int(rope["dims"]) if rope else 0
+        ins = [q + "q"]
+        if c.get("kv_from") is not None:
+            L.kv_from = int(c["kv_from"]) + 1
+        else:
+            ins += [q + "k", q + "v"]
+        L.a_head_gate = int(q + "g" in shapes)
+        if L.a_head_gate:
+            ins.append(q + "g")
+        return ins, rope if L.a_rot_dims > 0 else None
+
+    def _segment(self, names, shapes):
+        """the rows of `names` and the zeros behind them up to whole tiles"""
+        n = sum(int(shapes[x][0]) for x in names)
+        pad = -n % SEGMENT_ROWS
+        return names + ([ZeroRows(pad, self.width)] if pad else [])
+
+    def _time_mixing(self, L, q, c, shapes, slots):
+        L.d_heads, L.d_dim = int(c["heads"]), int(c["dim"])
+        L.d_vdim, L.d_a_rank = int(shapes[q + "v"][0]) // L.d_heads, int(shapes[q + "w1"][0])
+        slots[HW_T_MU] = [q + "mu." + n for n in "rkvgw"]
+        slots[HW_T_W2], slots[HW_T_W0], slots[HW_T_BONUS] = [HeadTranspose(q + "w2", 1)], [q + "w0"], [q + "u"]
+        slots[HW_D_NORM] = [q + "norm"]
+        return [x for n in ("r", "k", "v", "g", "w1") for x in self._segment([q + n], shapes)]
+
+    def _layer(self, p, lc, shapes):
+        L, slots, rope = HybridLayer(), {HW_NORM1: [p + "norm1"]}, None
+        c, kind, q = lc["mixer"], lc["type"], p + "mix."
+        L.a_out_scale = 1.0
+        if kind == "parallel":
+            L.mixer = MIX_PARALLEL_TIMEMIX
+            ins, rope = self._attention(L, q + "left.", c["left"], shapes, slots)
+            slots[HW_IN_PROJ] = self._segment(ins, shapes) + self._time_mixing(L, q + "right.", c["right"], shapes, slots)
+            L.a_out_scale, L.d_out_scale = float(c["left_scale"]), float(c["right_scale"])
+            slots[HW_OUT_PROJ] = [q + "left.o", q + "right.o"]
+        elif kind == "attention":
+            L.mixer = MIX_ATTENTION
+            slots[HW_IN_PROJ], rope = self._attention(L, q, c, shapes, slots)
+            L.a_qk_norm, L.a_norm_whole = 1, 1
+            slots[HW_A_QNORM] = [q + "q.norm"]
+            if not L.kv_from:
+                slots[HW_A_KNORM] = [q + "k.norm"]
+            L.a_dist_bias = DIST_LINEAR
+            slots[HW_A_DIST] = [Constants([2.0 ** (-8.0 * (h + 1) / L.a_heads) for h in range(L.a_heads)] + [0.0] * L.a_heads)]
+            slots[HW_OUT_PROJ] = [q + "o"]
+        else:
+            raise ValueError(f"layer type {kind!r} is not part of the design")
+        mlp = lc.get("mlp")
+        if mlp:
+            m = p + "mlp."
+            slots[HW_NORM2] = [p + "norm2"]
+            if mlp.get("kind") == "dense":
+                L.mlp_kind, L.mlp_ff = MLP_SILU_GLU, int(mlp["ff"])
+                slots[HW_MLP_GATE_UP], slots[HW_MLP_DOWN] = [m + "gate", m + "up"], [m + "down"]
+            elif mlp.get("kind") == "moe":
+                r = mlp["router"]
+                L.mlp_kind, L.mlp_ff = MLP_MOE, int(mlp["expert"]["ff"])
+                L.moe_experts, L.moe_top, L.moe_scale = int(r["experts"]), int(r["top"]), float(r.get("scale", 1.0))
+                slots[HW_MOE_ROUTER] = [m + "router"]
+                slots[HW_MOE_GATE_UP] = [m + "e%d.%s" % (e, n) for e in range(L.moe_experts) for n in ("gate", "up")]
+                slots[HW_MOE_DOWN] = [m + "e%d.down" % e for e in range(L.moe_experts)]
+            else:
+                raise ValueError(f"feed-forward kind {mlp.get('kind')!r} is not part of the design")
+        return L, slots, rope
+
+
 # config.json `architecture` -> its reader
-SPECS = {"Sogodra": SogodraSpec, "Vivazen": VivazenSpec, "Kerolorn": KerolornSpec, "Sabolorn": SabolornSpec, "Tosivik": TosivikSpec}
+SPECS = {"Sogodra": SogodraSpec, "Vivazen": VivazenSpec, "Kerolorn": KerolornSpec, "Sabolorn": SabolornSpec, "Tosivik": TosivikSpec,
+         "Devalorn": DevalornSpec}
 
 
 class HybridModel:
@@ -656,7 +769,7 @@ class HybridModel:
                     v = np.ascontiguousarray(names[0].values)
                     _check(lib.mi355_hybrid_set_weight_f32(self.h, i, which, v.ctypes.data, v.size), f"set_weight_f32 layer {i} slot {which}")
                 else:
-                    self._put(i, which, np.concatenate([nm.bits(bits, shapes) if isinstance(nm, (HeadTranspose, Ones))
+                    self._put(i, which, np.concatenate([nm.bits(bits, shapes) if isinstance(nm, (HeadTranspose, Ones, ZeroRows))
                                                         else np.asarray(bits[nm], np.uint16).reshape(-1) for nm in names]))
 
     def load_state_dict_f32(self, W):

@@ -3,8 +3,9 @@
  * state), attention and delta rule side by side, latent attention (keys and values read off one cached latent vector per token), or
  * attention behind a short convolution whose heads' softmax weights are mixed -- and which feed-forward (dense gate/up forms or a
  * mixture of experts), a state-space mixer with a scalar decay per head, or linear attention with one constant decay per head; the
- * residual stream is one vector per token or several mixed copies of it.  The Sogodra, Vivazen, Kerolorn, Sabolorn and Tosivik designs
- * are its users.
+ * residual stream is one vector per token or several mixed copies of it; time mixing (projections of a token mixed with the one before,
+ * a matrix state with a decay per key channel, a bonus for the current token).  The Sogodra, Vivazen, Kerolorn, Sabolorn, Tosivik and
+ * Devalorn designs are its users.
  *
  * What differs from the llama-family host layers (mi355_llama_*, mi355_dense_*):
  *   - the residual stream, norms, attention scores, decays, gates of a recurrence and the recurrent state are f32 in both dtypes;
@@ -42,6 +43,13 @@ extern "C" {
 #define MI355_HYB_MIX_DECAY 7       /* linear attention with a constant decay per head: q, k, v = silu of their projections (d_heads heads of
                                       d_dim | d_vdim, no sharing), S <- decay[h] S + k v^T, o = S^T q; RMS norm over all heads together,
                                       times sigmoid(W_g h), output projection.  The decays are MI355_HW_D_DECAY                       */
+
+#define MI355_HYB_MIX_TIMEMIX 8     /* time mixing: with h' the token before (zeros at the start), r, k, v, gate and decay input each read
+                                      h + (h' - h) mu_s (MI355_HW_T_MU); log w = -exp(W_2 tanh(W_1 mix) + w_0) per head and key channel (rank
+                                      d_a_rank); per head o = (S + diag(u) k v^T)^T r, then S <- diag(w) S + k v^T; o over its root mean square,
+                                      times MI355_HW_D_NORM, times silu(gate), output projection.  d_heads heads of d_dim | d_vdim; the slot
+                                      holds S and the last token's h.  Belongs to residual_form 5                                       */
+#define MI355_HYB_MIX_PARALLEL_TIMEMIX 9 /* attention ("left") and time mixing ("right") on the same input, outputs scaled and added     */
 
 #define MI355_HYB_MASK_SLIDING 0    /* a query at position i sees keys j with 0 <= i - j < window                                      */
 #define MI355_HYB_MASK_CHUNKED 1    /* it sees keys j <= i with floor(i / window) = floor(j / window)                                  */
@@ -132,6 +140,10 @@ typedef struct mi355_hybrid_layer {
                                       GATE_UP slots then hold [ff, width] up rows per expert                                 */
     int32_t moe_bias;              /* kind 3: z = router . h + bias (MI355_HW_MOE_BIAS), softmax over the chosen logits only   */
     int32_t moe_shared_plain;      /* kind 3: the shared expert is added as it is (no gate row in the router)                  */
+    /* more forms of the plain attention mixers: a_norm_whole (no rotation then), a_head_gate, a_softcap, kv_from (the lender: an earlier
+     * layer with the same kv heads and head sizes; its keys as cached and its values), a_dist_bias 1 as above or 2: score <- score -
+     * r1[h] (i - j) (MI355_HW_A_DIST as above, r2 unused).  mlp_kind 6: dense gate/up with y = silu(g) u (residual_form 5)       */
+    float a_temp_coef, a_temp_every; /* != 0: the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1)    */
 } mi355_hybrid_layer;
 
 typedef struct mi355_hybrid_config {
@@ -159,6 +171,7 @@ typedef struct mi355_hybrid_config {
      * MI355_HW_NORM1 / 2) reads one mixture of them and writes to all: y = sub(norm(sum_i in[i] X_i)),
      * X_j <- sum_i mix[i, j] X_i + out[j] y (MI355_HW_HC1_* in the mixer, _HC2_* in the feed-forward); the model's output is
      * the sum of the copies                                                                                                  */
+    /* residual_form 5: x <- x + (mixer(norm1(x)) + ff(norm2(x))), both norms (MI355_HW_NORM1 / 2) of the same x                 */
     int32_t streams;
     int32_t bigram_buckets;        /* > 0: the embedding also takes row (previous token mul_prev + token mul_cur) mod buckets of
                                       MI355_HW_BIGRAM (row `buckets` at a sequence's first token); the previous token lives in
@@ -220,14 +233,20 @@ typedef struct mi355_hybrid_config {
 #define MI355_HW_HC2_MIX 47
 #define MI355_HW_MOE_BIAS 48       /* [experts]                                                                      */
 #define MI355_HW_D_DECAY 49        /* [heads] f32, mi355_hybrid_set_weight_f32                                       */
-#define MI355_HW_COUNT 50
 #define MI355_HW_BIGRAM 50         /* global (layer -1): [bigram_buckets + 1, width]                                 */
+#define MI355_HW_T_MU 51           /* [5, width]  time mixing: the mixtures of r, k, v, gate, decay                  */
+#define MI355_HW_T_W2 52           /* [d_a_rank, heads * dim]: the TRANSPOSE of W_2                                   */
+#define MI355_HW_T_W0 53           /* [heads * dim]                                                                  */
+#define MI355_HW_T_BONUS 54        /* [heads * dim]                                                                  */
+#define MI355_HW_COUNT 55
 
 void* mi355_hybrid_create(const mi355_hybrid_config* cfg, const mi355_hybrid_layer* layers);
 void mi355_hybrid_destroy(void* model);
 /* rows of a layer's concatenated input projection, and where each part starts: parts = attention q, k, v, delta q, k, v, beta,
  * decay (a or a1), gate (g or g1) for the attention / delta / parallel mixers; z, x, g for the minGRU; q (heads x (dim + rot_dim)),
- * the latent down-projection (kv_rank + rot_dim) in the k part and the head gate in the gate part for latent attention.
+ * the latent down-projection (kv_rank + rot_dim) in the k part and the head gate in the gate part for latent attention.  Time mixing: r, k, v
+ * in the delta q, k, v parts, its gate in the beta part, W_1 in the decay part; the attention's rows together and every one of these
+ * parts are followed by rows of zeros up to a multiple of 128 (the attention's head gate, where there is one, is in the gate part).
  * offsets[9], -1 = absent */
 int32_t mi355_hybrid_in_proj_rows(const mi355_hybrid_layer* layer, int32_t* offsets);
 /* HOST bf16 bits (a checkpoint tensor), n elements; converted to the storage type of the slot */
@@ -531,6 +550,58 @@ int mi355_hyb_decay_attention(float* o, float* state, int64_t state_stride, cons
                               float* scratch, int64_t stream);
 /* floats of `scratch` that suit a step of this size; 0: the scan suits it (few tokens per sequence, or sizes that only the scan serves) */
 int64_t mi355_hyb_decay_attention_scratch(int32_t num_tokens, int32_t num_seqs, int32_t heads, int32_t dim, int32_t vdim);
+/* ---- mechanisms of the designs with a norm per sublayer of the same residual, and time mixing */
+/* a product whose column segments read different left operands: segment i (seg_rows[i] rows of w, multiples of 128, together n; HOST array, at
+ * most 8) reads a + (first + i) a_stride elements; else as mi355_hyb_linear */
+int mi355_hyb_linear_segments(float* out, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, int64_t a_stride, int32_t first, const void* w,
+                              const float* bias, const int32_t* seg_rows, int32_t n_seg, int32_t num_tokens, int32_t n, int32_t k, int32_t dtype,
+                              int64_t stream);
+/* the end of one layer and the start of the next in one launch:
+ *   x' = x + (y1 + (y2 or sum_j moe_w[t, j] moe_rows[moe_pos[t top + j]]))     (each part NULL = none) -> x_out (NULL: not written)
+ *   h = RMSnorm(x') norm1 -> out1 (dt_out) [T, width];   RMSnorm(x') norm2 -> out2 (dt_out) (and out2_f32, NULL or f32)   (norm2 NULL: neither)
+ *   mixture m < mixes: h + (h' - h) mu[m] -> out1 + (m + 1) seg_stride elements, h' = the h of the token before: of the same portion, or
+ *   for its first token h_state (f32 rows per slot, stride in floats; zeros at position 0); h_last f32 [num_seqs, width] <- the h of every
+ *   portion's last token (the caller moves it into h_state once nothing reads the old one: mi355_hyb_bonus_recurrence does)
+ * norm1 NULL: only the sum.  x_out may be x only without mixtures.  width <= 16384 */
+int mi355_hyb_pair_step(const float* x, const float* y1, const float* y2, const float* moe_rows, const int32_t* moe_pos, const float* moe_w,
+                        int32_t top, float* x_out, const float* norm1, const float* norm2, void* out1, int64_t seg_stride, void* out2,
+                        int32_t out_dtype, float* out2_f32, const float* mu, int32_t mixes, const float* h_state, int64_t state_stride,
+                        float* h_last, const uint32_t* context_lens, const uint32_t* cu_seqlens_q, const int32_t* state_slots,
+                        const int32_t* token_seq, int32_t num_tokens, int32_t width, float eps, int64_t stream);
+/* log_w f32 [T, ldw] = -exp(sum_r w2t[r, c] tanh(z[t, r]) + w0[c]), w2t f32 [rank, channels] */
+int mi355_hyb_lowrank_decay(float* log_w, int32_t ldw, const float* z, int32_t ldz, const float* w2t, const float* w0, int32_t num_tokens,
+                            int32_t rank, int32_t channels, int64_t stream);
+/* recurrence with a decay per key channel and a bonus for the current token over the new tokens of every sequence, state f32 [slots] x
+ * [heads, dim, vdim] (stride in floats): o f32 [T, heads, vdim] = (S + diag(bonus) k v^T)^T r, then S <- diag(exp(log_w)) S + k v^T.
+ * rkv f32 [T, ldq] holds r, k (heads x dim) and v (heads x vdim) at their offsets; log_w f32 [T, ldw] (heads x dim), bonus f32 [heads, dim].
+ * row != NULL: row f32 [num_seqs, row_n] moves into row_state (f32 per slot, the same stride).  dim <= 512 */
+int mi355_hyb_bonus_recurrence(float* o, float* state, int64_t state_stride, const float* rkv, int32_t ldq, int32_t r_off, int32_t k_off,
+                               int32_t v_off, const float* log_w, int32_t ldw, const float* bonus, const uint32_t* context_lens,
+                               const uint32_t* cu_seqlens_q, const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads,
+                               int32_t dim, int32_t vdim, const float* row, float* row_state, int32_t row_n, float* scratch, int64_t stream);
+/* mi355_hyb_gated_norm with weights per head: head h's start at w + h w_ld (w_ld 0: the same for all heads) */
+int mi355_hyb_gated_norm_heads(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const float* o, const float* w, int32_t w_ld,
+                               const float* gate_in, int32_t ldg, int32_t gate, int32_t num_tokens, int32_t heads, int32_t vdim, float eps,
+                               float out_scale, int64_t stream);
+/* mi355_hyb_attn_prepare_ex / _whole with a query temperature (temp_coef 0 = none): the query at position p times 1 + temp_coef
+ * ln(floor((p + 1) / temp_every) + 1); k_pages and v_pages NULL: the queries only (a layer that reads another layer's pages) */
+int mi355_hyb_attn_prepare_temp(void* q_out, void* k_pages, void* v_pages, const float* proj, int32_t ldp, int32_t q_off, int32_t k_off,
+                                int32_t v_off, const float* q_norm_w, const float* k_norm_w, const float* cos_t, const float* sin_t,
+                                const int64_t* positions, const int64_t* slot_mapping, int32_t num_tokens, int32_t heads, int32_t kv_heads,
+                                int32_t dim, int32_t vdim, int32_t rot_dims, int32_t interleaved, int32_t norm_mode, const float* q_head_scale,
+                                float temp_coef, float temp_every, float eps, int32_t dtype, int64_t stream);
+int mi355_hyb_attn_prepare_whole_temp(void* q_out, void* k_pages, void* v_pages, const float* src, int32_t ld, int32_t q_off, int32_t k_off,
+                                      int32_t v_off, const float* q_norm_w, const float* k_norm_w, const int64_t* positions,
+                                      const int64_t* slot_mapping, int32_t num_tokens, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim,
+                                      int32_t v_unit, float temp_coef, float temp_every, float eps, int32_t dtype, int64_t stream);
+/* mi355_hyb_attention with a linear distance bias (dist_linear: score - r1[h] (i - j)) and an output gate: head h's output of token t times
+ * sigmoid(gate[t ldg + h]) (gate NULL = none) */
+int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const void* q, const void* k_pages, const void* v_pages,
+                           const uint32_t* block_tables, const uint32_t* context_lens, const uint32_t* cu_seqlens_q, const int32_t* token_seq,
+                           const float* sink, const float* dist, int32_t dist_linear, const float* gate, int32_t ldg, int32_t num_seqs,
+                           int32_t num_tokens, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int32_t max_blocks,
+                           int32_t mask_kind, int32_t window, int32_t keep_first, float scale, float out_scale, int32_t k_ld, int32_t v_ld,
+                           float softcap, int32_t cross_values, int32_t dtype, int64_t stream);
 /* 0: prompt-sized steps over bf16 pages take the generic kernel instead of the matrix-core ones; 2: the matrix-core kernel with one
  * wave per head also where the query heads of a key/value head could share a workgroup (A/B switch, process-wide; default 1) */
 void mi355_hyb_set_attention_mfma(int32_t on);
