@@ -1,6 +1,6 @@
 """`python bench.py --hybrid`: prompt and decode throughput of the layer-list host layer (Sogodra design, or Vivazen / Kerolorn /
-Sabolorn / Tosivik with `--hybrid-design vivazen|kerolorn|sabolorn|tosivik`; random weights) at layer sizes of a real model, beside the framework's closest existing model -- the 16-bit llama host layer (dense_model.cpp) -- at equal
-width, depth, head geometry, feed-forward size and vocabulary.  One GPU, bf16, synthetic data.  The default workload of bench.py and
+Sabolorn / Tosivik / Devalorn with `--hybrid-design vivazen|kerolorn|sabolorn|tosivik|devalorn`; random weights) at layer sizes of a real
+model, beside the framework's closest existing model -- the 16-bit llama host layer (dense_model.cpp) -- at equal width, depth, head geometry, feed-forward size and vocabulary.  One GPU, bf16, synthetic data.  The default workload of bench.py and
 its one-line contract are not touched: this option prints its own JSON line.
 
 Per size: one prompt step of T tokens (tokens/s) and decode steps of B sequences behind `ctx` cached tokens (tokens/s), both models
@@ -60,6 +60,65 @@ TOSIVIK = {
     "3b": dict(l_heads=24, l_dim=128, l_vdim=128, streams=4, experts=16, top=3, buckets=40009, layers="lala"),
     "8b": dict(l_heads=32, l_dim=128, l_vdim=128, streams=4, experts=16, top=3, buckets=40009, layers="lala"),
 }
+
+
+# Devalorn at the same widths: attention with the llama geometry (window, kept first tokens, a gate per head; at 3b its values are twice as
+# wide) beside time mixing (width / 64 heads of 64) with a dense silu feed-forward of the llama size, and attention with a distance bias
+# and a query temperature with a mixture of experts whose ACTIVE size equals it (`top` experts of ff / 4), in turn; the fourth layer
+# reads the second one's keys and values
+DEVALORN = {
+    "1b": dict(vdim=128, rank=64, rdim=64, experts=16, top=4, keep=64, layers="paps"),
+    "3b": dict(vdim=256, rank=64, rdim=64, experts=16, top=4, keep=64, layers="paps"),
+    "8b": dict(vdim=128, rank=64, rdim=64, experts=16, top=4, keep=64, layers="paps"),
+}
+
+
+def devalorn_config(s, v):
+    left = {"dim": s["dim"], "heads": s["heads"], "kv_heads": s["kv"], "mask": {"keep_first": v["keep"], "size": s["window"]}, "scale": s["dim"] ** -0.5,
+            "rot": {"base": 500000.0, "dims": s["dim"]}, "vdim": v["vdim"]}
+    par = {"left": left, "left_scale": 1.1, "right": {"dim": v["rdim"], "heads": s["width"] // v["rdim"]}, "right_scale": 0.8}
+    att = {"dim": s["dim"], "heads": s["heads"], "kv_heads": s["kv"], "mask": {"size": s["window"] + 64}, "q_temp": {"coef": 0.1, "every": 1024},
+           "scale": s["dim"] ** -0.5, "vdim": s["dim"]}
+    dense = {"ff": s["ff"], "kind": "dense"}
+    moe = {"expert": {"ff": s["ff"] // 4}, "kind": "moe", "router": {"experts": v["experts"], "scale": 1.5, "top": v["top"]}}
+    kinds = {"p": {"type": "parallel", "mixer": par, "mlp": dense}, "a": {"type": "attention", "mixer": att, "mlp": moe},
+             "s": {"type": "attention", "mixer": dict(att, kv_from=v["layers"].index("a")), "mlp": moe}}
+    return {"architecture": "Devalorn", "layers": [kinds[c] for c in v["layers"]], "norm": {"eps": 1e-5}, "vocab": s["vocab"], "width": s["width"]}
+
+
+def devalorn_shapes(cfg, rank=64):
+    W, sh = cfg["width"], {}
+    sh["embed"], sh["final.norm"], sh["head"] = (cfg["vocab"], W), (W,), (cfg["vocab"], W)
+
+    def attention(q, c):
+        sh[q + "q"], sh[q + "o"] = (c["heads"] * c["dim"], W), (W, c["heads"] * c["vdim"])
+        if "kv_from" not in c:
+            sh[q + "k"], sh[q + "v"] = (c["kv_heads"] * c["dim"], W), (c["kv_heads"] * c["vdim"], W)
+    for i, lc in enumerate(cfg["layers"]):
+        p, c, mlp = "l%d." % i, lc["mixer"], lc["mlp"]
+        m = p + "mlp."
+        sh[p + "norm1"], sh[p + "norm2"] = (W,), (W,)
+        if lc["type"] == "parallel":
+            attention(p + "mix.left.", c["left"])
+            sh[p + "mix.left.g"] = (c["left"]["heads"], W)
+            q, H, d = p + "mix.right.", c["right"]["heads"], c["right"]["dim"]
+            for n in "rkvgw":
+                sh[q + "mu." + n] = (W,)
+            for n in "rkvg":
+                sh[q + n] = (H * d, W)
+            sh[q + "w1"], sh[q + "w2"], sh[q + "w0"], sh[q + "u"] = (rank, W), (H * d, rank), (H * d,), (H, d)
+            sh[q + "norm"], sh[q + "o"] = (H * d,), (W, H * d)
+        else:
+            attention(p + "mix.", c)
+            sh[p + "mix.q.norm"] = (c["heads"] * c["dim"],)
+            if "kv_from" not in c:
+                sh[p + "mix.k.norm"] = (c["kv_heads"] * c["dim"],)
+        for e in ([""] if mlp["kind"] == "dense" else ["e%d." % e for e in range(mlp["router"]["experts"])]):
+            ff = mlp["ff"] if mlp["kind"] == "dense" else mlp["expert"]["ff"]
+            sh[m + e + "gate"], sh[m + e + "up"], sh[m + e + "down"] = (ff, W), (ff, W), (W, ff)
+        if mlp["kind"] == "moe":
+            sh[m + "router"] = (mlp["router"]["experts"], W)
+    return sh
 
 
 def tosivik_config(s, v):
@@ -282,7 +341,7 @@ def build_hybrid(cfg, max_tokens, slots):
     import torch
     from candle_vllm_amd import hybrid_model as hm
     shapes = {"Vivazen": vivazen_shapes, "Kerolorn": kerolorn_shapes, "Sogodra": sogodra_shapes, "Sabolorn": sabolorn_shapes,
-              "Tosivik": tosivik_shapes}[cfg["architecture"]](cfg)
+              "Tosivik": tosivik_shapes, "Devalorn": devalorn_shapes}[cfg["architecture"]](cfg)
     spec = hm.SPECS[cfg["architecture"]](cfg, shapes)
     m = hm.HybridModel(spec, dtype="bfloat16", block_size=64, state_slots=slots)
     g = torch.Generator(device="cuda").manual_seed(7)
@@ -300,6 +359,10 @@ def build_hybrid(cfg, max_tokens, slots):
             return ((0.25 if cfg["architecture"] == "Sabolorn" else 1.0) * torch.randn(shape, generator=g, device="cuda")).to(torch.bfloat16)
         if name.endswith(".r1") or name.endswith(".r2"):                  # the distance bias: positive rates
             return (0.1 + torch.rand(shape, generator=g, device="cuda")).to(torch.bfloat16)
+        if ".mu." in name:                                                # how much of the token before a mixture takes
+            return torch.rand(shape, generator=g, device="cuda").to(torch.bfloat16)
+        if name.endswith(".w0"):                                          # decays between about 0.7 and 0.998 per token
+            return (-6 + 5 * torch.rand(shape, generator=g, device="cuda")).to(torch.bfloat16)
         if name.endswith(".dwa"):
             return torch.full(shape, 1.0 / shape[0], device="cuda").to(torch.bfloat16)
         if ".hc" in name:                                                 # mixing of the residual streams: near the identity, every stream takes part
@@ -318,7 +381,8 @@ def build_hybrid(cfg, max_tokens, slots):
             hm._check(hm.lib.mi355_hybrid_set_weight_f32(m.h, layer, which, v.ctypes.data, v.size), "set_weight_f32")
             return
         names = [n.name if isinstance(n, hm.HeadTranspose) else n for n in names]       # random values: the transposed layout is as random
-        ts = [rnd(shapes[n], n) if n else None for n in names]
+        ts = [None if not n else torch.zeros((n.rows, n.cols), dtype=torch.bfloat16, device="cuda") if isinstance(n, hm.ZeroRows) else rnd(shapes[n], n)
+              for n in names]
         if which == hm.HW_IN_BIAS:
             rows = [shapes[p][0] for p in spec.slots[layer][hm.HW_IN_PROJ]]
             ts = [t if t is not None else torch.zeros(r, dtype=torch.bfloat16, device="cuda") for t, r in zip(ts, rows)]
@@ -353,9 +417,10 @@ def run_size(name, T=2048, B=8, ctx=2048, dec_steps=16, design="sogodra"):
     from candle_vllm_amd.step_engine import StepEngine
     from oracle.dense_llama import DenseConfig
     s = SIZES[name]
-    extra = {"vivazen": VIVAZEN, "kerolorn": KEROLORN, "sabolorn": SABOLORN, "tosivik": TOSIVIK}.get(design, {}).get(name, {})
+    extra = {"vivazen": VIVAZEN, "kerolorn": KEROLORN, "sabolorn": SABOLORN, "tosivik": TOSIVIK, "devalorn": DEVALORN}.get(design, {}).get(name, {})
     cfg = (vivazen_config(s, extra) if design == "vivazen" else kerolorn_config(s, extra) if design == "kerolorn" else
-           sabolorn_config(s, extra) if design == "sabolorn" else tosivik_config(s, extra) if design == "tosivik" else sogodra_config(s))
+           sabolorn_config(s, extra) if design == "sabolorn" else tosivik_config(s, extra) if design == "tosivik" else devalorn_config(s, extra) if design == "devalorn" else
+           sogodra_config(s))
     rng = np.random.default_rng(5)
     out = {"size": name, "design": design, "shape": dict(s, **extra), "prompt_tokens": T, "decode_batch": B,
            "decode_ctx": ctx}
@@ -426,8 +491,8 @@ def run_size(name, T=2048, B=8, ctx=2048, dec_steps=16, design="sogodra"):
 
 
 def main(sizes="1b,3b", prompt_tokens=2048, batch=8, ctx=2048, design="sogodra"):
-    if design not in ("sogodra", "vivazen", "kerolorn", "sabolorn", "tosivik"):
-        raise SystemExit("--hybrid-design: sogodra, vivazen, kerolorn, sabolorn or tosivik")
+    if design not in ("sogodra", "vivazen", "kerolorn", "sabolorn", "tosivik", "devalorn"):
+        raise SystemExit("--hybrid-design: sogodra, vivazen, kerolorn, sabolorn, tosivik or devalorn")
     res = [run_size(n.strip(), T=prompt_tokens, B=batch, ctx=ctx, design=design) for n in sizes.split(",") if n.strip()]
     print(json.dumps({"metric": "hybrid_vs_llama_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
                       "note": "%s layer-list host layer beside the 16-bit llama host layer at equal sizes; the hybrid side's decode steps replay "

@@ -461,6 +461,7 @@ _sig("mi355_hyb_pair_step", ctypes.c_int, [c_vp] * 6 + [c_i32] + [c_vp] * 4 + [c
 _sig("mi355_hyb_lowrank_decay", ctypes.c_int, [c_vp, c_i32, c_vp, c_i32, c_vp, c_vp, c_i32, c_i32, c_i32, c_i64])
 _sig("mi355_hyb_bonus_recurrence", ctypes.c_int, [c_vp, c_vp, c_i64, c_vp, c_i32, c_i32, c_i32, c_i32, c_vp, c_i32] + [c_vp] * 4 + [c_i32] * 5 +
      [c_vp, c_vp, c_i32, c_vp, c_i64])
+_sig("mi355_hyb_bonus_recurrence_scratch", c_i64, [c_i32] * 5)
 _sig("mi355_hyb_gated_norm_heads", ctypes.c_int, [c_vp, c_i32, c_i32, c_i32, c_vp, c_vp, c_i32, c_vp, c_i32, c_i32, c_i32, c_i32, c_i32, c_f32, c_f32, c_i64])
 _sig("mi355_hyb_attn_prepare_temp", ctypes.c_int, [c_vp] * 4 + [c_i32] * 4 + [c_vp] * 6 + [c_i32] * 8 + [c_vp, c_f32, c_f32, c_f32, c_i32, c_i64])
 _sig("mi355_hyb_attn_prepare_whole_temp", ctypes.c_int, [c_vp] * 4 + [c_i32] * 4 + [c_vp] * 4 + [c_i32] * 6 + [c_f32, c_f32, c_f32, c_i32, c_i64])

@@ -103,7 +103,7 @@ struct HModel {
     float *y2 = nullptr, *hf = nullptr, *xs = nullptr, *side_g = nullptr;
     void *side_a = nullptr, *cq = nullptr;
     Weight side_table;
-    // form 4: the copies of the residual stream; embedding by pairs of tokens; scratch of the constant-decay attention by pieces
+    // form 4: the copies of the residual stream; embedding by pairs of tokens; scratch of the recurrences by pieces
     float *streams = nullptr, *pieces = nullptr;
     int64_t cap_pieces = 0;
     int32_t* bigram_rows = nullptr;
@@ -366,7 +366,8 @@ template <typename T> int grow(T*& p, size_t bytes) {
 int ensure_capacity(HModel* m, int T, int n_out, int n_seqs) {
     int64_t pieces = 0;
     for (const HLayer& L : m->layers)
-        if (L.is_decay()) pieces = std::max(pieces, mi355_hyb_decay_attention_scratch(T, n_seqs, L.c.d_heads, L.c.d_dim, L.c.d_vdim));
+        if (L.has_timemix()) pieces = std::max(pieces, mi355_hyb_bonus_recurrence_scratch(T, n_seqs, L.c.d_heads, L.c.d_dim, L.c.d_vdim));
+        else if (L.is_decay()) pieces = std::max(pieces, mi355_hyb_decay_attention_scratch(T, n_seqs, L.c.d_heads, L.c.d_dim, L.c.d_vdim));
     if (pieces > m->cap_pieces) {
         HHIP(hipDeviceSynchronize());
         drop_graphs(m);
@@ -916,10 +917,11 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             // the decays of the low-rank map, the recurrence over the state slot (which also takes the portions' last h), the norm per head
             // with the gate
             const int C = c.d_heads * c.d_dim;
+            const bool by_pieces = mi355_hyb_bonus_recurrence_scratch(T, num_seqs, c.d_heads, c.d_dim, c.d_vdim) > 0;
             HCHECK(mi355_hyb_lowrank_decay(m->log_w, C, m->proj + L.off[P_A], ldp, f(MI355_HW_T_W2), f(MI355_HW_T_W0), T, c.d_a_rank, C, stream));
             HCHECK(mi355_hyb_bonus_recurrence(m->o, m->state + L.state_off, m->slot_floats, m->proj, ldp, L.off[P_DQ], L.off[P_DK], L.off[P_DV], m->log_w,
                                               C, f(MI355_HW_T_BONUS), context_lens, cu_seqlens_q, state_slots, num_seqs, T, c.d_heads, c.d_dim, c.d_vdim,
-                                              m->h_last, m->state + L.row_off, W, nullptr, stream));
+                                              m->h_last, m->state + L.row_off, W, by_pieces ? m->pieces : nullptr, stream));
             HCHECK(mi355_hyb_gated_norm_heads(m->mix, dt, L.out_k, mix_col, m->o, f(MI355_HW_D_NORM), c.d_vdim, m->proj + L.off[P_B], ldp,
                                               MI355_HYB_GATE_SILU, T, c.d_heads, c.d_vdim, eps, L.side_by_side() ? c.d_out_scale : 1.f, stream));
         }

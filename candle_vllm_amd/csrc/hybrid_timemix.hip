@@ -266,6 +266,291 @@ template <int DP, int LPC, int CH> __global__ __launch_bounds__(256) void bonus_
         for (int r = 0; r < DP; ++r) { const int i = part * DP + r; if (i < d) stt[(size_t)i * vd + col] = S[r]; }
 }
 
+// ------------------------------------------------------------------------------------------------------------ the same by pieces
+// Portions of prompts: the new tokens of a sequence are cut into pieces of LC tokens that are worked on side by side, a piece into
+// sub-pieces of SB.  With w_t the decays per channel, E_m = the product of sub-piece m's decays, S_in the state in front of the piece:
+//   prepare:  r'_t = r_t prod_(a < t) w_a,  k'_t = k_t prod_(a > t) w_a  (a in t's own sub-piece), E_m, and the scores inside a sub-piece,
+//             D[t, s] = sum_i r_ti k_si prod_(s < a < t) w_ai for s < t,  D[t, t] = sum_i r_ti u_i k_ti  -- walked token by token: products of
+//             decays only, no quotient of two small numbers anywhere
+//   state:    U = sum_s diag(prod_(m > m(s)) E_m) k'_s v_s^T              what the piece adds to the state;  the product of all its E_m
+//   scan:     S_in of the next piece = diag(prod E) S_in + U               the only sequential part, elementwise over the state
+//   output:   o_t = sum_(s <= t, same sub-piece) D[t, s] v_s + sum_(s in sub-piece m < m(t)) (r'_t prod_(m < b < m(t)) E_b . k'_s) v_s
+//                   + (r'_t prod_(b < m(t)) E_b) S_in
+// All products run on the f32 matrix cores (16 x 16 tiles, 4 deep): the result is the recurrence's up to f32 rounding.
+constexpr int LC = 64, SB = 16, NSB = LC / SB;
+struct BonusPieces {
+    BonusArgs a;
+    float *rd, *kd, *E, *ptot, *D, *U;      // [T, H d] twice, [pieces NSB, H d], [pieces, H d], [T, H, SB], [pieces, H, d, vd]
+};
+__device__ __forceinline__ f32x4_t mfma_f32(float a, float b, const f32x4_t& c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+// piece b of the step -> its first token and its tokens (0: past the last piece)
+__device__ __forceinline__ int piece_of(const BonusArgs& p, int b, int& t0) {
+    for (int s = 0; s < p.n_seqs; ++s) {
+        const int tb = (int)p.cu_q[s], n = (int)p.cu_q[s + 1] - tb, pieces = (n + LC - 1) / LC;
+        if (b < pieces) { t0 = tb + b * LC; return min(LC, n - b * LC); }
+        b -= pieces;
+    }
+    return 0;
+}
+
+// a wave per sub-piece, 64 channels at a time: a lane first owns a channel (the running products of its decays), then a quarter of the
+// channels of one key (the scores inside the sub-piece)
+__global__ __launch_bounds__(256) void bonus_prepare_kernel(BonusPieces q) {
+    const BonusArgs& p = q.a;
+    constexpr int RS = 68;                                   // floats per staged row: 64 channels + 4 of padding
+    __shared__ __align__(16) float sr[NSB][SB * RS], sk[NSB][SB * RS], sw[NSB][SB * RS];
+    int t0;
+    const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y, d = p.d, C = p.H * d;
+    if (n == 0) return;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, key = lane & 15, kg = lane >> 4, first = wave * SB, cnt = min(SB, n - first);
+    float* R = sr[wave];
+    float* K = sk[wave];
+    float* Wd = sw[wave];
+    float acc[SB];
+#pragma unroll
+    for (int t = 0; t < SB; ++t) acc[t] = 0.f;
+    for (int c0 = 0; c0 < d; c0 += 64) {
+        const int ch = c0 + lane;
+        const bool on = ch < d;
+        float r[SB], k[SB], w[SB];
+#pragma unroll
+        for (int t = 0; t < SB; ++t) {
+            const bool ok_ = on && t < cnt;
+            const size_t row = (size_t)(t0 + first + (ok_ ? t : 0));
+            r[t] = ok_ ? p.rkv[row * p.ldq + p.r_off + h * d + ch] : 0.f;
+            k[t] = ok_ ? p.rkv[row * p.ldq + p.k_off + h * d + ch] : 0.f;
+            w[t] = ok_ ? expf(p.lw[row * p.ldw + h * d + ch]) : 1.f;
+        }
+        __syncthreads();                                     // (the chunk of channels before is used up)
+        float f = 1.f;
+#pragma unroll
+        for (int t = 0; t < SB; ++t) {
+            R[t * RS + lane] = r[t]; K[t * RS + lane] = k[t]; Wd[t * RS + lane] = w[t];
+            if (on && t < cnt) q.rd[(size_t)(t0 + first + t) * C + h * d + ch] = r[t] * f;
+            f *= w[t];
+        }
+        if (on) q.E[((size_t)blockIdx.x * NSB + wave) * C + h * d + ch] = f;
+        f = 1.f;
+#pragma unroll
+        for (int t = SB - 1; t >= 0; --t) {
+            if (on && t < cnt) q.kd[(size_t)(t0 + first + t) * C + h * d + ch] = k[t] * f;
+            f *= w[t];
+        }
+        __syncthreads();
+        float x[16];
+        const int cc = kg * 16;
+        float own = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; i += 4) {
+            const float4 kv = *reinterpret_cast<const float4*>(&K[key * RS + cc + i]), rv = *reinterpret_cast<const float4*>(&R[key * RS + cc + i]);
+            x[i] = kv.x; x[i + 1] = kv.y; x[i + 2] = kv.z; x[i + 3] = kv.w;
+            const float* u = p.u + h * d + c0 + cc + i;
+            if (c0 + cc + i < d) own = fmaf(rv.x * u[0], kv.x, fmaf(rv.y * u[1], kv.y, fmaf(rv.z * u[2], kv.z, fmaf(rv.w * u[3], kv.w, own))));
+        }
+#pragma unroll
+        for (int t = 0; t < SB; ++t) {
+            const bool past = key < t;
+            float dot = 0.f;
+#pragma unroll
+            for (int i = 0; i < 16; i += 4) {
+                const float4 rv = *reinterpret_cast<const float4*>(&R[t * RS + cc + i]), wv = *reinterpret_cast<const float4*>(&Wd[t * RS + cc + i]);
+                dot = fmaf(rv.x, x[i], fmaf(rv.y, x[i + 1], fmaf(rv.z, x[i + 2], fmaf(rv.w, x[i + 3], dot))));
+                x[i] *= past ? wv.x : 1.f; x[i + 1] *= past ? wv.y : 1.f; x[i + 2] *= past ? wv.z : 1.f; x[i + 3] *= past ? wv.w : 1.f;
+            }
+            acc[t] += past ? dot : (key == t ? own : 0.f);
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < SB; ++t) {
+        float v = acc[t];
+        v += __shfl_xor(v, 16);
+        v += __shfl_xor(v, 32);
+        if (kg == (t & 3) && t < cnt) q.D[((size_t)(t0 + first + t) * p.H + h) * SB + key] = v;
+    }
+}
+
+// a wave takes 16 columns of U and walks its rows 16 RT at a time: RT tiles of K'^T against one of V
+template <int RT> __global__ __launch_bounds__(256) void bonus_state_kernel(BonusPieces q) {
+    const BonusArgs& p = q.a;
+    int t0;
+    const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y, d = p.d, C = p.H * d;
+    if (n == 0) return;
+    const float* E = q.E + (size_t)blockIdx.x * NSB * C + h * d;
+    if (blockIdx.z == 0)
+        for (int i = threadIdx.x; i < d; i += blockDim.x) {
+            float f = 1.f;
+#pragma unroll
+            for (int b = 0; b < NSB; ++b) if (b * SB < n) f *= E[(size_t)b * C + i];
+            q.ptot[(size_t)blockIdx.x * C + h * d + i] = f;
+        }
+    const int lane = threadIdx.x & 63, m16 = lane & 15, kg = lane >> 4, col = (blockIdx.z * 4 + (threadIdx.x >> 6)) * 16 + m16;
+    if (col - m16 >= p.vd) return;
+    const float* K = q.kd + (size_t)t0 * C + h * d + m16;
+    const float* V = p.rkv + (size_t)t0 * p.ldq + p.v_off + h * p.vd + col;
+    float* U = q.U + ((size_t)blockIdx.x * p.H + h) * d * p.vd;
+    const int last = (n - 1) / SB;
+    for (int r0 = 0; r0 < d; r0 += 16 * RT) {
+        f32x4_t acc[RT];
+        float f[RT];
+#pragma unroll
+        for (int i = 0; i < RT; ++i) { acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f}; f[i] = 1.f; }
+        for (int b = last; b >= 0; --b) {                    // from the piece's end: the factor of a sub-piece is the product of those behind it
+#pragma unroll
+            for (int tt = 0; tt < SB; tt += 4) {
+                const int t = b * SB + tt + kg;
+                const bool on = t < n;
+                const float v = on ? V[(size_t)t * p.ldq] : 0.f;
+                float a[RT];
+#pragma unroll
+                for (int i = 0; i < RT; ++i) a[i] = (on && r0 + 16 * i < d) ? K[(size_t)t * C + r0 + 16 * i] * f[i] : 0.f;
+#pragma unroll
+                for (int i = 0; i < RT; ++i) acc[i] = mfma_f32(a[i], v, acc[i]);
+            }
+            if (b > 0)
+#pragma unroll
+                for (int i = 0; i < RT; ++i) if (r0 + 16 * i < d) f[i] *= E[(size_t)b * C + r0 + 16 * i + m16];
+        }
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+            if (r0 + 16 * i < d)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) U[(size_t)(r0 + 16 * i + 4 * kg + v) * p.vd + col] = acc[i][v];
+    }
+}
+
+// a thread per element of a (sequence, head)'s state: the states in front of its pieces, then the one behind the last
+__global__ __launch_bounds__(256) void bonus_piece_scan_kernel(BonusPieces q) {
+    const BonusArgs& p = q.a;
+    const int s = blockIdx.x, h = blockIdx.y, e = blockIdx.z * 256 + threadIdx.x, per = p.d * p.vd;
+    const int n = (int)p.cu_q[s + 1] - (int)p.cu_q[s];
+    if (n <= 0) return;
+    if (p.row && h == 0)
+        for (int i = e; i < p.row_n; i += gridDim.z * 256) (p.row_state + (size_t)p.slots[s] * p.state_stride)[i] = p.row[(size_t)s * p.row_n + i];
+    if (e >= per) return;
+    int first = 0;
+    for (int i = 0; i < s; ++i) first += ((int)p.cu_q[i + 1] - (int)p.cu_q[i] + LC - 1) / LC;
+    const int pieces = (n + LC - 1) / LC;
+    float* stt = p.state + (size_t)p.slots[s] * p.state_stride + (size_t)h * per + e;
+    float S = (int)p.ctx[s] > n ? *stt : 0.f;
+    const size_t step = (size_t)p.H * per, fstep = (size_t)p.H * p.d;
+    float* u = q.U + (size_t)first * step + (size_t)h * per + e;
+    const float* f = q.ptot + (size_t)first * fstep + h * p.d + e / p.vd;
+    constexpr int AHEAD = 8;                      // pieces whose contributions are requested together
+    for (int c0 = 0; c0 < pieces; c0 += AHEAD) {
+        float add[AHEAD], mul[AHEAD];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) { add[i] = c0 + i < pieces ? u[(size_t)(c0 + i) * step] : 0.f; mul[i] = c0 + i < pieces ? f[(size_t)(c0 + i) * fstep] : 0.f; }
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i)
+            if (c0 + i < pieces) { u[(size_t)(c0 + i) * step] = S; S = fmaf(mul[i], S, add[i]); }
+    }
+    *stt = S;
+}
+
+// a wave takes the 16 queries of one sub-piece and 16 VT columns of the output: its scores against the sub-pieces before it and the ones
+// inside it through LDS into the layout of a left operand, then the two products into one accumulator.  (The depth of a product is walked
+// in the order 16 j + 4 kg + e, e innermost, on both operands: rows are read 16 bytes at a time.)
+template <int VT> __global__ __launch_bounds__(256) void bonus_output_kernel(BonusPieces q) {
+    const BonusArgs& p = q.a;
+    constexpr int PR = LC + 4;
+    __shared__ __align__(16) float P[NSB][SB * PR];
+    int t0;
+    const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y;
+    if (n == 0) return;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4, row0 = SB * wave;
+    if (row0 >= n) return;
+    const int d = p.d, vd = p.vd, C = p.H * d, col0 = blockIdx.z * 16 * VT;
+    const float* R = q.rd + (size_t)(t0 + min(row0 + m16, n - 1)) * C + h * d + 4 * kg;
+    const float* K = q.kd + (size_t)(t0 + m16) * C + h * d + 4 * kg;
+    const float* E = q.E + (size_t)blockIdx.x * NSB * C + h * d + 4 * kg;
+    const float* V = p.rkv + (size_t)t0 * p.ldq + p.v_off + h * vd + col0 + m16;
+    const float* S = q.U + ((size_t)blockIdx.x * p.H + h) * d * vd + col0 + m16;
+    f32x4_t sc[NSB - 1], acc[VT];
+#pragma unroll
+    for (int i = 0; i < NSB - 1; ++i) sc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int c = 0; c < VT; ++c) acc[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    // (the operands of the next 16 of the depth are requested before the current ones are multiplied)
+    float4 rn, kn[NSB - 1], en[NSB - 1], k[NSB - 1], e4[NSB - 1];
+    float b[4][VT], bn[4][VT];
+    auto fetch = [&](int j) {
+        rn = *reinterpret_cast<const float4*>(R + j);
+#pragma unroll
+        for (int i = 0; i < NSB - 1; ++i)
+            if (i < wave) { kn[i] = *reinterpret_cast<const float4*>(K + (size_t)i * SB * C + j); en[i] = *reinterpret_cast<const float4*>(E + (size_t)i * C + j); }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) bn[e][c] = col0 + 16 * c < vd ? S[(size_t)(j + 4 * kg + e) * vd + 16 * c] : 0.f;
+    };
+    auto fetch_values = [&](int j) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) {
+                const int t = j + 4 * kg + e;
+                bn[e][c] = (t < n && col0 + 16 * c < vd) ? V[(size_t)t * p.ldq + 16 * c] : 0.f;
+            }
+    };
+    auto take = [&]() {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) b[e][c] = bn[e][c];
+    };
+    fetch(0);
+    float* Pw = P[wave];
+    for (int v = 0; v < 4; ++v) {                            // the scores inside the sub-piece (rows past the portion's end are not stored below)
+        const int r = min(row0 + 4 * kg + v, n - 1);
+        Pw[(4 * kg + v) * PR + row0 + m16] = q.D[((size_t)(t0 + r) * p.H + h) * SB + m16];
+    }
+    for (int j = 0; j < d; j += 16) {
+        float g[4] = {rn.x, rn.y, rn.z, rn.w};
+#pragma unroll
+        for (int i = 0; i < NSB - 1; ++i) { k[i] = kn[i]; e4[i] = en[i]; }
+        take();
+        if (j + 16 < d) fetch(j + 16); else fetch_values(0);
+#pragma unroll
+        for (int i = NSB - 2; i >= 0; --i) {                 // from the sub-piece before this one back to the piece's first
+            if (i >= wave) continue;
+            const float ka[4] = {k[i].x, k[i].y, k[i].z, k[i].w}, ea[4] = {e4[i].x, e4[i].y, e4[i].z, e4[i].w};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) sc[i] = mfma_f32(g[e], ka[e], sc[i]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) g[e] *= ea[e];
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) acc[c] = mfma_f32(g[e], b[e][c], acc[c]);
+    }
+#pragma unroll
+    for (int i = 0; i < NSB - 1; ++i)
+        if (i < wave)
+#pragma unroll
+            for (int v = 0; v < 4; ++v) Pw[(4 * kg + v) * PR + SB * i + m16] = sc[i][v];
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); __builtin_amdgcn_wave_barrier();
+    for (int j = 0; j <= row0; j += 16) {
+        take();
+        if (j + 16 <= row0) fetch_values(j + 16);
+        const float4 a4 = *reinterpret_cast<const float4*>(&Pw[m16 * PR + j + 4 * kg]);
+        const float a[4] = {a4.x, a4.y, a4.z, a4.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int c = 0; c < VT; ++c) acc[c] = mfma_f32(a[e], b[e][c], acc[c]);
+    }
+#pragma unroll
+    for (int c = 0; c < VT; ++c) {
+        if (col0 + 16 * c >= vd) break;
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const int r = row0 + 4 * kg + v;
+            if (r < n) p.o[((size_t)(t0 + r) * p.H + h) * vd + col0 + 16 * c + m16] = acc[c][v];
+        }
+    }
+}
+
 template <typename TO> int pair_launch(const PairStepArgs& p, TO* out1, TO* out2, int T, hipStream_t s_) {
     auto aligned = [](const void* q) { return (uintptr_t)q % 16 == 0; };
     const bool vec = p.width % 4 == 0 && p.seg % 4 == 0 && aligned(p.x) && aligned(p.y1) && aligned(p.y2) && aligned(p.rows) &&
@@ -319,6 +604,12 @@ int mi355_hyb_lowrank_decay(float* log_w, int32_t ldw, const float* z, int32_t l
     LAUNCH_OK(); return 0;
 }
 
+int64_t mi355_hyb_bonus_recurrence_scratch(int32_t num_tokens, int32_t num_seqs, int32_t heads, int32_t dim, int32_t vdim) {
+    if (num_tokens < LC || num_tokens <= 8 * (int64_t)num_seqs || heads <= 0 || dim <= 0 || vdim <= 0 || dim % 16 || vdim % 16 || dim > 512) return 0;
+    const int64_t C = (int64_t)heads * dim, np = (int64_t)num_tokens / LC + num_seqs;
+    return 2 * num_tokens * C + np * (NSB + 1) * C + (int64_t)num_tokens * heads * SB + np * C * vdim;
+}
+
 int mi355_hyb_bonus_recurrence(float* o, float* state, int64_t state_stride, const float* rkv, int32_t ldq, int32_t r_off, int32_t k_off,
                                int32_t v_off, const float* log_w, int32_t ldw, const float* bonus, const uint32_t* context_lens,
                                const uint32_t* cu_seqlens_q, const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads,
@@ -327,10 +618,26 @@ int mi355_hyb_bonus_recurrence(float* o, float* state, int64_t state_stride, con
     if (heads <= 0 || heads > 65535 || dim <= 0 || dim > 512 || vdim <= 0 || r_off < 0 || k_off < 0 || v_off < 0 || ldw < heads * dim) return -1;
     if (ldq < r_off + heads * dim || ldq < k_off + heads * dim || ldq < v_off + heads * vdim) return -1;
     if (num_seqs <= 0 || num_tokens <= 0) return 0;
-    (void)scratch;
     BonusArgs p{o, state, state_stride, rkv, ldq, r_off, k_off, v_off, log_w, ldw, bonus, context_lens, cu_seqlens_q, state_slots, num_seqs, heads, dim,
                 vdim, row, row_state, row_n};
     hipStream_t s_ = to_stream(stream);
+    if (scratch && dim % 16 == 0 && vdim % 16 == 0 && (uintptr_t)scratch % 16 == 0) {
+        const size_t C = (size_t)heads * dim, np = (size_t)num_tokens / LC + num_seqs;
+        BonusPieces q{p, scratch, scratch + num_tokens * C};
+        q.E = q.kd + num_tokens * C;
+        q.ptot = q.E + np * NSB * C;
+        q.D = q.ptot + np * C;
+        q.U = q.D + (size_t)num_tokens * heads * SB;
+        const dim3 pg((unsigned)np, heads);
+        bonus_prepare_kernel<<<pg, 256, 0, s_>>>(q);
+        if (dim <= 64) bonus_state_kernel<4><<<dim3((unsigned)np, heads, (vdim + 63) / 64), 256, 0, s_>>>(q);
+        else bonus_state_kernel<8><<<dim3((unsigned)np, heads, (vdim + 63) / 64), 256, 0, s_>>>(q);
+        bonus_piece_scan_kernel<<<dim3(num_seqs, heads, (dim * vdim + 255) / 256), 256, 0, s_>>>(q);
+        if (vdim <= 32) bonus_output_kernel<2><<<pg, 256, 0, s_>>>(q);
+        else if (vdim <= 64) bonus_output_kernel<4><<<pg, 256, 0, s_>>>(q);
+        else bonus_output_kernel<8><<<dim3((unsigned)np, heads, (vdim + 127) / 128), 256, 0, s_>>>(q);
+        LAUNCH_OK(); return 0;
+    }
     if (dim < 64) {
         const dim3 grid(num_seqs, heads, (vdim + 63) / 64);
         if (dim <= 16) bonus_scan_kernel<4, 4, 8><<<grid, 256, 0, s_>>>(p);

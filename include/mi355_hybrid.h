@@ -574,11 +574,15 @@ int mi355_hyb_lowrank_decay(float* log_w, int32_t ldw, const float* z, int32_t l
 /* recurrence with a decay per key channel and a bonus for the current token over the new tokens of every sequence, state f32 [slots] x
  * [heads, dim, vdim] (stride in floats): o f32 [T, heads, vdim] = (S + diag(bonus) k v^T)^T r, then S <- diag(exp(log_w)) S + k v^T.
  * rkv f32 [T, ldq] holds r, k (heads x dim) and v (heads x vdim) at their offsets; log_w f32 [T, ldw] (heads x dim), bonus f32 [heads, dim].
- * row != NULL: row f32 [num_seqs, row_n] moves into row_state (f32 per slot, the same stride).  dim <= 512 */
+ * row != NULL: row f32 [num_seqs, row_n] moves into row_state (f32 per slot, the same stride).  dim <= 512.  scratch != NULL (16-byte
+ * aligned, the floats below; dim and vdim multiples of 16): portions are cut into pieces of 64 tokens that are worked on side by side on the
+ * f32 matrix cores; NULL: one scan over the tokens */
 int mi355_hyb_bonus_recurrence(float* o, float* state, int64_t state_stride, const float* rkv, int32_t ldq, int32_t r_off, int32_t k_off,
                                int32_t v_off, const float* log_w, int32_t ldw, const float* bonus, const uint32_t* context_lens,
                                const uint32_t* cu_seqlens_q, const int32_t* state_slots, int32_t num_seqs, int32_t num_tokens, int32_t heads,
                                int32_t dim, int32_t vdim, const float* row, float* row_state, int32_t row_n, float* scratch, int64_t stream);
+/* floats of `scratch` that suit a step of this size; 0: the scan suits it (few tokens per sequence, or sizes that only the scan serves) */
+int64_t mi355_hyb_bonus_recurrence_scratch(int32_t num_tokens, int32_t num_seqs, int32_t heads, int32_t dim, int32_t vdim);
 /* mi355_hyb_gated_norm with weights per head: head h's start at w + h w_ld (w_ld 0: the same for all heads) */
 int mi355_hyb_gated_norm_heads(void* out, int32_t out_dtype, int32_t ldo, int32_t out_off, const float* o, const float* w, int32_t w_ld,
                                const float* gate_in, int32_t ldg, int32_t gate, int32_t num_tokens, int32_t heads, int32_t vdim, float eps,

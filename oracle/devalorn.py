@@ -122,7 +122,7 @@ def time_mixing(h, W, p, c, eps):
     """the right branch, up to its output projection"""
     T, H, d = h.shape[0], c["heads"], c["dim"]
     xr, xk, xv, xg, xw = token_mixes(h, [W[p + "mu." + n] for n in "rkvgw"])
-    r, k, v = ((x @ W[p + n].T).reshape(T, H, d) for x, n in ((xr, "r"), (xk, "k"), (xv, "v")))
+    r, k, v = ((x @ W[p + n].T).reshape(T, H, -1) for x, n in ((xr, "r"), (xk, "k"), (xv, "v")))
     w = lowrank_decay(xw, W[p + "w1"], W[p + "w2"], W[p + "w0"]).reshape(T, H, d)
     o, _ = bonus_recurrence(r, k, v, w, W[p + "u"].reshape(H, d))
     return head_norm_gate(o, W[p + "norm"], silu(xg @ W[p + "g"].T), eps)
@@ -196,3 +196,62 @@ def forward(cfg, W, tokens, margins=None, operand=None):
         x = x + y
         trace.append(x)
     return (unit_rms(x, eps) * W["final.norm"]) @ W["head"].T, np.stack(trace)
+
+
+# ---------------------------------------------------------------------------------------------------------------- weights for tests
+def bf16_round(a):
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    r = ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint32) << 16
+    return r.view(np.float32).astype(np.float64)
+
+
+def random_devalorn(rng, cfg, rank=6, right_vdim=None):
+    """random bf16-representable weights for a config (f64 arrays): projections ~ N(0, 1/in), norms near 1, decays from nearly none to
+    a tenth per token, mixtures that take anything from none to all of the token before"""
+    W = {}
+
+    def mat(name, rows, cols, s=None):
+        W[name] = bf16_round(rng.standard_normal((rows, cols)) * (s if s is not None else 1.0 / math.sqrt(cols)))
+
+    def vec(name, n, mean=0.0, s=0.1):
+        W[name] = bf16_round(mean + s * rng.standard_normal(n))
+
+    def attention(q, c):
+        H, G, d, vd = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
+        mat(q + "q", H * d, Wd)
+        if c.get("kv_from") is None:
+            mat(q + "k", G * d, Wd); mat(q + "v", G * vd, Wd)
+        mat(q + "o", Wd, H * vd)
+
+    Wd, V = cfg["width"], cfg["vocab"]
+    mat("embed", V, Wd, 1.0)
+    vec("final.norm", Wd, 1.0)
+    mat("head", V, Wd, 2.0 / math.sqrt(Wd))
+    for i, lc in enumerate(cfg["layers"]):
+        p, c, m = "l%d." % i, lc["mixer"], lc.get("mlp")
+        vec(p + "norm1", Wd, 1.0)
+        if lc["type"] == "parallel":
+            attention(p + "mix.left.", c["left"])
+            mat(p + "mix.left.g", c["left"]["heads"], Wd, 2.0 / math.sqrt(Wd))
+            q, H, d = p + "mix.right.", c["right"]["heads"], c["right"]["dim"]
+            vd = right_vdim or d
+            for n in "rkvgw":
+                W[q + "mu." + n] = bf16_round(rng.uniform(0, 1, Wd))
+            mat(q + "r", H * d, Wd); mat(q + "k", H * d, Wd); mat(q + "v", H * vd, Wd); mat(q + "g", H * vd, Wd)
+            mat(q + "w1", rank, Wd); mat(q + "w2", H * d, rank)
+            W[q + "w0"] = bf16_round(rng.uniform(-6, 1, H * d))
+            vec(q + "u", (H, d), 0.3, 0.5); vec(q + "norm", H * vd, 1.0); mat(q + "o", Wd, H * vd)
+        else:
+            attention(p + "mix.", c)
+            vec(p + "mix.q.norm", c["heads"] * c["dim"], 1.0, 0.2)
+            if c.get("kv_from") is None:
+                vec(p + "mix.k.norm", c["kv_heads"] * c["dim"], 1.0, 0.2)
+        if not m:
+            continue
+        vec(p + "norm2", Wd, 1.0)
+        for e in ([""] if m["kind"] == "dense" else ["e%d." % e for e in range(m["router"]["experts"])]):
+            ff = m["ff"] if m["kind"] == "dense" else m["expert"]["ff"]
+            mat(p + "mlp." + e + "gate", ff, Wd); mat(p + "mlp." + e + "up", ff, Wd); mat(p + "mlp." + e + "down", Wd, ff)
+        if m["kind"] == "moe":
+            mat(p + "mlp.router", m["router"]["experts"], Wd, 2.0 / math.sqrt(Wd))
+    return W
