@@ -456,6 +456,9 @@ _sig("mi355_hyb_norm_sigmoid_gate", ctypes.c_int, [c_vp, c_i32, c_vp, c_vp, c_i3
 _sig("mi355_hyb_decay_attention", ctypes.c_int, [c_vp, c_vp, c_i64, c_vp, c_i32, c_i32, c_i32, c_i32] + [c_vp] * 4 + [c_i32] * 5 + [c_vp, c_i64])
 _sig("mi355_hyb_decay_attention_scratch", c_i64, [c_i32] * 5)
 _sig("mi355_hyb_linear_segments", ctypes.c_int, [c_vp, c_i32, c_vp, c_i32, c_i32, c_i64, c_i32, c_vp, c_vp, c_vp] + [c_i32] * 5 + [c_i64])
+_sig("mi355_hyb_linear_glu", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i32, c_vp] + [c_i32] * 5 + [c_i64])
+_sig("mi355_hyb_linear_grouped_glu", ctypes.c_int, [c_vp, c_i32, c_i32, c_vp, c_i32, c_vp, c_vp, c_i64, c_vp] + [c_i32] * 6 + [c_i64])
+_sig("mi355_hyb_interleave_gate_up", ctypes.c_int, [c_vp, c_vp] + [c_i32] * 4 + [c_i64])
 _sig("mi355_hyb_pair_step", ctypes.c_int, [c_vp] * 6 + [c_i32] + [c_vp] * 4 + [c_i64, c_vp, c_i32, c_vp, c_vp, c_i32, c_vp, c_i64] + [c_vp] * 5 +
      [c_i32, c_i32, c_f32, c_i64])
 _sig("mi355_hyb_lowrank_decay", ctypes.c_int, [c_vp, c_i32, c_vp, c_i32, c_vp, c_vp, c_i32, c_i32, c_i32, c_i64])

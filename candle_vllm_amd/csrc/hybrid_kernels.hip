@@ -56,9 +56,11 @@ struct LinArgs {
     int act, act_cols, out16;
     // segments: columns [.., seg_end[i]) are a product of their own left operand, a + (seg0 + i) seg_a elements (ends are multiples of 128)
     int n_seg, seg0; int64_t seg_a; int seg_end[LIN_MAX_SEG];
+    // gate/up pairs: the rows of w come as 16 gate rows, their 16 up rows, the next 16 gate rows, ...; out [T, N / 2] = act(gate) up
+    int glu;
 };
 // (what a product can do beyond the plain one is a build of its own, so that the plain products pay nothing for it)
-enum { LIN_PLAIN = 0, LIN_EPI_BUILD = 1, LIN_SEG_BUILD = 2 };
+enum { LIN_PLAIN = 0, LIN_EPI_BUILD = 1, LIN_SEG_BUILD = 2, LIN_GLU_BUILD = 3 };
 template <int B> __device__ __forceinline__ void lin_store(const LinArgs& p, int t, int n, float v) {
     if (B == LIN_EPI_BUILD) {
         if (p.act && n < p.act_cols) {
@@ -69,6 +71,11 @@ template <int B> __device__ __forceinline__ void lin_store(const LinArgs& p, int
         if (p.out16) { reinterpret_cast<uint16_t*>(p.out)[(size_t)t * p.ldo + n] = f32_to_bf16(v); return; }
     }
     p.out[(size_t)t * p.ldo + n] = v;
+}
+__device__ __forceinline__ void lin_store_glu(const LinArgs& p, int t, int c, float g, float u) {
+    const float v = (p.act == MI355_HYB_ACT_GELU ? gelu_tanhf_(g) : siluf_(g)) * u;
+    if (p.out16) reinterpret_cast<uint16_t*>(p.out)[(size_t)t * p.ldo + c] = f32_to_bf16(v);
+    else p.out[(size_t)t * p.ldo + c] = v;
 }
 // the block's matrix and the end of its rows (one past the last); false = nothing to do
 __device__ __forceinline__ bool lin_group(LinArgs& p, int t0, int64_t& w_off) {
@@ -100,8 +107,9 @@ template <typename TA, int B> __device__ __forceinline__ void lin_batch(LinArgs&
 // 32-wide K step on both sides, the accumulator holds tokens 4 kg + v of column m16.
 template <typename TA, int MT, int B> __global__ __launch_bounds__(256) void linear_bf16_tile_kernel(LinArgs p) {
     lin_batch<TA, B>(p, blockIdx.x * 64);
+    constexpr int NC = B == LIN_GLU_BUILD ? 2 : 1;                  // column tiles per wave: a gate tile and its up tile
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4;
-    const int n = blockIdx.x * 64 + wave * 16 + m16;
+    const int n = (blockIdx.x * 64 + wave * 16) * NC + m16;
     const int t0 = blockIdx.y * (16 * MT);
     int64_t w_off;
     if (!lin_group(p, t0, w_off)) return;
@@ -114,17 +122,22 @@ template <typename TA, int MT, int B> __global__ __launch_bounds__(256) void lin
         aok[i] = t < p.T;
         arow[i] = static_cast<const TA*>(p.a) + (size_t)(aok[i] ? lin_row(p, t) : 0) * p.lda;
     }
-    f32x4_t acc[MT];
+    f32x4_t acc[NC][MT];
 #pragma unroll
-    for (int i = 0; i < MT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+        for (int i = 0; i < MT; ++i) acc[c][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     const bool nok = n < p.N;
     for (int k0 = 0; k0 < p.K; k0 += 32) {
         const int k = k0 + 8 * kg;
-        const uint4 b = nok ? frag8<uint16_t>(wrow, k, p.K, p.w_vec) : uint4{0, 0, 0, 0};
+        uint4 b[NC];
+#pragma unroll
+        for (int c = 0; c < NC; ++c) b[c] = nok ? frag8<uint16_t>(wrow + (size_t)(16 * c) * p.K, k, p.K, p.w_vec) : uint4{0, 0, 0, 0};
 #pragma unroll
         for (int i = 0; i < MT; ++i) {
             const uint4 a = aok[i] ? frag8<TA>(arow[i], k, p.K, p.a_vec) : uint4{0, 0, 0, 0};
-            acc[i] = mfma_bf16(a, b, acc[i]);
+#pragma unroll
+            for (int c = 0; c < NC; ++c) acc[c][i] = mfma_bf16(a, b[c], acc[c][i]);
         }
     }
     if (!nok) return;
@@ -134,7 +147,9 @@ template <typename TA, int MT, int B> __global__ __launch_bounds__(256) void lin
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const int t = t0 + i * 16 + 4 * kg + v;
-            if (t < p.T) lin_store<B>(p, t, n, acc[i][v] + bias);
+            if (t >= p.T) continue;
+            if (B == LIN_GLU_BUILD) lin_store_glu(p, t, blockIdx.x * 64 + wave * 16 + m16, acc[0][i][v], acc[NC - 1][i][v]);
+            else lin_store<B>(p, t, n, acc[0][i][v] + bias);
         }
 }
 
@@ -202,6 +217,21 @@ template <int B> __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(L
         if (more) stage(buf ^ 1);
         __syncthreads();
     }
+    if (B == LIN_GLU_BUILD) {
+#pragma unroll
+        for (int j = 0; j < 4; j += 2) {
+            const int n = n0 + wc * 64 + j * 16;
+            if (n >= p.N) continue;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const int t = t0 + wr * 64 + i * 16 + 4 * kg + v;
+                    if (t < p.T) lin_store_glu(p, t, n / 2 + m16, acc[i][j][v], acc[i][j + 1][v]);
+                }
+        }
+        return;
+    }
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
         const int n = n0 + wc * 64 + j * 16 + m16;
@@ -220,40 +250,54 @@ template <int B> __global__ __launch_bounds__(256) void linear_bf16_lds_kernel(L
 // Up to 16 tokens, bf16 weights: the product is a stream over the weights.  A workgroup owns 16 weight rows; its NW waves take the
 // 32-wide K steps in turn (UNR steps in flight per wave) and add their partial tiles through LDS.
 template <typename TA, int NW, int UNR, int B> __global__ __launch_bounds__(64 * NW) void linear_bf16_stream_kernel(LinArgs p) {
-    __shared__ float part[NW][4][64];
+    constexpr int NC = B == LIN_GLU_BUILD ? 2 : 1;                  // column tiles: a gate tile and its up tile
+    __shared__ float part[NW][4 * NC][64];
     lin_batch<TA, B>(p, blockIdx.x * 16);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m16 = lane & 15, kg = lane >> 4;
-    const int n = blockIdx.x * 16 + m16;
+    const int n = blockIdx.x * 16 * NC + m16;
     const int t0 = blockIdx.y * 16;                                  // a grouped product: block blockIdx.y of 16 rows; else 0
     int64_t w_off;
     if (!lin_group(p, t0, w_off)) return;
     const bool nok = n < p.N, aok = t0 + m16 < p.T;
     const uint16_t* wrow = static_cast<const uint16_t*>(p.w) + w_off + (size_t)(nok ? n : 0) * p.K;
     const TA* arow = static_cast<const TA*>(p.a) + (size_t)(aok ? lin_row(p, t0 + m16) : 0) * p.lda;
-    f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    f32x4_t acc[NC];
+#pragma unroll
+    for (int c = 0; c < NC; ++c) acc[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     for (int k0 = wave * 32 * UNR; k0 < p.K; k0 += NW * 32 * UNR) {
-        uint4 a[UNR], b[UNR];
+        uint4 a[UNR], b[NC][UNR];
 #pragma unroll
         for (int u = 0; u < UNR; ++u) {
             const int k = k0 + u * 32 + 8 * kg;
-            b[u] = (nok && k < p.K) ? frag8<uint16_t>(wrow, k, p.K, p.w_vec) : uint4{0, 0, 0, 0};
+#pragma unroll
+            for (int c = 0; c < NC; ++c) b[c][u] = (nok && k < p.K) ? frag8<uint16_t>(wrow + (size_t)(16 * c) * p.K, k, p.K, p.w_vec) : uint4{0, 0, 0, 0};
             a[u] = (aok && k < p.K) ? frag8<TA>(arow, k, p.K, p.a_vec) : uint4{0, 0, 0, 0};
         }
 #pragma unroll
-        for (int u = 0; u < UNR; ++u) acc = mfma_bf16(a[u], b[u], acc);
+        for (int u = 0; u < UNR; ++u)
+#pragma unroll
+            for (int c = 0; c < NC; ++c) acc[c] = mfma_bf16(a[u], b[c][u], acc[c]);
     }
 #pragma unroll
-    for (int v = 0; v < 4; ++v) part[wave][v][lane] = acc[v];
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) part[wave][4 * c + v][lane] = acc[c][v];
     __syncthreads();
     if (wave == 0) {
         const float bias = (p.bias && nok) ? p.bias[n] : 0.f;
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
-            float s = 0.f;
+            float s[NC];
 #pragma unroll
-            for (int w = 0; w < NW; ++w) s += part[w][v][lane];
+            for (int c = 0; c < NC; ++c) {
+                s[c] = 0.f;
+#pragma unroll
+                for (int w = 0; w < NW; ++w) s[c] += part[w][4 * c + v][lane];
+            }
             const int t = t0 + 4 * kg + v;
-            if (nok && t < p.T) lin_store<B>(p, t, n, s + bias);
+            if (!nok || t >= p.T) continue;
+            if (B == LIN_GLU_BUILD) lin_store_glu(p, t, blockIdx.x * 16 + m16, s[0], s[NC - 1]);
+            else lin_store<B>(p, t, n, s[0] + bias);
         }
     }
 }
@@ -295,11 +339,14 @@ template <int B> __global__ __launch_bounds__(256) void linear_f32_kernel(LinArg
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const int t = t0 + ty * 4 + i;
-        if (t >= p.T) continue;
+        if (B != LIN_GLU_BUILD && t >= p.T) continue;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < p.N) lin_store<B>(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
+            if (B == LIN_GLU_BUILD) {                                       // the up column of a gate column is four threads further
+                const float up = __shfl_xor(acc[i][j], 4);
+                if (!(tx & 4) && n < p.N && t < p.T) lin_store_glu(p, t, (n & ~31) / 2 + (n & 15), acc[i][j], up);
+            } else if (n < p.N) lin_store<B>(p, t, n, acc[i][j] + (p.bias ? p.bias[n] : 0.f));
         }
     }
 }
@@ -1786,6 +1833,15 @@ __global__ void scale_f32_kernel(float* x, float s, int64_t n) {
     if (i < n) x[i] *= s;
 }
 
+// a matrix of ff gate rows and ff up rows -> 16 gate rows, their 16 up rows, the next 16 gate rows, ...  (a workgroup per row)
+template <typename T> __global__ void interleave_gate_up_kernel(T* out, const T* in, int ff, int k) {
+    const int r = blockIdx.x, up = r >= ff, j = r - up * ff;
+    const size_t base = (size_t)blockIdx.y * 2 * ff;
+    const T* src = in + (base + r) * k;
+    T* dst = out + (base + (size_t)(j / 16) * 32 + up * 16 + j % 16) * k;
+    for (int i = threadIdx.x; i < k; i += blockDim.x) dst[i] = src[i];
+}
+
 int g_attn_wider = 1;           // A/B: twelve waves per (token, head) for the smallest decoding batches
 int g_attn_group = 1;           // 0: grouped-query prompt steps take the kernel with one wave per head (A/B, tests of both paths)
 int g_attn_mfma = 1;            // mi355_hyb_set_attention_mfma(0): prompt steps take the generic kernel too (A/B, tests of both paths)
@@ -1819,18 +1875,21 @@ int mi355_hyb_fill_f32(float* out, float v, int64_t n, int64_t stream) {
 }
 
 // which build of a product kernel: with an activation or a 16-bit result, or the plain one
-#define LIN_EPI(p, CALL) do { if ((p).n_seg) { constexpr int EPI = LIN_SEG_BUILD; CALL; } else if ((p).act || (p).out16) { constexpr int EPI = LIN_EPI_BUILD; CALL; } \
+#define LIN_EPI(p, CALL) do { if ((p).glu) { constexpr int EPI = LIN_GLU_BUILD; CALL; } else LIN_EPI_(p, CALL); } while (0)
+#define LIN_EPI_(p, CALL) do { if ((p).n_seg) { constexpr int EPI = LIN_SEG_BUILD; CALL; } else if ((p).act || (p).out16) { constexpr int EPI = LIN_EPI_BUILD; CALL; } \
                               else { constexpr int EPI = LIN_PLAIN; CALL; } } while (0)
-// (the experts' products have no segments)
-#define LIN_EPI2(p, CALL) do { if ((p).act || (p).out16) { constexpr int EPI = LIN_EPI_BUILD; CALL; } else { constexpr int EPI = LIN_PLAIN; CALL; } } while (0)
+// (the experts' products have no segments; a gate/up product's operands are both of the model's type)
+#define LIN_EPI2(p, CALL) do { if ((p).glu) { constexpr int EPI = LIN_GLU_BUILD; CALL; } else LIN_EPI2_(p, CALL); } while (0)
+#define LIN_EPI2_(p, CALL) do { if ((p).act || (p).out16) { constexpr int EPI = LIN_EPI_BUILD; CALL; } else { constexpr int EPI = LIN_PLAIN; CALL; } } while (0)
 struct LinSegments { int32_t n, first; int64_t a_stride; const int32_t* rows; };
 static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, int32_t a_dtype, int32_t lda, int64_t a_bs, const void* w,
                          int64_t w_bs, const float* bias, int32_t T, int32_t n, int32_t k, int32_t batch, int32_t dtype, int64_t stream,
-                         int32_t act = 0, int32_t act_cols = 0, int32_t out16 = 0, const LinSegments* seg = nullptr) {
-    if (!out || !a || !w || T < 0 || n <= 0 || k <= 0 || ldo < n || lda < k || batch <= 0 || batch > 65535 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
+                         int32_t act = 0, int32_t act_cols = 0, int32_t out16 = 0, const LinSegments* seg = nullptr, int32_t glu = 0) {
+    if (!out || !a || !w || T < 0 || n <= 0 || k <= 0 || ldo < (glu ? n / 2 : n) || lda < k || batch <= 0 || batch > 65535 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
     if (T == 0) return 0;
     LinArgs p{out, ldo, a, lda, w, bias, T, n, k, 0, 0, a_bs, w_bs, o_bs};
-    p.act = act; p.act_cols = act_cols; p.out16 = out16;
+    p.act = act; p.act_cols = act_cols; p.out16 = out16; p.glu = glu;
+    if (glu && (n % 32 || a_dtype != dtype || bias)) return -1;
     if (seg) {
         if (seg->n < 1 || seg->n > LIN_MAX_SEG || seg->first < 0 || seg->a_stride < 0 || !seg->rows || batch != 1 || act || out16) return -1;
         int end = 0;
@@ -1851,17 +1910,17 @@ static int linear_launch(float* out, int32_t ldo, int64_t o_bs, const void* a, i
     p.a_vec = ((size_t)lda * a_bytes % 16 == 0) && ((uintptr_t)a % 16 == 0) && ((size_t)a_bs * a_bytes % 16 == 0);
     const bool af = a_dtype == MI355_DTYPE_F32;
     if (T <= 16) {
-        const dim3 grid((n + 15) / 16, 1, nz);
-        if (k >= 2048) { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
-        else { if (af) LIN_EPI(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
+        const dim3 grid(glu ? n / 32 : (n + 15) / 16, 1, nz);
+        if (k >= 2048) { if (af) LIN_EPI_(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
+        else { if (af) LIN_EPI_(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
     } else if (T > 32 && !af && p.a_vec && p.w_vec && k % 32 == 0) {
         LIN_EPI(p, (linear_bf16_lds_kernel<EPI><<<dim3((n + 127) / 128, (T + 127) / 128, nz), 256, 0, st_>>>(p)));
     } else if (T <= 32) {
-        const dim3 grid((n + 63) / 64, (T + 31) / 32, nz);
-        if (af) LIN_EPI(p, (linear_bf16_tile_kernel<float, 2, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 2, EPI><<<grid, 256, 0, st_>>>(p)));
+        const dim3 grid(glu ? (n + 127) / 128 : (n + 63) / 64, (T + 31) / 32, nz);
+        if (af) LIN_EPI_(p, (linear_bf16_tile_kernel<float, 2, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 2, EPI><<<grid, 256, 0, st_>>>(p)));
     } else {
-        const dim3 grid((n + 63) / 64, (T + 63) / 64, nz);
-        if (af) LIN_EPI(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
+        const dim3 grid(glu ? (n + 127) / 128 : (n + 63) / 64, (T + 63) / 64, nz);
+        if (af) LIN_EPI_(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
     }
     LAUNCH_OK(); return 0;
 }
@@ -2054,13 +2113,15 @@ int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t ou
         const int dk = dim / 32, vt = vdim / 16;
         // grouped-query attention: the query heads of a key/value head share a workgroup and its staged rows
         const int hpk = heads / kv_heads, hpg = cross ? 1 : (hpk % 4 == 0 ? 4 : hpk % 3 == 0 ? 3 : hpk % 2 == 0 ? 2 : 1);
-        if (hpg > 1 && dk <= 4 && vt <= 8 && vt % 2 == 0 && g_attn_group) {
+        if (hpg > 1 && ((dk <= 4 && vt <= 8 && vt % 2 == 0) || (dk == 3 && vt == 12) || (dk == 4 && vt == 16)) && g_attn_group) {
             const dim3 ggrid((T + 15) / 16 + num_seqs, heads / hpg, 1);
 #define WG2(DK, VT) do { if (hpg == 4) window_attention_group_kernel<DK, VT, 4><<<ggrid, 256, 0, s_>>>(p); \
                          else if (hpg == 3) window_attention_group_kernel<DK, VT, 3><<<ggrid, 192, 0, s_>>>(p); \
                          else window_attention_group_kernel<DK, VT, 2><<<ggrid, 128, 0, s_>>>(p); } while (0)
 #define WGV(DK) do { switch (vt) { case 2: WG2(DK, 2); break; case 4: WG2(DK, 4); break; case 6: WG2(DK, 6); break; default: WG2(DK, 8); break; } } while (0)
-            switch (dk) { case 1: WGV(1); break; case 2: WGV(2); break; case 3: WGV(3); break; default: WGV(4); break; }
+            if (vt == 12) WG2(3, 12);
+            else if (vt == 16) WG2(4, 16);
+            else switch (dk) { case 1: WGV(1); break; case 2: WGV(2); break; case 3: WGV(3); break; default: WGV(4); break; }
 #undef WGV
 #undef WG2
             LAUNCH_OK(); return 0;
@@ -2406,15 +2467,16 @@ int mi355_hyb_linear_grouped(float* out, int32_t ldo, const void* a, int32_t a_d
                                         MI355_HYB_ACT_NONE, dtype, stream);
 }
 
-int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const int32_t* row_token,
-                                 const void* w, int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t n,
-                                 int32_t k, int32_t act, int32_t dtype, int64_t stream) {
+static int grouped_launch(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const int32_t* row_token,
+                          const void* w, int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t n,
+                          int32_t k, int32_t act, int32_t glu, int32_t dtype, int64_t stream) {
     if (act < 0 || act > MI355_HYB_ACT_RELU2 || !is_dt(out_dtype)) return -1;
-    if (!out || !a || !w || !block_table || n <= 0 || k <= 0 || ldo < n || lda < k || w_bs < 0 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
+    if (glu && (n % 32 || a_dtype != dtype)) return -1;
+    if (!out || !a || !w || !block_table || n <= 0 || k <= 0 || ldo < (glu ? n / 2 : n) || lda < k || w_bs < 0 || !is_dt(dtype) || !is_dt(a_dtype)) return -1;
     if (n_blocks <= 0) return 0;
     if (n_blocks > 65535) return -1;
     LinArgs p{static_cast<float*>(out), ldo, a, lda, w, nullptr, n_blocks * block_rows, n, k, 0, 0, 0, w_bs, 0, block_table, row_token, block_rows};
-    p.act = act; p.act_cols = n; p.out16 = out_dtype == MI355_DTYPE_BF16;
+    p.act = act; p.act_cols = n; p.glu = glu; p.out16 = out_dtype == MI355_DTYPE_BF16;
     hipStream_t st_ = to_stream(stream);
     if (dtype == MI355_DTYPE_F32) {
         if (a_dtype != MI355_DTYPE_F32 || block_rows != 64) return -1;
@@ -2426,17 +2488,42 @@ int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, cons
     p.a_vec = ((size_t)lda * a_bytes % 16 == 0) && ((uintptr_t)a % 16 == 0);
     const bool af = a_dtype == MI355_DTYPE_F32;
     if (block_rows == 16) {
-        const dim3 grid((n + 15) / 16, n_blocks, 1);
-        if (k >= 2048) { if (af) LIN_EPI2(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
-        else { if (af) LIN_EPI2(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
+        const dim3 grid(glu ? n / 32 : (n + 15) / 16, n_blocks, 1);
+        if (k >= 2048) { if (af) LIN_EPI2_(p, (linear_bf16_stream_kernel<float, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_stream_kernel<uint16_t, 4, 4, EPI><<<grid, 256, 0, st_>>>(p))); }
+        else { if (af) LIN_EPI2_(p, (linear_bf16_stream_kernel<float, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_stream_kernel<uint16_t, 2, 2, EPI><<<grid, 128, 0, st_>>>(p))); }
     } else if (block_rows == 64) {
-        const dim3 grid((n + 63) / 64, n_blocks, 1);
-        if (af) LIN_EPI2(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
+        const dim3 grid(glu ? (n + 127) / 128 : (n + 63) / 64, n_blocks, 1);
+        if (af) LIN_EPI2_(p, (linear_bf16_tile_kernel<float, 4, EPI><<<grid, 256, 0, st_>>>(p))); else LIN_EPI2(p, (linear_bf16_tile_kernel<uint16_t, 4, EPI><<<grid, 256, 0, st_>>>(p)));
     } else if (block_rows == 128 && !af && p.a_vec && p.w_vec && k % 32 == 0) {
         LIN_EPI2(p, (linear_bf16_lds_kernel<EPI><<<dim3((n + 127) / 128, n_blocks, 1), 256, 0, st_>>>(p)));
     } else {
         return -1;
     }
+    LAUNCH_OK(); return 0;
+}
+
+int mi355_hyb_linear_grouped_act(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, const int32_t* row_token,
+                                 const void* w, int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t n,
+                                 int32_t k, int32_t act, int32_t dtype, int64_t stream) {
+    return grouped_launch(out, out_dtype, ldo, a, a_dtype, lda, row_token, w, w_bs, block_table, block_rows, n_blocks, n, k, act, 0, dtype, stream);
+}
+int mi355_hyb_linear_grouped_glu(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t lda, const int32_t* row_token, const void* w,
+                                 int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t ff, int32_t k, int32_t act,
+                                 int32_t dtype, int64_t stream) {
+    if (act != MI355_HYB_ACT_SILU && act != MI355_HYB_ACT_GELU) return -1;
+    return grouped_launch(out, out_dtype, ldo, a, dtype, lda, row_token, w, w_bs, block_table, block_rows, n_blocks, 2 * ff, k, act, 1, dtype, stream);
+}
+int mi355_hyb_linear_glu(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t lda, const void* w, int32_t T, int32_t ff, int32_t k,
+                         int32_t act, int32_t dtype, int64_t stream) {
+    if ((act != MI355_HYB_ACT_SILU && act != MI355_HYB_ACT_GELU) || !is_dt(out_dtype)) return -1;
+    return linear_launch(static_cast<float*>(out), ldo, 0, a, dtype, lda, 0, w, 0, nullptr, T, 2 * ff, k, 1, dtype, stream, act, 0,
+                         out_dtype == MI355_DTYPE_BF16, nullptr, 1);
+}
+int mi355_hyb_interleave_gate_up(void* out, const void* in, int32_t matrices, int32_t ff, int32_t k, int32_t dtype, int64_t stream) {
+    if (!out || !in || out == in || matrices <= 0 || ff <= 0 || ff % 16 || k <= 0 || !is_dt(dtype)) return -1;
+    const dim3 grid(2 * ff, matrices);
+    if (dtype == MI355_DTYPE_F32) interleave_gate_up_kernel<float><<<grid, 256, 0, to_stream(stream)>>>((float*)out, (const float*)in, ff, k);
+    else interleave_gate_up_kernel<uint16_t><<<grid, 256, 0, to_stream(stream)>>>((uint16_t*)out, (const uint16_t*)in, ff, k);
     LAUNCH_OK(); return 0;
 }
 

@@ -79,6 +79,10 @@ struct HLayer {
     int conv_channels() const { return 2 * c.d_kv_heads * c.d_dim + c.d_heads * c.d_vdim; }
     int a_conv_channels() const { return (c.a_heads + c.a_kv_heads) * c.a_dim + c.a_kv_heads * c.a_vdim; }
     // elements of a token's row in the key / value pages (latent attention: one row [latent | rotated key part], no value pages)
+    // gate and up rows are stored interleaved by 16 so that the activation is the product's epilogue: the experts', and the dense
+    // feed-forward's where its activation is silu or gelu
+    bool glu_experts() const { return c.mlp_kind == 3 && !c.moe_relu2 && c.mlp_ff % 16 == 0; }
+    bool glu_dense() const { return (c.mlp_kind == 2 || c.mlp_kind == 6) && c.mlp_ff % 16 == 0; }
     // a shared expert of the experts' size runs as one more group of the grouped products (and one more pair of every token)
     bool shared_merged() const { return c.mlp_kind == 3 && c.moe_shared_ff > 0 && c.moe_shared_ff == c.mlp_ff; }
     int k_row() const { return is_latent() ? c.a_kv_rank + c.a_rot_dim : c.a_kv_heads * c.a_dim; }
@@ -348,6 +352,24 @@ int store_weight(HModel* m, int layer, int which, const uint16_t* dev_bits, int6
     if (w->p) { (void)hipFree(w->p); w->p = nullptr; }
     HHIP(hipMalloc(&w->p, (size_t)n * (as_bf16 ? 2 : 4)));
     w->n = n;
+    const HLayer* L = layer >= 0 ? &m->layers[layer] : nullptr;
+    if (L && ((which == MI355_HW_MOE_GATE_UP && L->glu_experts()) || (which == MI355_HW_MLP_GATE_UP && L->glu_dense()))) {
+        const int64_t per = (int64_t)2 * L->c.mlp_ff * m->cfg.width;
+        const void* src = dev_bits;
+        float* wide = nullptr;
+        if (!as_bf16) {
+            HHIP(hipMalloc(reinterpret_cast<void**>(&wide), (size_t)n * 4));
+            const int rc = mi355_hyb_bf16_to_f32(wide, dev_bits, n, stream);
+            if (rc != 0) { (void)hipFree(wide); return rc; }
+            src = wide;
+        }
+        int rc = mi355_hyb_interleave_gate_up(w->p, src, (int32_t)(n / per), L->c.mlp_ff, m->cfg.width, m->cfg.dtype, stream);
+        if (wide) {
+            if (rc == 0) rc = (int)hipStreamSynchronize(reinterpret_cast<hipStream_t>(stream));
+            (void)hipFree(wide);
+        }
+        return rc;
+    }
     if (as_bf16) HHIP(hipMemcpyAsync(w->p, dev_bits, (size_t)n * 2, hipMemcpyDeviceToDevice, reinterpret_cast<hipStream_t>(stream)));
     else HCHECK(mi355_hyb_bf16_to_f32(static_cast<float*>(w->p), dev_bits, n, stream));
     return 0;
@@ -748,6 +770,27 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
         if (to) xcur = to;
         return 0;
     };
+    // gate, up and silu of all experts (behind the grouping): one product with the activation in its epilogue, or a product and a launch
+    auto expert_gate_up = [&](const HLayer& WL, int bm, int nb) -> int {
+        const int ff = WL.c.mlp_ff;
+        if (WL.glu_experts())
+            return mi355_hyb_linear_grouped_glu(m->moe_act, dt, ff, xin, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)2 * ff * W, m->moe_table,
+                                                bm, nb, ff, W, MI355_HYB_ACT_SILU, dt, stream);
+        HCHECK(mi355_hyb_linear_grouped(m->moe_gu, 2 * ff, xin, xin_dt, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)2 * ff * W,
+                                        m->moe_table, bm, nb, 2 * ff, W, dt, stream));
+        return mi355_hyb_silu_glu(m->moe_act, dt, m->moe_gu, nb * bm, ff, m->moe_table, bm, stream);
+    };
+    // gate, up and activation of a dense feed-forward (kinds 1, 2, 6)
+    auto dense_gate_up = [&](const HLayer& WL) -> int {
+        const int ff = WL.c.mlp_ff, kind = WL.c.mlp_kind;
+        if (WL.glu_dense())
+            return mi355_hyb_linear_glu(m->act, dt, ff, xin, W, WL.w[MI355_HW_MLP_GATE_UP].p, T, ff, W, kind == 2 ? MI355_HYB_ACT_GELU : MI355_HYB_ACT_SILU, dt,
+                                        stream);
+        HCHECK(mi355_hyb_linear(m->gu, 2 * ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, 2 * ff, W, dt, stream));
+        if (kind == 2) return mi355_hyb_gelu_glu(m->act, dt, m->gu, T, ff, stream);
+        if (kind == 6) return mi355_hyb_silu_glu(m->act, dt, m->gu, T, ff, nullptr, 0, stream);
+        return mi355_hyb_clamped_glu(m->act, dt, m->gu, T, ff, WL.c.mlp_limit, WL.c.mlp_alpha, stream);
+    };
     // the experts of a feed-forward without an output norm: routing on the f32 norm output, the pairs grouped, gate/up, silu, down -> moe_y
     auto run_experts = [&](const mi355_hybrid_layer& c, const HLayer& WL) -> int {
         const int E = c.moe_experts, K = c.moe_top, ff = c.mlp_ff, pairs = T * K;
@@ -758,9 +801,7 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
         const int bm = std::min(mi355_hyb_moe_block_rows(pairs, E, 2 * ff, W, dt), mi355_hyb_moe_block_rows(pairs, E, W, ff, dt));
         const int nb = (pairs + bm - 1) / bm + E;
         HCHECK(mi355_hyb_moe_group(m->moe_pos, m->moe_row_token, m->moe_table, m->moe_ids, pairs, K, E, bm, nb, stream));
-        HCHECK(mi355_hyb_linear_grouped(m->moe_gu, 2 * ff, xin, xin_dt, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)2 * ff * W,
-                                        m->moe_table, bm, nb, 2 * ff, W, dt, stream));
-        HCHECK(mi355_hyb_silu_glu(m->moe_act, dt, m->moe_gu, nb * bm, ff, m->moe_table, bm, stream));
+        HCHECK(expert_gate_up(WL, bm, nb));
         return mi355_hyb_linear_grouped(m->moe_y, W, m->moe_act, dt, ff, nullptr, WL.w[MI355_HW_MOE_DOWN].p, (int64_t)W * ff, m->moe_table, bm,
                                         nb, W, ff, dt, stream);
     };
@@ -966,11 +1007,7 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             else if (c.mlp_kind == 4 || c.mlp_kind == 5) {
                 HCHECK(mi355_hyb_linear_act(m->act, dt, c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, c.mlp_ff, W,
                                             c.mlp_kind == 5 ? MI355_HYB_ACT_GELU : MI355_HYB_ACT_RELU2, c.mlp_ff, dt, stream));
-            } else if (c.mlp_kind) {
-                HCHECK(mi355_hyb_linear(m->gu, 2 * c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, 2 * c.mlp_ff, W, dt, stream));
-                if (c.mlp_kind == 2) HCHECK(mi355_hyb_gelu_glu(m->act, dt, m->gu, T, c.mlp_ff, stream));
-                else HCHECK(mi355_hyb_silu_glu(m->act, dt, m->gu, T, c.mlp_ff, nullptr, 0, stream));
-            }
+            } else if (c.mlp_kind) HCHECK(dense_gate_up(WL));
             const bool dense = c.mlp_kind && c.mlp_kind != 3;
             if (dense) HCHECK(mi355_hyb_linear(m->y2, W, m->act, dt, c.mlp_ff, WL.w[MI355_HW_MLP_DOWN].p, nullptr, T, W, c.mlp_ff, dt, stream));
             HCHECK(pair_step((int)li, m->y, dense ? m->y2 : nullptr, c.mlp_kind == 3, c.moe_top));
@@ -1035,9 +1072,7 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
             const int bm = std::min(mi355_hyb_moe_block_rows(pairs, E, 2 * ff, W, dt), mi355_hyb_moe_block_rows(pairs, E, W, ff, dt));
             const int nb = (pairs + bm - 1) / bm + E;
             HCHECK(mi355_hyb_moe_group(m->moe_pos, m->moe_row_token, m->moe_table, m->moe_ids, pairs, K, E, bm, nb, stream));
-            HCHECK(mi355_hyb_linear_grouped(m->moe_gu, 2 * ff, xin, xin_dt, W, m->moe_row_token, WL.w[MI355_HW_MOE_GATE_UP].p, (int64_t)2 * ff * W,
-                                            m->moe_table, bm, nb, 2 * ff, W, dt, stream));
-            HCHECK(mi355_hyb_silu_glu(m->moe_act, dt, m->moe_gu, nb * bm, ff, m->moe_table, bm, stream));
+            HCHECK(expert_gate_up(WL, bm, nb));
             HCHECK(mi355_hyb_linear_grouped(m->moe_y, W, m->moe_act, dt, ff, nullptr, WL.w[MI355_HW_MOE_DOWN].p, (int64_t)W * ff, m->moe_table, bm,
                                             nb, W, ff, dt, stream));
             if (fs) {
@@ -1049,9 +1084,7 @@ static int forward_enqueue(HModel* m, const uint32_t* tokens, const int64_t* pos
                                                   f(MI355_HW_NORM2), T, W, K, eps, stream));
         } else if (c.mlp_kind) {
             if (sandwich) HCHECK(mi355_hyb_pre_norm(m->pre, dt, m->x, f(MI355_HW_PRE_NORM2), T, W, eps, stream));
-            HCHECK(mi355_hyb_linear(m->gu, 2 * c.mlp_ff, xin, xin_dt, W, WL.w[MI355_HW_MLP_GATE_UP].p, nullptr, T, 2 * c.mlp_ff, W, dt, stream));
-            if (c.mlp_kind == 2) HCHECK(mi355_hyb_gelu_glu(m->act, dt, m->gu, T, c.mlp_ff, stream));
-            else HCHECK(mi355_hyb_clamped_glu(m->act, dt, m->gu, T, c.mlp_ff, c.mlp_limit, c.mlp_alpha, stream));
+            HCHECK(dense_gate_up(WL));
             HCHECK(mi355_hyb_linear(m->y, W, m->act, dt, c.mlp_ff, WL.w[MI355_HW_MLP_DOWN].p, nullptr, T, W, c.mlp_ff, dt, stream));
             HCHECK(residual(MI355_HW_NORM2));
         }

@@ -556,6 +556,16 @@ int64_t mi355_hyb_decay_attention_scratch(int32_t num_tokens, int32_t num_seqs, 
 int mi355_hyb_linear_segments(float* out, int32_t ldo, const void* a, int32_t a_dtype, int32_t lda, int64_t a_stride, int32_t first, const void* w,
                               const float* bias, const int32_t* seg_rows, int32_t n_seg, int32_t num_tokens, int32_t n, int32_t k, int32_t dtype,
                               int64_t stream);
+/* gate and up in one product with the activation (MI355_HYB_ACT_SILU or _GELU) behind it: w [2 ff, k] holds 16 gate rows, their 16 up rows, the
+ * next 16 gate rows, ... (mi355_hyb_interleave_gate_up makes that order of [ff gate rows | ff up rows]; ff a multiple of 16); out (dt_out)
+ * [T, ldo] = act(gate) up; a and w are both (dt) */
+int mi355_hyb_linear_glu(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t lda, const void* w, int32_t num_tokens, int32_t ff,
+                         int32_t k, int32_t act, int32_t dtype, int64_t stream);
+/* the same per block of a table (mi355_hyb_linear_grouped) */
+int mi355_hyb_linear_grouped_glu(void* out, int32_t out_dtype, int32_t ldo, const void* a, int32_t lda, const int32_t* row_token, const void* w,
+                                 int64_t w_bs, const int32_t* block_table, int32_t block_rows, int32_t n_blocks, int32_t ff, int32_t k, int32_t act,
+                                 int32_t dtype, int64_t stream);
+int mi355_hyb_interleave_gate_up(void* out, const void* in, int32_t matrices, int32_t ff, int32_t k, int32_t dtype, int64_t stream);
 /* the end of one layer and the start of the next in one launch:
  *   x' = x + (y1 + (y2 or sum_j moe_w[t, j] moe_rows[moe_pos[t top + j]]))     (each part NULL = none) -> x_out (NULL: not written)
  *   h = RMSnorm(x') norm1 -> out1 (dt_out) [T, width];   RMSnorm(x') norm2 -> out2 (dt_out) (and out2_f32, NULL or f32)   (norm2 NULL: neither)

@@ -178,6 +178,66 @@ def test_products_whose_segments_read_different_operands(lib, dtype, T, k, segs,
     _KEEP.clear()
 
 
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("T,ff,k", [(3, 16, 24), (1, 48, 2080), (12, 160, 2048), (20, 80, 40), (50, 112, 33), (130, 144, 64), (200, 64, 96), (65, 16, 32)])
+def test_gate_and_up_in_one_product(lib, dtype, T, ff, k):
+    """interleaved gate and up rows, every product kernel: act(gate) up with silu and gelu, results in f32 or bf16"""
+    _gpu()
+    rng = np.random.default_rng(ff)
+    rnd = f32 if dtype == F32 else D.bf16_round
+    a, w = rnd(rng.standard_normal((T, k + 8))), rnd(rng.standard_normal((2 * ff, k)) * 1.5 / math.sqrt(k))
+    il = empty_dt((2 * ff, k), dtype)
+    ok(lib.mi355_hyb_interleave_gate_up(il.data_ptr(), PD(w, dtype), 1, ff, k, dtype, _st()))
+    order = [h * ff + b * 16 + j for b in range(ff // 16) for h in (0, 1) for j in range(16)]
+    assert np.array_equal(host_dt(il, dtype), w[order])
+    z = a[:, :k] @ w.T
+    gelu = lambda x: 0.5 * x * (1 + np.tanh(math.sqrt(2 / math.pi) * (x + 0.044715 * x ** 3)))     # noqa: E731
+    for act, fn in ((1, D.silu), (2, gelu)):
+        for out_dt in ((F32,) if dtype == F32 else (F32, BF16)):
+            out = empty_dt((T, ff + 3), out_dt)
+            ok(lib.mi355_hyb_linear_glu(out.data_ptr(), out_dt, ff + 3, PD(a, dtype), k + 8, il.data_ptr(), T, ff, k, act, dtype, _st()))
+            want, got = fn(z[:, :ff]) * z[:, ff:], host_dt(out, out_dt)
+            assert np.abs(got[:, :ff] - want).max() < tol(out_dt, 3e-5, 8e-3) * max(1.0, np.abs(want).max()) and (got[:, ff:] == 0).all(), (act, out_dt)
+    assert lib.mi355_hyb_linear_glu(il.data_ptr(), dtype, ff, il.data_ptr(), k, il.data_ptr(), T, ff + 8, k, 1, dtype, _st()) != 0
+    assert lib.mi355_hyb_linear_glu(il.data_ptr(), dtype, ff, il.data_ptr(), k, il.data_ptr(), T, ff, k, 3, dtype, _st()) != 0
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("T,W,E,top,ff", [(5, 64, 6, 2, 32), (70, 64, 4, 3, 96), (300, 96, 3, 2, 64), (1, 32, 9, 9, 16), (40, 40, 7, 2, 24)])
+def test_grouped_gate_up_experts(lib, dtype, T, W, E, top, ff):
+    """grouping, gate and up with silu behind them in one product (ff a multiple of 16; else two launches), the down product and the
+    weighted sum of the rows equal every expert run alone"""
+    _gpu()
+    rng = np.random.default_rng(T + E)
+    h, gu, dn = D.bf16_round(rng.standard_normal((T, W))), D.bf16_round(rng.standard_normal((E, 2 * ff, W)) / math.sqrt(W)), D.bf16_round(rng.standard_normal((E, W, ff)) / math.sqrt(ff))
+    ids = np.stack([rng.permutation(E)[:top] for _ in range(T)])
+    wt = f32(rng.uniform(0.1, 1, (T, top)))
+    want = np.zeros((T, W))
+    for t in range(T):
+        for e, w in zip(ids[t], wt[t]):
+            a = D.silu(gu[e, :ff] @ h[t]) * (gu[e, ff:] @ h[t])
+            want[t] += w * (dn[e] @ (a if dtype == F32 else D.bf16_round(a)))
+    pairs = T * top
+    bm = min(lib.mi355_hyb_moe_block_rows(pairs, E, 2 * ff, W, dtype), lib.mi355_hyb_moe_block_rows(pairs, E, W, ff, dtype))
+    nb = (pairs + bm - 1) // bm + E
+    pos, tokrow, table = (torch.zeros(n, dtype=torch.int32, device="cuda") for n in (pairs, nb * bm, 2 * nb))
+    ok(lib.mi355_hyb_moe_group(pos.data_ptr(), tokrow.data_ptr(), table.data_ptr(), P(ids, np.int32), pairs, top, E, bm, nb, _st()))
+    act, y, hd, gud = empty_dt((nb * bm, ff), dtype), torch.zeros((nb * bm, W), device="cuda"), dev_dt(h, dtype), dev_dt(gu, dtype)
+    if ff % 16 == 0:
+        il = torch.zeros_like(gud)
+        ok(lib.mi355_hyb_interleave_gate_up(il.data_ptr(), gud.data_ptr(), E, ff, W, dtype, _st()))
+        ok(lib.mi355_hyb_linear_grouped_glu(act.data_ptr(), dtype, ff, hd.data_ptr(), W, tokrow.data_ptr(), il.data_ptr(), 2 * ff * W, table.data_ptr(), bm, nb, ff, W, 1,
+                                            dtype, _st()))
+    else:
+        z = torch.zeros((nb * bm, 2 * ff), device="cuda")
+        ok(lib.mi355_hyb_linear_grouped(z.data_ptr(), 2 * ff, hd.data_ptr(), dtype, W, tokrow.data_ptr(), gud.data_ptr(), 2 * ff * W, table.data_ptr(), bm, nb, 2 * ff, W, dtype,
+                                        _st()))
+        ok(lib.mi355_hyb_silu_glu(act.data_ptr(), dtype, z.data_ptr(), nb * bm, ff, table.data_ptr(), bm, _st()))
+    ok(lib.mi355_hyb_linear_grouped(y.data_ptr(), W, act.data_ptr(), dtype, ff, None, PD(dn, dtype), W * ff, table.data_ptr(), bm, nb, W, ff, dtype, _st()))
+    got = (wt[:, :, None] * y.cpu().numpy()[pos.cpu().numpy().reshape(T, top)]).sum(1)
+    assert np.abs(got - want).max() < tol(dtype, 2e-5, 2e-2) * max(1.0, np.abs(want).max())
+
+
 @pytest.mark.parametrize("T,rank,C", [(1, 1, 7), (3, 6, 96), (5, 64, 300), (70, 70, 256), (200, 130, 33), (65, 5, 513)])
 def test_low_rank_decay(lib, T, rank, C):
     _gpu()
@@ -321,7 +381,7 @@ def _edges(L, first, bs, window, keep):
 @pytest.mark.parametrize("H,G,d,vd,bs,L,n_new,window,keep,biased", [
     (4, 2, 16, 16, 16, 300, 1, 128, 0, 1), (4, 2, 16, 24, 16, 257, 1, 40, 6, 0), (6, 3, 12, 5, 8, 290, 7, 50, 0, 1), (3, 3, 20, 20, 8, 90, 40, 1, 0, 1), (3, 3, 20, 20, 8, 90, 40, 1, 3, 0),
     (3, 3, 32, 32, 64, 330, 130, 100, 0, 1), (8, 2, 64, 64, 32, 400, 400, 97, 33, 0), (6, 2, 32, 48, 16, 270, 80, 16, 0, 1), (4, 4, 128, 64, 64, 640, 1, 512, 0, 1),
-    (4, 1, 128, 128, 64, 520, 64, 200, 70, 0), (2, 2, 64, 128, 16, 150, 150, 70, 0, 1), (4, 2, 96, 192, 16, 200, 100, 30, 6, 0), (4, 2, 32, 160, 16, 200, 100, 64, 17, 0),
+    (4, 1, 128, 128, 64, 520, 64, 200, 70, 0), (2, 2, 64, 128, 16, 150, 150, 70, 0, 1), (4, 2, 96, 192, 16, 200, 100, 30, 6, 0), (4, 2, 32, 160, 16, 200, 100, 64, 17, 0), (4, 1, 128, 256, 16, 230, 150, 64, 17, 0),
     (4, 2, 64, 256, 32, 200, 140, 90, 0, 1), (4, 1, 64, 64, 64, 260, 200, 0, 0, 1), (1, 1, 1, 1, 16, 70, 5, 20, 2, 0), (5, 1, 16, 16, 16, 130, 66, 1000, 0, 1)])
 def test_attention_with_keys_that_stand_out(lib, dtype, H, G, d, vd, bs, L, n_new, window, keep, biased):
     """the last n_new tokens of a sequence of L against its scattered pages (the generic kernel, the matrix-core kernels with one wave per
