@@ -92,8 +92,9 @@ __device__ __forceinline__ int lin_row(const LinArgs& p, int t) { return p.row_s
 // n0: the tile's first column
 template <typename TA, int B> __device__ __forceinline__ void lin_batch(LinArgs& p, int n0) {
     if (B == LIN_SEG_BUILD) {
-        int i = 0;
-        while (i + 1 < p.n_seg && n0 >= p.seg_end[i]) ++i;
+        int i = 0;                                                  // (constant indices only: the arguments stay in scalar registers)
+#pragma unroll
+        for (int j = 0; j + 1 < LIN_MAX_SEG; ++j) i += (j + 1 < p.n_seg && n0 >= p.seg_end[j]) ? 1 : 0;
         p.a = static_cast<const TA*>(p.a) + (p.seg0 + i) * p.seg_a;
         return;
     }
@@ -1385,10 +1386,11 @@ template <int DP, int LPC, int CH> __global__ __launch_bounds__(256) void delta_
 }
 
 // out = o / rms(o) * w * gate * out_scale, one wave per (token, head); head h's weights start at w + h w_ld
-template <typename TO> __global__ __launch_bounds__(64) void gated_norm_kernel(TO* out, int ldo, int out_off, const float* o, const float* w,
+template <typename TO> __global__ __launch_bounds__(256) void gated_norm_kernel(TO* out, int ldo, int out_off, const float* o, const float* w,
                                                                               const float* gate_in, int ldg, int gate, int H, int vd, int w_ld,
                                                                               float eps, float out_scale) {
-    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+    const int t = blockIdx.x, h = blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (h >= H) return;
     const float* orow = o + ((size_t)t * H + h) * vd;
     float ss = 0.f;
     for (int i = lane; i < vd; i += 64) ss += orow[i] * orow[i];
@@ -2268,9 +2270,12 @@ int mi355_hyb_gated_norm_heads(void* out, int32_t out_dtype, int32_t ldo, int32_
                                float out_scale, int64_t stream) {
     if (!out || !o || !w || !gate_in || !is_dt(out_dtype) || heads <= 0 || vdim <= 0 || w_ld < 0) return -1;
     if (T <= 0) return 0;
-    const dim3 grid(T, heads);
-    if (out_dtype == MI355_DTYPE_F32) gated_norm_kernel<float><<<grid, 64, 0, to_stream(stream)>>>((float*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, w_ld, eps, out_scale);
-    else gated_norm_kernel<uint16_t><<<grid, 64, 0, to_stream(stream)>>>((uint16_t*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, w_ld, eps, out_scale);
+    const int waves = T <= 64 ? 1 : 4;                                   // heads per workgroup
+    const dim3 grid(T, (heads + waves - 1) / waves);
+    if (out_dtype == MI355_DTYPE_F32)
+        gated_norm_kernel<float><<<grid, 64 * waves, 0, to_stream(stream)>>>((float*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, w_ld, eps, out_scale);
+    else
+        gated_norm_kernel<uint16_t><<<grid, 64 * waves, 0, to_stream(stream)>>>((uint16_t*)out, ldo, out_off, o, w, gate_in, ldg, gate, heads, vdim, w_ld, eps, out_scale);
     LAUNCH_OK(); return 0;
 }
 

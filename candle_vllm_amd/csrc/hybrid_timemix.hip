@@ -127,8 +127,8 @@ template <typename TO, int E> __global__ __launch_bounds__(1024) void pair_step_
 }
 
 // ------------------------------------------------------------------------------------------------------------ low-rank decay
-// log w[t, c] = -exp(sum_r w2t[r, c] tanh(z[t, r]) + w0[c]).  A workgroup of 256 channels and TT tokens; the tanh values of RC ranks at a
-// time sit in LDS, neighbouring threads read neighbouring weights.
+// log w[t, c] = -exp(sum_r w2t[r, c] tanh(z[t, r]) + w0[c]).  Decoding batches: a workgroup of 256 channels and TT tokens; the tanh values
+// of RC ranks at a time sit in LDS, neighbouring threads read neighbouring weights.
 template <int TT> __global__ __launch_bounds__(256) void lowrank_decay_kernel(float* lw, int ldw, const float* z, int ldz, const float* w2t, const float* w0,
                                                                              int T, int R, int C) {
     constexpr int RC = 64;
@@ -168,6 +168,49 @@ template <int TT> __global__ __launch_bounds__(256) void lowrank_decay_kernel(fl
     if (c >= C) return;
 #pragma unroll
     for (int i = 0; i < TT; ++i) if (t0 + i < T) lw[(size_t)(t0 + i) * ldw + c] = -expf(acc[i]);
+}
+
+// prompts: a wave takes 16 tokens and 16 NC channels on the f32 matrix cores, its lanes make their own tanh values (operand layout of a
+// 4-deep step: lane (m16, kg) holds token m16 / channel m16 at depth kg)
+__device__ __forceinline__ f32x4_t mfma_f32(float a, float b, const f32x4_t& c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+template <int NC> __global__ __launch_bounds__(256) void lowrank_decay_tile_kernel(float* lw, int ldw, const float* z, int ldz, const float* w2t, const float* w0,
+                                                                                  int T, int R, int C) {
+    const int lane = threadIdx.x & 63, m16 = lane & 15, kg = lane >> 4;
+    const int c0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 16 * NC, t0 = blockIdx.y * 16;
+    if (c0 >= C) return;
+    const float* zr = z + (size_t)min(t0 + m16, T - 1) * ldz;
+    int ch[NC];
+    f32x4_t acc[NC];
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+        ch[i] = min(c0 + 16 * i + m16, C - 1);
+        const float b = w0[ch[i]];
+        acc[i] = f32x4_t{b, b, b, b};
+    }
+    constexpr int U = 4;                                 // steps whose operands are requested together
+    for (int r0 = 0; r0 < R; r0 += 4 * U) {
+        float a[U], w[U][NC];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int r = r0 + 4 * u + kg, rc = min(r, R - 1);
+            a[u] = r < R ? zr[rc] : 0.f;
+#pragma unroll
+            for (int i = 0; i < NC; ++i) w[u][i] = w2t[(size_t)rc * C + ch[i]];
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const float th = tanhf(a[u]);
+#pragma unroll
+            for (int i = 0; i < NC; ++i) acc[i] = mfma_f32(th, w[u][i], acc[i]);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const int t = t0 + 4 * kg + v;
+            if (t < T && c0 + 16 * i + m16 < C) lw[(size_t)t * ldw + ch[i]] = -expf(acc[i][v]);
+        }
 }
 
 // ------------------------------------------------------------------------------------------------------------ recurrence with a bonus
@@ -282,7 +325,6 @@ struct BonusPieces {
     BonusArgs a;
     float *rd, *kd, *E, *ptot, *D, *U;      // [T, H d] twice, [pieces NSB, H d], [pieces, H d], [T, H, SB], [pieces, H, d, vd]
 };
-__device__ __forceinline__ f32x4_t mfma_f32(float a, float b, const f32x4_t& c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 // piece b of the step -> its first token and its tokens (0: past the last piece)
 __device__ __forceinline__ int piece_of(const BonusArgs& p, int b, int& t0) {
     for (int s = 0; s < p.n_seqs; ++s) {
@@ -294,17 +336,23 @@ __device__ __forceinline__ int piece_of(const BonusArgs& p, int b, int& t0) {
 }
 
 // a wave per sub-piece, 64 channels at a time: a lane first owns a channel (the running products of its decays), then a quarter of the
-// channels of one key (the scores inside the sub-piece)
-__global__ __launch_bounds__(256) void bonus_prepare_kernel(BonusPieces q) {
+// channels of one key (the scores inside the sub-piece).  Every wave has its own part of the LDS; keys and queries pass through the same
+// rows one after the other.
+__device__ __forceinline__ void wave_lds_fence() {
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_sched_barrier(0);
+}
+__global__ __launch_bounds__(256, 4) void bonus_prepare_kernel(BonusPieces q) {
     const BonusArgs& p = q.a;
     constexpr int RS = 68;                                   // floats per staged row: 64 channels + 4 of padding
-    __shared__ __align__(16) float sr[NSB][SB * RS], sk[NSB][SB * RS], sw[NSB][SB * RS];
+    __shared__ __align__(16) float sx[NSB][SB * RS], sw[NSB][SB * RS];
     int t0;
     const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y, d = p.d, C = p.H * d;
     if (n == 0) return;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, key = lane & 15, kg = lane >> 4, first = wave * SB, cnt = min(SB, n - first);
-    float* R = sr[wave];
-    float* K = sk[wave];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);       // (scalar: so are the rows' addresses)
+    const int key = lane & 15, kg = lane >> 4, first = wave * SB, cnt = min(SB, n - first);
+    float* X = sx[wave];
     float* Wd = sw[wave];
     float acc[SB];
 #pragma unroll
@@ -313,51 +361,73 @@ __global__ __launch_bounds__(256) void bonus_prepare_kernel(BonusPieces q) {
         const int ch = c0 + lane;
         const bool on = ch < d;
         float r[SB], k[SB], w[SB];
+        const size_t row0 = (size_t)(t0 + (cnt > 0 ? first : 0));
+        const int cc = on ? ch : c0;
+        const float* rp = p.rkv + row0 * p.ldq + p.r_off + h * d;
+        const float* wp = p.lw + row0 * p.ldw + h * d;
+        const int k_from_r = p.k_off - p.r_off;
+        // (opaque copies: the addresses and comparisons below are made where they are used, not kept in registers across the chunks)
+        int ld_out = C, key_ = key;
+        asm volatile("" : "+s"(ld_out), "+v"(key_));
+#pragma unroll
+        for (int t = 0; t < SB; ++t) {                       // (rows past the portion's end: its last one again)
+            r[t] = rp[cc]; k[t] = (rp + k_from_r)[cc]; w[t] = wp[cc];
+            if (t + 1 < cnt) { rp += p.ldq; wp += p.ldw; }
+        }
 #pragma unroll
         for (int t = 0; t < SB; ++t) {
             const bool ok_ = on && t < cnt;
-            const size_t row = (size_t)(t0 + first + (ok_ ? t : 0));
-            r[t] = ok_ ? p.rkv[row * p.ldq + p.r_off + h * d + ch] : 0.f;
-            k[t] = ok_ ? p.rkv[row * p.ldq + p.k_off + h * d + ch] : 0.f;
-            w[t] = ok_ ? expf(p.lw[row * p.ldw + h * d + ch]) : 1.f;
+            r[t] = ok_ ? r[t] : 0.f; k[t] = ok_ ? k[t] : 0.f; w[t] = ok_ ? expf(w[t]) : 1.f;
         }
-        __syncthreads();                                     // (the chunk of channels before is used up)
+        wave_lds_fence();                                    // (the chunk of channels before is used up)
+#pragma unroll
+        for (int t = 0; t < SB; ++t) { X[t * RS + lane] = k[t]; Wd[t * RS + lane] = w[t]; }
+        wave_lds_fence();
+        float x[16];
+        const int c4 = kg * 16;
+#pragma unroll
+        for (int i = 0; i < 16; i += 4) {
+            const float4 kv = *reinterpret_cast<const float4*>(&X[key * RS + c4 + i]);
+            x[i] = kv.x; x[i + 1] = kv.y; x[i + 2] = kv.z; x[i + 3] = kv.w;
+        }
+        wave_lds_fence();
+        float* rd = q.rd + row0 * C + h * d;
+        float* kd = q.kd + row0 * C + h * d;
         float f = 1.f;
 #pragma unroll
         for (int t = 0; t < SB; ++t) {
-            R[t * RS + lane] = r[t]; K[t * RS + lane] = k[t]; Wd[t * RS + lane] = w[t];
-            if (on && t < cnt) q.rd[(size_t)(t0 + first + t) * C + h * d + ch] = r[t] * f;
+            X[t * RS + lane] = r[t];
+            if (on && t < cnt) (rd + (size_t)t * ld_out)[ch] = r[t] * f;
             f *= w[t];
         }
         if (on) q.E[((size_t)blockIdx.x * NSB + wave) * C + h * d + ch] = f;
         f = 1.f;
 #pragma unroll
         for (int t = SB - 1; t >= 0; --t) {
-            if (on && t < cnt) q.kd[(size_t)(t0 + first + t) * C + h * d + ch] = k[t] * f;
+            if (on && t < cnt) (kd + (size_t)t * ld_out)[ch] = k[t] * f;
             f *= w[t];
         }
-        __syncthreads();
-        float x[16];
-        const int cc = kg * 16;
+        wave_lds_fence();
         float own = 0.f;
 #pragma unroll
         for (int i = 0; i < 16; i += 4) {
-            const float4 kv = *reinterpret_cast<const float4*>(&K[key * RS + cc + i]), rv = *reinterpret_cast<const float4*>(&R[key * RS + cc + i]);
-            x[i] = kv.x; x[i + 1] = kv.y; x[i + 2] = kv.z; x[i + 3] = kv.w;
-            const float* u = p.u + h * d + c0 + cc + i;
-            if (c0 + cc + i < d) own = fmaf(rv.x * u[0], kv.x, fmaf(rv.y * u[1], kv.y, fmaf(rv.z * u[2], kv.z, fmaf(rv.w * u[3], kv.w, own))));
+            const float4 rv = *reinterpret_cast<const float4*>(&X[key * RS + c4 + i]);
+            const float* u = p.u + h * d + c0 + c4 + i;
+            if (c0 + c4 + i < d)
+                own = fmaf(rv.x * u[0], x[i], fmaf(rv.y * u[1], x[i + 1], fmaf(rv.z * u[2], x[i + 2], fmaf(rv.w * u[3], x[i + 3], own))));
         }
 #pragma unroll
         for (int t = 0; t < SB; ++t) {
-            const bool past = key < t;
+            const bool past = key_ < t;
             float dot = 0.f;
 #pragma unroll
             for (int i = 0; i < 16; i += 4) {
-                const float4 rv = *reinterpret_cast<const float4*>(&R[t * RS + cc + i]), wv = *reinterpret_cast<const float4*>(&Wd[t * RS + cc + i]);
+                const float4 rv = *reinterpret_cast<const float4*>(&X[t * RS + c4 + i]), wv = *reinterpret_cast<const float4*>(&Wd[t * RS + c4 + i]);
                 dot = fmaf(rv.x, x[i], fmaf(rv.y, x[i + 1], fmaf(rv.z, x[i + 2], fmaf(rv.w, x[i + 3], dot))));
                 x[i] *= past ? wv.x : 1.f; x[i + 1] *= past ? wv.y : 1.f; x[i + 2] *= past ? wv.z : 1.f; x[i + 3] *= past ? wv.w : 1.f;
             }
-            acc[t] += past ? dot : (key == t ? own : 0.f);
+            acc[t] += past ? dot : (key_ == t ? own : 0.f);
+            if (t & 1) __builtin_amdgcn_sched_barrier(0);        // (rows read further ahead than this only cost registers)
         }
     }
 #pragma unroll
@@ -369,12 +439,14 @@ __global__ __launch_bounds__(256) void bonus_prepare_kernel(BonusPieces q) {
     }
 }
 
-// a wave takes 16 columns of U and walks its rows 16 RT at a time: RT tiles of K'^T against one of V
+// a wave makes 16 columns of RT 16-row tiles of U: tiles of K'^T against one of V, the whole piece's operands requested at once.  Rows past
+// the portion's end read its last row against values of zero; blockIdx.z: 16 RT rows, then 64 columns.
 template <int RT> __global__ __launch_bounds__(256) void bonus_state_kernel(BonusPieces q) {
     const BonusArgs& p = q.a;
     int t0;
     const int n = piece_of(p, blockIdx.x, t0), h = blockIdx.y, d = p.d, C = p.H * d;
     if (n == 0) return;
+    const int row_blocks = (d + 16 * RT - 1) / (16 * RT), r0 = (blockIdx.z % row_blocks) * 16 * RT;
     const float* E = q.E + (size_t)blockIdx.x * NSB * C + h * d;
     if (blockIdx.z == 0)
         for (int i = threadIdx.x; i < d; i += blockDim.x) {
@@ -383,39 +455,44 @@ template <int RT> __global__ __launch_bounds__(256) void bonus_state_kernel(Bonu
             for (int b = 0; b < NSB; ++b) if (b * SB < n) f *= E[(size_t)b * C + i];
             q.ptot[(size_t)blockIdx.x * C + h * d + i] = f;
         }
-    const int lane = threadIdx.x & 63, m16 = lane & 15, kg = lane >> 4, col = (blockIdx.z * 4 + (threadIdx.x >> 6)) * 16 + m16;
+    const int lane = threadIdx.x & 63, m16 = lane & 15, kg = lane >> 4, col = ((blockIdx.z / row_blocks) * 4 + (threadIdx.x >> 6)) * 16 + m16;
     if (col - m16 >= p.vd) return;
     const float* K = q.kd + (size_t)t0 * C + h * d + m16;
     const float* V = p.rkv + (size_t)t0 * p.ldq + p.v_off + h * p.vd + col;
     float* U = q.U + ((size_t)blockIdx.x * p.H + h) * d * p.vd;
-    const int last = (n - 1) / SB;
-    for (int r0 = 0; r0 < d; r0 += 16 * RT) {
-        f32x4_t acc[RT];
-        float f[RT];
+    float a[NSB][4][RT], v[NSB][4], e[NSB][RT];
 #pragma unroll
-        for (int i = 0; i < RT; ++i) { acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f}; f[i] = 1.f; }
-        for (int b = last; b >= 0; --b) {                    // from the piece's end: the factor of a sub-piece is the product of those behind it
+    for (int b = 0; b < NSB; ++b) {
 #pragma unroll
-            for (int tt = 0; tt < SB; tt += 4) {
-                const int t = b * SB + tt + kg;
-                const bool on = t < n;
-                const float v = on ? V[(size_t)t * p.ldq] : 0.f;
-                float a[RT];
+        for (int j = 0; j < 4; ++j) {
+            const int t = b * SB + 4 * j + kg, tc = min(t, n - 1);
+            v[b][j] = V[(size_t)tc * p.ldq];
+            v[b][j] = t < n ? v[b][j] : 0.f;
 #pragma unroll
-                for (int i = 0; i < RT; ++i) a[i] = (on && r0 + 16 * i < d) ? K[(size_t)t * C + r0 + 16 * i] * f[i] : 0.f;
-#pragma unroll
-                for (int i = 0; i < RT; ++i) acc[i] = mfma_f32(a[i], v, acc[i]);
-            }
-            if (b > 0)
-#pragma unroll
-                for (int i = 0; i < RT; ++i) if (r0 + 16 * i < d) f[i] *= E[(size_t)b * C + r0 + 16 * i + m16];
+            for (int i = 0; i < RT; ++i) a[b][j][i] = K[(size_t)tc * C + min(r0 + 16 * i, d - 16)];
         }
 #pragma unroll
-        for (int i = 0; i < RT; ++i)
-            if (r0 + 16 * i < d)
-#pragma unroll
-                for (int v = 0; v < 4; ++v) U[(size_t)(r0 + 16 * i + 4 * kg + v) * p.vd + col] = acc[i][v];
+        for (int i = 0; i < RT; ++i) e[b][i] = b * SB < n ? E[(size_t)b * C + min(r0 + 16 * i, d - 16) + m16] : 1.f;
     }
+    f32x4_t acc[RT];
+    float f[RT];
+#pragma unroll
+    for (int i = 0; i < RT; ++i) { acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f}; f[i] = 1.f; }
+#pragma unroll
+    for (int b = NSB - 1; b >= 0; --b) {                     // from the piece's end: the factor of a sub-piece is the product of those behind it
+        if (b * SB < n)
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int i = 0; i < RT; ++i) acc[i] = mfma_f32(a[b][j][i] * f[i], v[b][j], acc[i]);
+#pragma unroll
+        for (int i = 0; i < RT; ++i) f[i] *= e[b][i];
+    }
+#pragma unroll
+    for (int i = 0; i < RT; ++i)
+        if (r0 + 16 * i < d)
+#pragma unroll
+            for (int x = 0; x < 4; ++x) U[(size_t)(r0 + 16 * i + 4 * kg + x) * p.vd + col] = acc[i][x];
 }
 
 // a thread per element of a (sequence, head)'s state: the states in front of its pieces, then the one behind the last
@@ -450,7 +527,7 @@ __global__ __launch_bounds__(256) void bonus_piece_scan_kernel(BonusPieces q) {
 // a wave takes the 16 queries of one sub-piece and 16 VT columns of the output: its scores against the sub-pieces before it and the ones
 // inside it through LDS into the layout of a left operand, then the two products into one accumulator.  (The depth of a product is walked
 // in the order 16 j + 4 kg + e, e innermost, on both operands: rows are read 16 bytes at a time.)
-template <int VT> __global__ __launch_bounds__(256) void bonus_output_kernel(BonusPieces q) {
+template <int VT> __global__ __launch_bounds__(256, VT <= 4 ? 3 : 2) void bonus_output_kernel(BonusPieces q) {
     const BonusArgs& p = q.a;
     constexpr int PR = LC + 4;
     __shared__ __align__(16) float P[NSB][SB * PR];
@@ -529,7 +606,7 @@ template <int VT> __global__ __launch_bounds__(256) void bonus_output_kernel(Bon
         if (i < wave)
 #pragma unroll
             for (int v = 0; v < 4; ++v) Pw[(4 * kg + v) * PR + SB * i + m16] = sc[i][v];
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); __builtin_amdgcn_wave_barrier();
+    wave_lds_fence();
     for (int j = 0; j <= row0; j += 16) {
         take();
         if (j + 16 <= row0) fetch_values(j + 16);
@@ -598,9 +675,8 @@ int mi355_hyb_lowrank_decay(float* log_w, int32_t ldw, const float* z, int32_t l
     if (!log_w || !z || !w2t || !w0 || rank <= 0 || channels <= 0 || ldw < channels || ldz < rank) return -1;
     if (T <= 0) return 0;
     hipStream_t s_ = to_stream(stream);
-    const unsigned nx = (unsigned)((channels + 255) / 256);
-    if (T <= 64) lowrank_decay_kernel<1><<<dim3(nx, T), 256, 0, s_>>>(log_w, ldw, z, ldz, w2t, w0, T, rank, channels);
-    else lowrank_decay_kernel<16><<<dim3(nx, (T + 15) / 16), 256, 0, s_>>>(log_w, ldw, z, ldz, w2t, w0, T, rank, channels);
+    if (T <= 64) lowrank_decay_kernel<1><<<dim3((unsigned)((channels + 255) / 256), T), 256, 0, s_>>>(log_w, ldw, z, ldz, w2t, w0, T, rank, channels);
+    else lowrank_decay_tile_kernel<8><<<dim3((unsigned)((channels + 511) / 512), (T + 15) / 16), 256, 0, s_>>>(log_w, ldw, z, ldz, w2t, w0, T, rank, channels);
     LAUNCH_OK(); return 0;
 }
 
@@ -630,8 +706,7 @@ int mi355_hyb_bonus_recurrence(float* o, float* state, int64_t state_stride, con
         q.U = q.D + (size_t)num_tokens * heads * SB;
         const dim3 pg((unsigned)np, heads);
         bonus_prepare_kernel<<<pg, 256, 0, s_>>>(q);
-        if (dim <= 64) bonus_state_kernel<4><<<dim3((unsigned)np, heads, (vdim + 63) / 64), 256, 0, s_>>>(q);
-        else bonus_state_kernel<8><<<dim3((unsigned)np, heads, (vdim + 63) / 64), 256, 0, s_>>>(q);
+        bonus_state_kernel<4><<<dim3((unsigned)np, heads, ((dim + 63) / 64) * ((vdim + 63) / 64)), 256, 0, s_>>>(q);
         bonus_piece_scan_kernel<<<dim3(num_seqs, heads, (dim * vdim + 255) / 256), 256, 0, s_>>>(q);
         if (vdim <= 32) bonus_output_kernel<2><<<pg, 256, 0, s_>>>(q);
         else if (vdim <= 64) bonus_output_kernel<4><<<pg, 256, 0, s_>>>(q);

@@ -379,9 +379,9 @@ def _edges(L, first, bs, window, keep):
 
 @pytest.mark.parametrize("dtype", [F32, BF16])
 @pytest.mark.parametrize("H,G,d,vd,bs,L,n_new,window,keep,biased", [
-    (4, 2, 16, 16, 16, 300, 1, 128, 0, 1), (4, 2, 16, 24, 16, 257, 1, 40, 6, 0), (6, 3, 12, 5, 8, 290, 7, 50, 0, 1), (3, 3, 20, 20, 8, 90, 40, 1, 0, 1), (3, 3, 20, 20, 8, 90, 40, 1, 3, 0),
+    (4, 2, 16, 16, 16, 300, 1, 128, 0, 1), (4, 2, 16, 24, 16, 257, 1, 43, 7, 0), (6, 3, 12, 5, 8, 290, 7, 50, 0, 1), (3, 3, 20, 20, 8, 90, 40, 1, 0, 1), (3, 3, 20, 20, 8, 90, 40, 1, 3, 0),
     (3, 3, 32, 32, 64, 330, 130, 100, 0, 1), (8, 2, 64, 64, 32, 400, 400, 97, 33, 0), (6, 2, 32, 48, 16, 270, 80, 16, 0, 1), (4, 4, 128, 64, 64, 640, 1, 512, 0, 1),
-    (4, 1, 128, 128, 64, 520, 64, 200, 70, 0), (2, 2, 64, 128, 16, 150, 150, 70, 0, 1), (4, 2, 96, 192, 16, 200, 100, 30, 6, 0), (4, 2, 32, 160, 16, 200, 100, 64, 17, 0), (4, 1, 128, 256, 16, 230, 150, 64, 17, 0),
+    (4, 1, 128, 128, 64, 520, 64, 200, 70, 0), (2, 2, 64, 128, 16, 150, 150, 70, 0, 1), (6, 3, 96, 192, 16, 200, 100, 30, 9, 0), (4, 2, 32, 160, 16, 200, 100, 64, 17, 0), (4, 1, 128, 256, 16, 230, 150, 64, 17, 0),
     (4, 2, 64, 256, 32, 200, 140, 90, 0, 1), (4, 1, 64, 64, 64, 260, 200, 0, 0, 1), (1, 1, 1, 1, 16, 70, 5, 20, 2, 0), (5, 1, 16, 16, 16, 130, 66, 1000, 0, 1)])
 def test_attention_with_keys_that_stand_out(lib, dtype, H, G, d, vd, bs, L, n_new, window, keep, biased):
     """the last n_new tokens of a sequence of L against its scattered pages (the generic kernel, the matrix-core kernels with one wave per
