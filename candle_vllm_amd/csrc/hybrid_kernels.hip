@@ -568,6 +568,7 @@ struct AttnArgs {
     int chunked;            // the window is a chunk: a query sees the keys from the last multiple of `window` at or below its position on
     int dist_linear;        // the distance bias is r1[h] (query position - key position)
     const float* gate; int ldg;   // != NULL: head h's output times sigmoid(gate[t ldg + h])
+    int bs_log2;            // log2 of the page size (kernels that are only launched for powers of two)
     // the lowest key that a query sees (beside the kept first tokens)
     __device__ __forceinline__ int first_key(int pos) const {
         if (window <= 0) return 0;
@@ -582,6 +583,7 @@ __device__ __forceinline__ float distance_off(const AttnArgs& p, float r1, float
 __device__ __forceinline__ float head_out_scale(const AttnArgs& p, int t, int h) {
     return p.gate ? p.out_scale * sigmoidf_(p.gate[(size_t)t * p.ldg + h]) : p.out_scale;
 }
+constexpr float LOG2E = 1.4426950408889634f;
 __device__ __forceinline__ float cap_score(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
 // 16 bytes of a page row as floats (EPV = 8 bf16 or 4 f32)
 template <typename TC> struct Vec16;
@@ -977,8 +979,15 @@ void window_attention_mfma_kernel(AttnArgs p) {
 // The same prompt-sized step for grouped-query attention: a workgroup of HPG waves takes HPG query heads that share ONE key/value head
 // for the same tile of 16 tokens -- same keys, same mask -- so the 64 key rows and the transposed 64 value rows of a chunk are staged in
 // LDS once per workgroup (cooperatively, the next chunk's rows already in flight in registers) instead of once per head from L2, and
-// the key fragments of S = Q K^T are 16-byte LDS reads.  Softmax, the two probability planes and the products are as above, per wave.
-template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void window_attention_group_kernel(AttnArgs p) {
+// the key fragments of S = Q K^T are 16-byte LDS reads.  Two probability planes and the products are as above, per wave.  The vector
+// work of a chunk is what a wave waits for, so: scores in units of log 2, row maxima by data-parallel moves, row sums kept per lane
+// until the end, masks only in chunks that some query does not see whole, and the columns of P in the order 4 (key mod 16) + key / 16 -- a lane's
+// four probabilities of a query are one 8-byte store; the lanes that bring the value rows take their keys in that order.
+// Workgroups: head groups first (neighbouring workgroups go to different chiplets, so a key/value head stays with one L2 where their
+// number allows it), the tiles with the most keys first.
+// (registers for two waves per SIMD; the few shapes that would not fit without spills keep one)
+constexpr int group_waves(int DK, int VT, int HPG) { return (VT > 8 && !(HPG == 4 || (DK == 3 && HPG == 3))) ? 1 : 2; }
+template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG, group_waves(DK, VT, HPG)) void window_attention_group_kernel(AttnArgs p) {
     constexpr int RS = 72;                                           // bf16 per row of P and V^T: 64 keys + 8 of padding
     constexpr int KRS = DK * 32 + 8;                                 // bf16 per staged key row (16 rows of a fragment read: 16 different bank groups)
     constexpr int NT = 64 * HPG;
@@ -987,7 +996,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
     constexpr int VPT = (VT * 2 + HPG - 1) / HPG;                    // value chunks (8 columns) per wave and stage
     __shared__ __align__(16) uint16_t Ks[64 * KRS], Vt[VT * 16 * RS], Ph[HPG][16 * RS], Pl[HPG][16 * RS];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m16 = lane & 15, kg = lane >> 4;
-    int b = blockIdx.x, s = 0, n_new = 0;
+    int b = (int)(gridDim.y - 1 - blockIdx.y), s = 0, n_new = 0;
     for (; s < p.n_seqs; ++s) {
         n_new = (int)(p.cu_q[s + 1] - p.cu_q[s]);
         const int tiles = (n_new + 15) >> 4;
@@ -997,7 +1006,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
     if (s >= p.n_seqs) return;
     const int t0 = (int)p.cu_q[s] + b * 16, nq = min(16, (int)p.cu_q[s + 1] - t0);
     const int pos0 = (int)p.ctx[s] - n_new + b * 16;
-    const int h = blockIdx.y * HPG + wave, g = h / (p.H / p.G), d = p.d, vd = p.vd;
+    const int h = blockIdx.x * HPG + wave, g = h / (p.H / p.G), d = p.d, vd = p.vd;
     const uint16_t* Q = static_cast<const uint16_t*>(p.q);
     const uint16_t* K = static_cast<const uint16_t*>(p.k_pages);
     const uint16_t* V = static_cast<const uint16_t*>(p.v_pages);
@@ -1009,7 +1018,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
     float mrow[4], lrow[4];
     f32x4_t acc[VT];
 #pragma unroll
-    for (int v = 0; v < 4; ++v) { mrow[v] = -INFINITY; lrow[v] = 0.f; }
+    for (int v = 0; v < 4; ++v) { mrow[v] = -1e30f; lrow[v] = 0.f; }
 #pragma unroll
     for (int c = 0; c < VT; ++c) acc[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     const int hi = pos0 + nq - 1;
@@ -1018,9 +1027,11 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
     int low[4];                                                      // lowest key of this lane's four query rows
 #pragma unroll
     for (int v = 0; v < 4; ++v) low[v] = p.first_key(pos0 + 4 * kg + v);
+    const int top = p.first_key(hi);                                 // keys from here on are in every query's window
     const int nkeep = min(p.keep, lo), n_vis = nkeep + hi - lo + 1;
     auto key_at = [&](int i) { return i < nkeep ? i : (i < n_vis ? lo + (i - nkeep) : hi + 1); };
-    auto page_row = [&](int key) { return (size_t)bt[key / p.bs] * p.bs + (key % p.bs); };
+    auto page_row = [&](int key) { return ((size_t)bt[key >> p.bs_log2] << p.bs_log2) + (key & (p.bs - 1)); };
+    const int vslot = (lane & 3) * 16 + (lane >> 2);                 // the key of a chunk whose value row this lane brings
     uint4 kreg[KPT], vreg[VPT];
     auto fetch = [&](int j0) {
 #pragma unroll
@@ -1029,7 +1040,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
             const int key = ki < 64 ? key_at(j0 + ki) : hi + 1;
             kreg[n] = key <= hi ? *reinterpret_cast<const uint4*>(K + page_row(key) * p.k_ld + g * d + c * 8) : uint4{0, 0, 0, 0};
         }
-        const int vkey = key_at(j0 + lane);
+        const int vkey = key_at(j0 + vslot);
         const uint16_t* vrow = V + (vkey <= hi ? page_row(vkey) : 0) * p.v_ld + g * vd;
 #pragma unroll
         for (int n = 0; n < VPT; ++n) {
@@ -1077,42 +1088,64 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
                 sacc[kt] = mfma_bf16(qf[ks], kf, sacc[kt]);
             }
         }
-        float mx[4], sc[4][4];
+        float sc[4][4], corr[4];
+        const float sl = p.scale * LOG2E;
 #pragma unroll
-        for (int v = 0; v < 4; ++v) {
-            const int r = 4 * kg + v, qpos = pos0 + r;
-            mx[v] = -INFINITY;
+        for (int v = 0; v < 4; ++v)
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt) sc[v][kt] = sacc[kt][v] * sl;
+        if (p.softcap > 0.f)
+#pragma unroll
+            for (int v = 0; v < 4; ++v)
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt) sc[v][kt] = cap_score(sacc[kt][v] * p.scale, p.softcap) * LOG2E;
+        if (p.dist)
 #pragma unroll
             for (int kt = 0; kt < 4; ++kt) {
                 const int key = key_at(j0 + kt * 16 + m16);
-                const bool ok_ = r < nq && key <= qpos && (key >= low[v] || key < p.keep);
-                sc[v][kt] = ok_ ? cap_score(sacc[kt][v] * p.scale, p.softcap) - distance_off(p, r1, r2, qpos - key) : -INFINITY;
-                mx[v] = fmaxf(mx[v], sc[v][kt]);
+#pragma unroll
+                for (int v = 0; v < 4; ++v) sc[v][kt] -= distance_off(p, r1, r2, max(pos0 + 4 * kg + v - key, 0)) * LOG2E;
             }
-#pragma unroll
-            for (int o = 1; o < 16; o <<= 1) mx[v] = fmaxf(mx[v], __shfl_xor(mx[v], o));
-        }
-#pragma unroll
-        for (int v = 0; v < 4; ++v) {
-            const float mn = fmaxf(mrow[v], mx[v]);
-            const float corr = (mn == -INFINITY || mrow[v] == -INFINITY) ? (mn == -INFINITY ? 1.f : 0.f) : expf(mrow[v] - mn);
-            float rs = 0.f;
+        const int chunk_lo = lo + (j0 - nkeep);                      // (whole: no kept key in it, every query sees all 64)
+        if (j0 < nkeep || chunk_lo + 63 > pos0 || chunk_lo < top) {
 #pragma unroll
             for (int kt = 0; kt < 4; ++kt) {
-                const float pv = sc[v][kt] == -INFINITY ? 0.f : expf(sc[v][kt] - mn);
-                rs += pv;
-                const uint16_t hb = f32_to_bf16(pv);
-                ph[(4 * kg + v) * RS + kt * 16 + m16] = hb;
-                pl[(4 * kg + v) * RS + kt * 16 + m16] = f32_to_bf16(pv - bf16_to_f32(hb));
+                const int key = key_at(j0 + kt * 16 + m16);
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const int r = 4 * kg + v;
+                    if (!(r < nq && key <= pos0 + r && (key >= low[v] || key < p.keep))) sc[v][kt] = -INFINITY;
+                }
             }
-#pragma unroll
-            for (int o = 1; o < 16; o <<= 1) rs += __shfl_xor(rs, o);
-            lrow[v] = lrow[v] * corr + rs;
-            mrow[v] = mn;
-#pragma unroll
-            for (int c = 0; c < VT; ++c) acc[c][v] *= corr;
         }
-        __syncthreads();                                             // this wave's probability planes are written
+        bool same = true;
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            float mx = fmaxf(fmaxf(sc[v][0], sc[v][1]), fmaxf(sc[v][2], sc[v][3]));
+            mx = fmaxf(mx, dpp_move<0xB1>(mx));                      // over the 16 lanes of a row
+            mx = fmaxf(mx, dpp_move<0x4E>(mx));
+            mx = fmaxf(mx, dpp_move<0x141>(mx));
+            mx = fmaxf(mx, dpp_move<0x140>(mx));
+            const float mn = fmaxf(mrow[v], mx);                     // (a row that has seen no key yet: -1e30, all its weights are 0)
+            same = same && mn == mrow[v];
+            corr[v] = __builtin_amdgcn_exp2f(mrow[v] - mn);
+            mrow[v] = mn;
+            float pv[4];
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt) pv[kt] = __builtin_amdgcn_exp2f(sc[v][kt] - mn);
+            lrow[v] = fmaf(lrow[v], corr[v], (pv[0] + pv[1]) + (pv[2] + pv[3]));
+            const uint2 hb = uint2{cvt_pk_bf16(pv[0], pv[1]), cvt_pk_bf16(pv[2], pv[3])};
+            *reinterpret_cast<uint2*>(&ph[(4 * kg + v) * RS + 4 * m16]) = hb;
+            *reinterpret_cast<uint2*>(&pl[(4 * kg + v) * RS + 4 * m16]) =
+                uint2{cvt_pk_bf16(pv[0] - bf16lo_to_f32(hb.x), pv[1] - bf16hi_to_f32(hb.x)), cvt_pk_bf16(pv[2] - bf16lo_to_f32(hb.y), pv[3] - bf16hi_to_f32(hb.y))};
+        }
+        if (!__all(same))
+#pragma unroll
+            for (int c = 0; c < VT; ++c)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) acc[c][v] *= corr[v];
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");       // this wave's probability planes are written
+        __builtin_amdgcn_wave_barrier();
 #pragma unroll
         for (int k2 = 0; k2 < 2; ++k2) {
             const uint4 ah = *reinterpret_cast<const uint4*>(&ph[m16 * RS + k2 * 32 + 8 * kg]);
@@ -1125,14 +1158,15 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG) void w
             }
         }
     }
-    const float sink = p.sink ? p.sink[h] : -INFINITY;
+    const float sink = p.sink ? p.sink[h] * LOG2E : -INFINITY;
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
         const int r = 4 * kg + v;
+        const float l = column_sum<16>(lrow[v]);
         if (r >= nq) continue;
         const float M = fmaxf(mrow[v], sink);
-        const float cm = expf(mrow[v] - M);
-        const float L = lrow[v] * cm + (p.sink ? expf(sink - M) : 0.f);
+        const float cm = exp2f(mrow[v] - M);
+        const float L = l * cm + (p.sink ? exp2f(sink - M) : 0.f);
         const float f = cm / L * head_out_scale(p, t0 + r, h);
         const size_t base = (size_t)(t0 + r) * p.ldo + p.out_off + (size_t)h * vd;
 #pragma unroll
@@ -2107,6 +2141,7 @@ int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t ou
     p.chunked = mask_kind == MI355_HYB_MASK_CHUNKED;
     p.dist_linear = dist_linear ? 1 : 0;
     p.gate = gate; p.ldg = ldg;
+    p.bs_log2 = __builtin_ctz((unsigned)block_size);
     if (vec) { int c = 1; while (c < vdim / epv) c <<= 1; p.cp2 = c; c = 1; while (c < dim / epv) c <<= 1; p.cpk = c; }
     else if (vdim > 512) return -1;
     // prompt-sized steps over bf16 pages: the matrix-core kernel (a tile of 16 tokens never spans two sequences)
@@ -2115,8 +2150,9 @@ int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t ou
         const int dk = dim / 32, vt = vdim / 16;
         // grouped-query attention: the query heads of a key/value head share a workgroup and its staged rows
         const int hpk = heads / kv_heads, hpg = cross ? 1 : (hpk % 4 == 0 ? 4 : hpk % 3 == 0 ? 3 : hpk % 2 == 0 ? 2 : 1);
-        if (hpg > 1 && ((dk <= 4 && vt <= 8 && vt % 2 == 0) || (dk == 3 && vt == 12) || (dk == 4 && vt == 16)) && g_attn_group) {
-            const dim3 ggrid((T + 15) / 16 + num_seqs, heads / hpg, 1);
+        if (hpg > 1 && ((dk <= 4 && vt <= 8 && vt % 2 == 0) || (dk == 3 && vt == 12) || (dk == 4 && vt == 16)) && g_attn_group &&
+            (block_size & (block_size - 1)) == 0 && (T + 15) / 16 + num_seqs <= 65535) {
+            const dim3 ggrid(heads / hpg, (T + 15) / 16 + num_seqs, 1);
 #define WG2(DK, VT) do { if (hpg == 4) window_attention_group_kernel<DK, VT, 4><<<ggrid, 256, 0, s_>>>(p); \
                          else if (hpg == 3) window_attention_group_kernel<DK, VT, 3><<<ggrid, 192, 0, s_>>>(p); \
                          else window_attention_group_kernel<DK, VT, 2><<<ggrid, 128, 0, s_>>>(p); } while (0)
