@@ -603,8 +603,8 @@ template <> struct Vec16<float> {
     }
 };
 
-// One workgroup of NW waves per (new token, head).  Wave w takes the 64-key chunks w, w + NW, ... of the token's window: a lane
-// scores one key (q from LDS, the key row from its page), the wave keeps a running maximum / denominator / value sum, and the waves'
+// One workgroup of NW waves per (new token, head).  The waves share the token's visible keys evenly (multiples of 32), 64 at a time: a
+// lane scores one key (q from LDS, the key row from its page), the wave keeps a running maximum / denominator / value sum, and the waves'
 // partial results are merged through LDS.  The sink enters the merge as a partial result with maximum sink, denominator 1 and no
 // value.  VEC (head sizes that are multiples of 16 bytes): rows are read 16 bytes at a time; for the value sum the wave's lanes
 // are (key, 16-byte chunk of the row) pairs -- 64 / cp2 keys per pass -- and the keys' partial sums are added by lane exchanges.
@@ -647,8 +647,9 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
     for (int n = 0; n < NV; ++n)
 #pragma unroll
         for (int e = 0; e < NACC; ++e) acc[n][e] = 0.f;
-    for (int i0 = wave * 64; i0 < n_vis; i0 += NW * 64) {
-        const int cnt = min(64, n_vis - i0);
+    const int share = ((n_vis + NW - 1) / NW + 31) & ~31, end = min(n_vis, (wave + 1) * share);
+    for (int i0 = wave * share; i0 < end; i0 += 64) {
+        const int cnt = min(64, end - i0);
         const int j = lane < cnt ? (i0 + lane < nkeep ? i0 + lane : lo + (i0 + lane - nkeep)) : pos + 1;
         float sc = -INFINITY;
         unsigned page_row = 0;
@@ -671,6 +672,19 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
                     for (int e = 0; e < EPV; ++e) a = fmaf(qv[e], x[e], a);
                     part[u] = on ? a : 0.f;
                 }
+                if (cpk == 16) {
+                    // lane u of a group of 16 keeps pass u's sum, one exchange brings a key's sum to the lane that owns it
+                    float mine = 0.f;
+#pragma unroll
+                    for (int u = 0; u < SU; ++u) {
+                        const float v = column_sum<16>(part[u]);
+                        mine = qchunk == u ? v : mine;
+                    }
+                    const int pass = lane / kq - u0;
+                    const float v = __shfl(mine, (lane % kq) * cpk + (pass & (SU - 1)));
+                    if (pass >= 0 && pass < SU) dot = v;
+                    continue;
+                }
                 for (int o = 1; o < cpk; o <<= 1)
 #pragma unroll
                     for (int u = 0; u < SU; ++u) part[u] += __shfl_xor(part[u], o);
@@ -687,21 +701,21 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
             for (int i = 0; i < p.d; ++i) dot = fmaf(qs[i], ld<TC>(kr, i), dot);
             sc = cap_score(dot * p.scale, p.softcap) - distance_off(p, r1, r2, pos - j);
         }
-        const float mn = fmaxf(m, wave_max(sc));
+        const float mn = fmaxf(m, wave_max_dpp(sc));
         const float pj = (j <= pos) ? expf(sc - mn) : 0.f;
         const float corr = (m == -INFINITY) ? 0.f : expf(m - mn);
-        l = l * corr + wave_sum(pj);
+        l = fmaf(l, corr, pj);                                            // (per lane until the end)
 #pragma unroll
         for (int n = 0; n < NV; ++n)
 #pragma unroll
             for (int e = 0; e < NACC; ++e) acc[n][e] *= corr;
         m = mn;
         if (VEC) {
+            constexpr int PU = NV >= 2 ? 2 : 8;
+            const int vcol = chunk_ok ? chunk * EPV : 0;
             // PU passes of kpp keys at a time: the value rows of all of them are requested before the first is summed, so a chunk
             // costs 64 / (kpp PU) memory round trips instead of 64 / kpp.  A pass beyond the chunk's end (or a lane whose 16-byte
             // chunk lies beyond the row) reads a valid row with weight 0 and its values are replaced by zeros.
-            constexpr int PU = NV >= 2 ? 2 : 8;
-            const int vcol = chunk_ok ? chunk * EPV : 0;
             for (int k0 = 0; k0 < cnt; k0 += kpp * PU) {
                 float pv[PU], x[PU][NV][EPV];
 #pragma unroll
@@ -735,6 +749,7 @@ template <typename TC, int NW, bool VEC, int DQ, int NV> __global__ __launch_bou
             }
         }
     }
+    l = wave_sum_dpp(l);
     if (lane == 0) { pm[wave] = m; pl[wave] = l; }
     if (VEC) {
         for (int off = cp2; off < 64; off <<= 1)
@@ -985,28 +1000,30 @@ void window_attention_mfma_kernel(AttnArgs p) {
 // four probabilities of a query are one 8-byte store; the lanes that bring the value rows take their keys in that order.
 // Workgroups: head groups first (neighbouring workgroups go to different chiplets, so a key/value head stays with one L2 where their
 // number allows it), the tiles with the most keys first.
-// (registers for two waves per SIMD; the few shapes that would not fit without spills keep one)
-constexpr int group_waves(int DK, int VT, int HPG) { return (VT > 8 && !(HPG == 4 || (DK == 3 && HPG == 3))) ? 1 : 2; }
-template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG, group_waves(DK, VT, HPG)) void window_attention_group_kernel(AttnArgs p) {
+// QT: token tiles of 16 per workgroup (2 where few heads share the rows: the rows on their way take half the registers per thread).
+constexpr int group_tiles(int VT, int HPG) { return HPG < 4 ? 2 : 1; }
+template <int DK, int VT, int HPG, int QT> __global__ __launch_bounds__(64 * HPG * QT, 2) void window_attention_group_kernel(AttnArgs p) {
     constexpr int RS = 72;                                           // bf16 per row of P and V^T: 64 keys + 8 of padding
     constexpr int KRS = DK * 32 + 8;                                 // bf16 per staged key row (16 rows of a fragment read: 16 different bank groups)
-    constexpr int NT = 64 * HPG;
+    constexpr int NW = HPG * QT, NT = 64 * NW;
     constexpr int KCH = DK * 4;                                      // 16-byte chunks of a key row
     constexpr int KPT = (64 * KCH + NT - 1) / NT;                    // key chunks per thread and stage
-    constexpr int VPT = (VT * 2 + HPG - 1) / HPG;                    // value chunks (8 columns) per wave and stage
-    __shared__ __align__(16) uint16_t Ks[64 * KRS], Vt[VT * 16 * RS], Ph[HPG][16 * RS], Pl[HPG][16 * RS];
+    constexpr int VPT = (VT * 2 + NW - 1) / NW;                    // value chunks (8 columns) per wave and stage
+    __shared__ __align__(16) uint16_t Ks[64 * KRS], Vt[VT * 16 * RS], Ph[NW][16 * RS], Pl[NW][16 * RS];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m16 = lane & 15, kg = lane >> 4;
     int b = (int)(gridDim.y - 1 - blockIdx.y), s = 0, n_new = 0;
     for (; s < p.n_seqs; ++s) {
         n_new = (int)(p.cu_q[s + 1] - p.cu_q[s]);
-        const int tiles = (n_new + 15) >> 4;
+        const int tiles = (n_new + 16 * QT - 1) / (16 * QT);
         if (b < tiles) break;
         b -= tiles;
     }
     if (s >= p.n_seqs) return;
-    const int t0 = (int)p.cu_q[s] + b * 16, nq = min(16, (int)p.cu_q[s + 1] - t0);
-    const int pos0 = (int)p.ctx[s] - n_new + b * 16;
-    const int h = blockIdx.x * HPG + wave, g = h / (p.H / p.G), d = p.d, vd = p.vd;
+    // the workgroup's tokens, then this wave's 16 of them (none: nq <= 0)
+    const int first = b * 16 * QT, part = QT == 1 ? 0 : 16 * (wave / HPG);
+    const int wg_pos0 = (int)p.ctx[s] - n_new + first, hi = wg_pos0 + min(16 * QT, n_new - first) - 1;
+    const int t0 = (int)p.cu_q[s] + first + part, nq = min(16, n_new - first - part), pos0 = wg_pos0 + part;
+    const int h = blockIdx.x * HPG + (QT == 1 ? wave : wave % HPG), g = h / (p.H / p.G), d = p.d, vd = p.vd;
     const uint16_t* Q = static_cast<const uint16_t*>(p.q);
     const uint16_t* K = static_cast<const uint16_t*>(p.k_pages);
     const uint16_t* V = static_cast<const uint16_t*>(p.v_pages);
@@ -1021,13 +1038,12 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG, group_
     for (int v = 0; v < 4; ++v) { mrow[v] = -1e30f; lrow[v] = 0.f; }
 #pragma unroll
     for (int c = 0; c < VT; ++c) acc[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    const int hi = pos0 + nq - 1;
     const float r1 = p.dist ? p.dist[h] : 0.f, r2 = p.dist ? p.dist[p.H + h] : 0.f;
-    const int lo = p.first_key(pos0);
+    const int lo = p.first_key(wg_pos0);
     int low[4];                                                      // lowest key of this lane's four query rows
 #pragma unroll
     for (int v = 0; v < 4; ++v) low[v] = p.first_key(pos0 + 4 * kg + v);
-    const int top = p.first_key(hi);                                 // keys from here on are in every query's window
+    const int top = p.first_key(pos0 + 15);                           // keys from here on are in every query's window
     const int nkeep = min(p.keep, lo), n_vis = nkeep + hi - lo + 1;
     auto key_at = [&](int i) { return i < nkeep ? i : (i < n_vis ? lo + (i - nkeep) : hi + 1); };
     auto page_row = [&](int key) { return ((size_t)bt[key >> p.bs_log2] << p.bs_log2) + (key & (p.bs - 1)); };
@@ -1044,7 +1060,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG, group_
         const uint16_t* vrow = V + (vkey <= hi ? page_row(vkey) : 0) * p.v_ld + g * vd;
 #pragma unroll
         for (int n = 0; n < VPT; ++n) {
-            const int c8 = wave + n * HPG;
+            const int c8 = wave + n * NW;
             vreg[n] = (vkey <= hi && c8 < VT * 2) ? *reinterpret_cast<const uint4*>(vrow + c8 * 8) : uint4{0, 0, 0, 0};
         }
     };
@@ -1059,7 +1075,7 @@ template <int DK, int VT, int HPG> __global__ __launch_bounds__(64 * HPG, group_
         const int col_odd = lane & 1, key_even = lane & ~1;
 #pragma unroll
         for (int n = 0; n < VPT; ++n) {
-            const int c8 = wave + n * HPG;
+            const int c8 = wave + n * NW;
             if (c8 >= VT * 2) break;
             const uint32_t w[4] = {vreg[n].x, vreg[n].y, vreg[n].z, vreg[n].w};
 #pragma unroll
@@ -2152,16 +2168,16 @@ int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t ou
         const int hpk = heads / kv_heads, hpg = cross ? 1 : (hpk % 4 == 0 ? 4 : hpk % 3 == 0 ? 3 : hpk % 2 == 0 ? 2 : 1);
         if (hpg > 1 && ((dk <= 4 && vt <= 8 && vt % 2 == 0) || (dk == 3 && vt == 12) || (dk == 4 && vt == 16)) && g_attn_group &&
             (block_size & (block_size - 1)) == 0 && (T + 15) / 16 + num_seqs <= 65535) {
-            const dim3 ggrid(heads / hpg, (T + 15) / 16 + num_seqs, 1);
-#define WG2(DK, VT) do { if (hpg == 4) window_attention_group_kernel<DK, VT, 4><<<ggrid, 256, 0, s_>>>(p); \
-                         else if (hpg == 3) window_attention_group_kernel<DK, VT, 3><<<ggrid, 192, 0, s_>>>(p); \
-                         else window_attention_group_kernel<DK, VT, 2><<<ggrid, 128, 0, s_>>>(p); } while (0)
+#define WG1(DK, VT, N) do { constexpr int QT = group_tiles(VT, N); \
+        window_attention_group_kernel<DK, VT, N, QT><<<dim3(heads / N, (T + 16 * QT - 1) / (16 * QT) + num_seqs, 1), 64 * N * QT, 0, s_>>>(p); } while (0)
+#define WG2(DK, VT) do { if (hpg == 4) WG1(DK, VT, 4); else if (hpg == 3) WG1(DK, VT, 3); else WG1(DK, VT, 2); } while (0)
 #define WGV(DK) do { switch (vt) { case 2: WG2(DK, 2); break; case 4: WG2(DK, 4); break; case 6: WG2(DK, 6); break; default: WG2(DK, 8); break; } } while (0)
             if (vt == 12) WG2(3, 12);
             else if (vt == 16) WG2(4, 16);
             else switch (dk) { case 1: WGV(1); break; case 2: WGV(2); break; case 3: WGV(3); break; default: WGV(4); break; }
 #undef WGV
 #undef WG2
+#undef WG1
             LAUNCH_OK(); return 0;
         }
         // cross mode: 2 value heads per block where the head sizes have such a build (dim <= 128, vdim <= 128), the rest of the
