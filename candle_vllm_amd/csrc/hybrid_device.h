@@ -1,4 +1,4 @@
-// Device helpers shared by the translation units of the layer-list host layer (hybrid_kernels.hip, hybrid_blocks.hip): typed loads and
+// Device helpers shared by the translation units of the layer-list host layer (hybrid_kernels.hip, hybrid_blocks.hip, hybrid_streams.hip, hybrid_timemix.hip): typed loads and
 // stores of f32 / bf16 operands, the scalar activations, and the sum over neighbouring lanes that share a state column.
 #pragma once
 #include <hip/hip_runtime.h>

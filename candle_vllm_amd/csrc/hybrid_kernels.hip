@@ -1001,14 +1001,14 @@ void window_attention_mfma_kernel(AttnArgs p) {
 // Workgroups: head groups first (neighbouring workgroups go to different chiplets, so a key/value head stays with one L2 where their
 // number allows it), the tiles with the most keys first.
 // QT: token tiles of 16 per workgroup (2 where few heads share the rows: the rows on their way take half the registers per thread).
-constexpr int group_tiles(int VT, int HPG) { return HPG < 4 ? 2 : 1; }
+constexpr int group_tiles(int HPG) { return HPG < 4 ? 2 : 1; }
 template <int DK, int VT, int HPG, int QT> __global__ __launch_bounds__(64 * HPG * QT, 2) void window_attention_group_kernel(AttnArgs p) {
     constexpr int RS = 72;                                           // bf16 per row of P and V^T: 64 keys + 8 of padding
     constexpr int KRS = DK * 32 + 8;                                 // bf16 per staged key row (16 rows of a fragment read: 16 different bank groups)
     constexpr int NW = HPG * QT, NT = 64 * NW;
     constexpr int KCH = DK * 4;                                      // 16-byte chunks of a key row
     constexpr int KPT = (64 * KCH + NT - 1) / NT;                    // key chunks per thread and stage
-    constexpr int VPT = (VT * 2 + NW - 1) / NW;                    // value chunks (8 columns) per wave and stage
+    constexpr int VPT = (VT * 2 + NW - 1) / NW;                      // value chunks (8 columns) per wave and stage
     __shared__ __align__(16) uint16_t Ks[64 * KRS], Vt[VT * 16 * RS], Ph[NW][16 * RS], Pl[NW][16 * RS];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m16 = lane & 15, kg = lane >> 4;
     int b = (int)(gridDim.y - 1 - blockIdx.y), s = 0, n_new = 0;
@@ -2168,7 +2168,7 @@ int mi355_hyb_attention_ex(void* out, int32_t out_dtype, int32_t ldo, int32_t ou
         const int hpk = heads / kv_heads, hpg = cross ? 1 : (hpk % 4 == 0 ? 4 : hpk % 3 == 0 ? 3 : hpk % 2 == 0 ? 2 : 1);
         if (hpg > 1 && ((dk <= 4 && vt <= 8 && vt % 2 == 0) || (dk == 3 && vt == 12) || (dk == 4 && vt == 16)) && g_attn_group &&
             (block_size & (block_size - 1)) == 0 && (T + 15) / 16 + num_seqs <= 65535) {
-#define WG1(DK, VT, N) do { constexpr int QT = group_tiles(VT, N); \
+#define WG1(DK, VT, N) do { constexpr int QT = group_tiles(N); \
         window_attention_group_kernel<DK, VT, N, QT><<<dim3(heads / N, (T + 16 * QT - 1) / (16 * QT) + num_seqs, 1), 64 * N * QT, 0, s_>>>(p); } while (0)
 #define WG2(DK, VT) do { if (hpg == 4) WG1(DK, VT, 4); else if (hpg == 3) WG1(DK, VT, 3); else WG1(DK, VT, 2); } while (0)
 #define WGV(DK) do { switch (vt) { case 2: WG2(DK, 2); break; case 4: WG2(DK, 4); break; case 6: WG2(DK, 6); break; default: WG2(DK, 8); break; } } while (0)
